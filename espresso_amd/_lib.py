@@ -115,6 +115,14 @@ def _declare_llama(L: C.CDLL) -> None:
     L.esp_llama_read_last_hidden.argtypes = [vp, i32, vp]
     L.esp_llama_read_logits.restype = i32
     L.esp_llama_read_logits.argtypes = [vp, i32, vp]
+    L.esp_llama_append.restype = i32
+    L.esp_llama_append.argtypes = [vp, i32, vp, i32, vp, i32, vp]
+    L.esp_llama_acquire_sequence.restype = i32
+    L.esp_llama_acquire_sequence.argtypes = [vp, C.POINTER(i32)]
+    L.esp_llama_release_sequence.restype = i32
+    L.esp_llama_release_sequence.argtypes = [vp, i32]
+    L.esp_llama_generate_sampled.restype = i32
+    L.esp_llama_generate_sampled.argtypes = [vp, vp, i32, i32, C.c_float, C.c_uint64, vp, C.POINTER(i32), C.POINTER(GenerationStatsStruct)]
     L.esp_llama_generate.restype = i32
     L.esp_llama_generate.argtypes = [vp, vp, i32, i32, vp, C.POINTER(i32), C.POINTER(GenerationStatsStruct), vp]
     L.esp_llama_generate_two_token.restype = i32

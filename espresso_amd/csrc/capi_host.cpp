@@ -8,6 +8,7 @@
 #include "host/gguf.h"
 #include "host/bundle.h"
 #include "host/harness.h"
+#include "host/layered_loader.h"
 #include "host/tokenizer.h"
 
 using namespace esp;
@@ -26,7 +27,8 @@ MultiModelConfig from_c(const ESPModelConfig &c) {
     m.hiddenDim = c.hidden_dim; m.vocab = c.vocab; m.maxSeq = c.max_seq; m.normEps = c.norm_eps; m.ropeTheta = c.rope_theta;
     m.hasEosToken = c.eos_token >= 0;
     m.eosToken = c.eos_token >= 0 ? (TokenID)c.eos_token : 0;
-    m.architecture = c.architecture == 0 ? MultiModelConfig::Architecture::gpt2 : MultiModelConfig::Architecture::llama;
+    m.architecture = c.architecture == 0 ? MultiModelConfig::Architecture::gpt2
+                     : c.architecture == 2 ? MultiModelConfig::Architecture::layered : MultiModelConfig::Architecture::llama;
     return m;
 }
 
@@ -36,7 +38,7 @@ void to_c(const MultiModelConfig &m, ESPModelConfig *c) {
     c->n_layer = m.nLayer; c->n_head = m.nHead; c->n_kv_head = m.nKVHead; c->d_model = m.dModel; c->head_dim = m.headDim;
     c->hidden_dim = m.hiddenDim; c->vocab = m.vocab; c->max_seq = m.maxSeq; c->norm_eps = m.normEps; c->rope_theta = m.ropeTheta;
     c->eos_token = m.hasEosToken ? (int32_t)m.eosToken : -1;
-    c->architecture = m.architecture == MultiModelConfig::Architecture::gpt2 ? 0 : 1;
+    c->architecture = m.architecture == MultiModelConfig::Architecture::gpt2 ? 0 : m.architecture == MultiModelConfig::Architecture::layered ? 2 : 1;
 }
 
 Environment env_from(const char *const *keys, const char *const *values, int count) {
@@ -135,6 +137,25 @@ int esp_model_config_write_metadata(const ESPModelConfig *config, const char *pa
     if (!path || !config) return fail(ESP_ERR_INVALID_ARGUMENT, "null pointer");
     const std::string j = metadataJSON(from_c(*config));
     return writeFile(path, j.data(), j.size()) ? ESP_OK : fail(ESP_ERR_IO, "cannot write %s", path);
+}
+
+int esp_model_config_load_dir(const char *model_dir, int max_seq, ESPModelConfig *out) {
+    if (!model_dir || !out) return fail(ESP_ERR_INVALID_ARGUMENT, "null argument");
+    MultiModelConfig m;
+    if (is_layered_model_dir(model_dir) || !fileExists(joinPath(model_dir, "metadata.json"))) {
+        const int rc = layered_model_config(model_dir, max_seq, &m);
+        if (rc != ESP_OK) return rc;
+    } else {
+        std::string err;
+        if (!loadConfigFromMetadataFile(joinPath(model_dir, "metadata.json"), &m, &err)) return fail(ESP_ERR_INVALID_ARGUMENT, "%s", err.c_str());
+    }
+    to_c(m, out);
+    return ESP_OK;
+}
+
+int esp_layered_architecture_count(void) { return (int)layered_architectures().size(); }
+const char *esp_layered_architecture_at(int index) {
+    return index >= 0 && index < (int)layered_architectures().size() ? layered_architectures()[index].name : nullptr;
 }
 
 int esp_model_registry_count(void) { return (int)ModelRegistry::all().size(); }
@@ -564,9 +585,10 @@ int esp_exact_two_token_harness_generate(const ESPExactTwoTokenModel *model, ESP
     } else {
         if (!target || !draft) return fail(ESP_ERR_INVALID_ARGUMENT, "no model given");
         if (!target->rt->finalized() || !draft->rt->finalized()) return fail(ESP_ERR_INVALID_ARGUMENT, "runtime is not finalized");
-        if (!prompt.empty() && (int)prompt.size() + max_new_tokens + 1 > target->rt->config().max_seq)
-            return fail(ESP_ERR_OUT_OF_RANGE, "prompt %zu + %d new tokens exceed context %d", prompt.size(), max_new_tokens, target->rt->config().max_seq);
-        HipExactTwoTokenModel m(*target->rt, *draft->rt);
+        if (!prompt.empty() && (int)prompt.size() + max_new_tokens + 1 > target->rt->shape().max_seq)
+            return fail(ESP_ERR_OUT_OF_RANGE, "prompt %zu + %d new tokens exceed context %d", prompt.size(), max_new_tokens, target->rt->shape().max_seq);
+        if (!target->rt->as_llama() || !draft->rt->as_llama()) return fail(ESP_ERR_UNSUPPORTED, "the two-token harness needs llama runtimes");
+        HipExactTwoTokenModel m(*target->rt->as_llama(), *draft->rt->as_llama());
         rc = exactTwoTokenHarnessGenerate(m, prompt, max_new_tokens, &trace);
     }
     if (rc != ESP_OK) return rc;

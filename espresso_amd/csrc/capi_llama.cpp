@@ -5,6 +5,12 @@ using namespace esp;
 
 namespace {
 int bad_handle() { return fail(ESP_ERR_INVALID_ARGUMENT, "null runtime handle"); }
+// the llama runtime behind a handle, for the calls that only it has
+int llama_of(const ESPLlamaRuntime *h, LlamaRuntime **out) {
+    if (!h || !h->rt) return bad_handle();
+    *out = h->rt->as_llama();
+    return *out ? ESP_OK : fail(ESP_ERR_UNSUPPORTED, "this call needs a llama runtime");
+}
 void fill_stats(ESPGenerationStats *stats, const GenerationTiming &t, size_t generated) {
     if (!stats) return;
     stats->generated = (int32_t)generated;
@@ -39,9 +45,15 @@ void esp_llama_free(ESPLlamaRuntime *runtime) {
 }
 
 int esp_llama_set_weight(ESPLlamaRuntime *runtime, int layer, int slot, int format, const void *data, size_t bytes) {
-    return runtime ? runtime->rt->set_weight(layer, slot, format, data, bytes) : bad_handle();
+    LlamaRuntime *rt = nullptr;
+    const int rc = llama_of(runtime, &rt);
+    return rc == ESP_OK ? rt->set_weight(layer, slot, format, data, bytes) : rc;
 }
-int esp_llama_finalize(ESPLlamaRuntime *runtime) { return runtime ? runtime->rt->finalize() : bad_handle(); }
+int esp_llama_finalize(ESPLlamaRuntime *runtime) {
+    LlamaRuntime *rt = nullptr;
+    const int rc = llama_of(runtime, &rt);
+    return rc == ESP_OK ? rt->finalize() : rc;
+}
 size_t esp_llama_weight_bytes(const ESPLlamaRuntime *runtime) { return runtime ? runtime->rt->weight_bytes_per_token() : 0; }
 size_t esp_llama_resident_weight_bytes(const ESPLlamaRuntime *runtime) { return runtime ? runtime->rt->resident_weight_bytes() : 0; }
 int esp_llama_reset(ESPLlamaRuntime *runtime) { return runtime ? runtime->rt->reset() : bad_handle(); }
@@ -69,6 +81,28 @@ int esp_llama_read_last_hidden(ESPLlamaRuntime *runtime, int sequence, float *ou
 }
 int esp_llama_read_logits(ESPLlamaRuntime *runtime, int sequence, float *out) {
     return runtime ? runtime->rt->read_logits(sequence, out) : bad_handle();
+}
+
+int esp_llama_append(ESPLlamaRuntime *runtime, int sequence, const uint32_t *tokens, int count, const int *want, int want_count, float *logits) {
+    if (!runtime) return bad_handle();
+    return runtime->rt->append(sequence, tokens, count, want, want_count, logits);
+}
+int esp_llama_acquire_sequence(ESPLlamaRuntime *runtime, int *sequence) { return runtime ? runtime->rt->acquire_sequence(sequence) : bad_handle(); }
+int esp_llama_release_sequence(ESPLlamaRuntime *runtime, int sequence) { return runtime ? runtime->rt->release_sequence(sequence) : bad_handle(); }
+
+int esp_llama_generate_sampled(ESPLlamaRuntime *runtime, const uint32_t *prompt, int prompt_count, int max_tokens, float temperature,
+                               uint64_t seed, uint32_t *out_tokens, int *out_count, ESPGenerationStats *stats) {
+    if (!runtime) return bad_handle();
+    if (!runtime->rt->finalized()) return fail(ESP_ERR_INVALID_ARGUMENT, "runtime is not finalized");
+    if (out_count) *out_count = 0;
+    std::vector<uint32_t> toks;
+    GenerationTiming timing;
+    const int rc = generate_sampled(*runtime->rt, prompt, prompt_count, max_tokens, temperature, seed, &toks, &timing);
+    if (rc != ESP_OK) return rc;
+    for (size_t i = 0; i < toks.size(); i++) if (out_tokens) out_tokens[i] = toks[i];
+    if (out_count) *out_count = (int)toks.size();
+    fill_stats(stats, timing, toks.size());
+    return ESP_OK;
 }
 
 int esp_llama_generate(ESPLlamaRuntime *runtime, const uint32_t *prompt, int prompt_count, int max_tokens,
@@ -99,7 +133,11 @@ int esp_llama_generate_two_token(ESPLlamaRuntime *target, ESPLlamaRuntime *draft
     std::vector<uint32_t> toks;
     GenerationTiming timing;
     TwoTokenStats st;
-    int rc = generate_two_token(*target->rt, *draft->rt, prompt, prompt_count, max_tokens, reference_accounting != 0,
+    LlamaRuntime *full = nullptr, *small = nullptr;
+    int rc = llama_of(target, &full);
+    if (rc == ESP_OK) rc = llama_of(draft, &small);
+    if (rc != ESP_OK) return rc;
+    rc = generate_two_token(*full, *small, prompt, prompt_count, max_tokens, reference_accounting != 0,
                                 &toks, &st, &timing);
     if (rc != ESP_OK) return rc;
     for (size_t i = 0; i < toks.size(); i++) if (out_tokens) out_tokens[i] = toks[i];
@@ -124,8 +162,11 @@ int esp_llama_generate_batch(ESPLlamaRuntime *target, ESPLlamaRuntime *draft_or_
     if (!prompts || !prompt_counts || n_seq < 1 || max_tokens < 0) return fail(ESP_ERR_INVALID_ARGUMENT, "generate_batch: bad argument");
     std::vector<std::vector<uint32_t>> toks;
     TwoTokenStats st;
-    int rc = draft_or_null ? generate_two_token_batch(*target->rt, *draft_or_null->rt, prompts, prompt_counts, n_seq, max_tokens, &toks, &st, decode_ms)
-                           : generate_greedy_batch(*target->rt, prompts, prompt_counts, n_seq, max_tokens, &toks, decode_ms);
+    LlamaRuntime *full = nullptr, *small = nullptr;
+    int rc = ESP_OK;
+    if (draft_or_null && ((rc = llama_of(target, &full)) != ESP_OK || (rc = llama_of(draft_or_null, &small)) != ESP_OK)) return rc;
+    rc = draft_or_null ? generate_two_token_batch(*full, *small, prompts, prompt_counts, n_seq, max_tokens, &toks, &st, decode_ms)
+                       : generate_greedy_batch(*target->rt, prompts, prompt_counts, n_seq, max_tokens, &toks, decode_ms);
     if (rc != ESP_OK) return rc;
     for (int s = 0; s < n_seq; s++) {
         if (out_counts) out_counts[s] = (int)toks[s].size();
@@ -155,19 +196,23 @@ int esp_llama_set_graph_replay(ESPLlamaRuntime *runtime, int enabled) {
 }
 
 int esp_llama_set_merged_attention(ESPLlamaRuntime *runtime, int enabled) {
-    if (!runtime || !runtime->rt) return fail(ESP_ERR_INVALID_ARGUMENT, "set_merged_attention: null runtime");
-    runtime->rt->set_merged_attention(enabled != 0);
-    return runtime->rt->merged_attention_in_use() ? 1 : 0;
+    LlamaRuntime *rt = nullptr;
+    const int rc = llama_of(runtime, &rt);
+    if (rc != ESP_OK) return rc;
+    rt->set_merged_attention(enabled != 0);
+    return rt->merged_attention_in_use() ? 1 : 0;
 }
 
 int esp_llama_set_split_activations(ESPLlamaRuntime *runtime, int enabled) {
-    if (!runtime || !runtime->rt) return fail(ESP_ERR_INVALID_ARGUMENT, "set_split_activations: null runtime");
-    runtime->rt->set_split_activations(enabled != 0);
+    LlamaRuntime *rt = nullptr;
+    const int rc = llama_of(runtime, &rt);
+    if (rc != ESP_OK) return rc;
+    rt->set_split_activations(enabled != 0);
     return ESP_OK;
 }
 
 int esp_llama_set_matrix_prefill(ESPLlamaRuntime *runtime, int enabled) {
-    if (!runtime || !runtime->rt) return fail(ESP_ERR_INVALID_ARGUMENT, "set_matrix_prefill: null runtime");
+    if (!runtime || !runtime->rt) return bad_handle();
     runtime->rt->set_matrix_prefill(enabled != 0);
     return ESP_OK;
 }
@@ -183,24 +228,28 @@ int esp_llama_kernel_times(ESPLlamaRuntime *runtime, double *total_us, int64_t *
     if (!runtime) return bad_handle();
     double t[LlamaRuntime::K_CLASS_COUNT];
     long n[LlamaRuntime::K_CLASS_COUNT];
-    int rc = runtime->rt->collect_kernel_times(t, n, reset != 0);
+    LlamaRuntime *rt = nullptr;
+    int rc = llama_of(runtime, &rt);
+    if (rc == ESP_OK) rc = rt->collect_kernel_times(t, n, LlamaRuntime::K_CLASS_COUNT, reset != 0);
     if (rc != ESP_OK) return rc;
     for (int k = 0; k < LlamaRuntime::K_CLASS_COUNT; k++) {
         if (total_us) total_us[k] = t[k];
         if (launches) launches[k] = n[k];
-        if (bytes_per_launch) bytes_per_launch[k] = runtime->rt->kernel_bytes(k);
+        if (bytes_per_launch) bytes_per_launch[k] = rt->kernel_bytes(k);
     }
     return ESP_OK;
 }
 
 int esp_llama_time_kernel(ESPLlamaRuntime *runtime, int kernel_class, int iters, double *mean_us) {
-    if (!runtime) return bad_handle();
-    return runtime->rt->time_kernel_class(kernel_class, iters, mean_us);
+    LlamaRuntime *rt = nullptr;
+    const int rc = llama_of(runtime, &rt);
+    return rc == ESP_OK ? rt->time_kernel_class(kernel_class, iters, mean_us) : rc;
 }
 
 int esp_llama_time_kernel_dispatch(ESPLlamaRuntime *runtime, int kernel_class, int iters, double *back_to_back_us, double *kernel_us) {
-    if (!runtime) return bad_handle();
-    return runtime->rt->time_kernel_class(kernel_class, iters, back_to_back_us, kernel_us);
+    LlamaRuntime *rt = nullptr;
+    const int rc = llama_of(runtime, &rt);
+    return rc == ESP_OK ? rt->time_kernel_class(kernel_class, iters, back_to_back_us, kernel_us) : rc;
 }
 
 int esp_synth_weights(int format, uint64_t seed, float std_dev, size_t elements, void *out_blocks) {

@@ -139,10 +139,10 @@ int run_two_token_passes_on_device(LlamaRuntime &full, LlamaRuntime &draft, TwoT
 }
 }  // namespace
 
-int generate_greedy(LlamaRuntime &rt, const uint32_t *prompt, int prompt_count, int max_tokens,
+int generate_greedy(DecoderRuntime &rt, const uint32_t *prompt, int prompt_count, int max_tokens,
                     std::vector<uint32_t> *out, GenerationTiming *timing) {
     out->clear();
-    const LlamaConfig &c = rt.config();
+    const DecoderShape &c = rt.shape();
     if (prompt_count <= 0 || !prompt) return fail(ESP_ERR_INVALID_ARGUMENT, "Prompt tokens must not be empty");       // (:6200-6202)
     if (max_tokens < 0) return fail(ESP_ERR_INVALID_ARGUMENT, "maxTokens must be >= 0");                               // (:1411-1413)
     if (prompt_count >= c.max_seq) return fail(ESP_ERR_OUT_OF_RANGE, "prompt of %d tokens does not fit context %d", prompt_count, c.max_seq);
@@ -354,10 +354,10 @@ int sample_token(const float *logits, int count, float temperature, double unit)
     return count - 1;
 }
 
-int generate_sampled(LlamaRuntime &rt, const uint32_t *prompt, int prompt_count, int max_tokens, float temperature,
+int generate_sampled(DecoderRuntime &rt, const uint32_t *prompt, int prompt_count, int max_tokens, float temperature,
                      uint64_t seed, std::vector<uint32_t> *out, GenerationTiming *timing) {
     out->clear();
-    const LlamaConfig &c = rt.config();
+    const DecoderShape &c = rt.shape();
     if (prompt_count <= 0 || !prompt) return fail(ESP_ERR_INVALID_ARGUMENT, "Prompt tokens must not be empty");
     if (max_tokens < 0) return fail(ESP_ERR_INVALID_ARGUMENT, "maxTokens must be >= 0");
     if (prompt_count >= c.max_seq) return fail(ESP_ERR_OUT_OF_RANGE, "prompt of %d tokens does not fit the context", prompt_count);
@@ -392,11 +392,11 @@ int generate_sampled(LlamaRuntime &rt, const uint32_t *prompt, int prompt_count,
 // ---- lock-step batches of independent sequences ---------------------------------------------------
 // Sequence s of `n_seq` uses KV cache s of both runtimes.  Greedy, no EOS handling (the batched configs
 // decode a fixed budget); every sequence produces exactly `eff` tokens.
-static int batch_budget(const LlamaRuntime &a, const LlamaRuntime *b, const int *prompt_counts, int n_seq, int max_tokens, int *eff) {
-    if (n_seq < 1 || n_seq > a.config().max_sequences || (b && n_seq > b->config().max_sequences) || 2 * n_seq > kMaxStepRows)
+static int batch_budget(const DecoderRuntime &a, const DecoderRuntime *b, const int *prompt_counts, int n_seq, int max_tokens, int *eff) {
+    if (n_seq < 1 || n_seq > a.shape().max_sequences || (b && n_seq > b->shape().max_sequences) || 2 * n_seq > kMaxStepRows)
         return fail(ESP_ERR_INVALID_ARGUMENT, "batch of %d sequences does not fit the runtime", n_seq);
-    int max_seq = a.config().max_seq;
-    if (b && b->config().max_seq < max_seq) max_seq = b->config().max_seq;
+    int max_seq = a.shape().max_seq;
+    if (b && b->shape().max_seq < max_seq) max_seq = b->shape().max_seq;
     int budget = max_tokens;
     for (int s = 0; s < n_seq; s++) {
         if (prompt_counts[s] <= 0) return fail(ESP_ERR_INVALID_ARGUMENT, "Prompt tokens must not be empty");
@@ -407,7 +407,7 @@ static int batch_budget(const LlamaRuntime &a, const LlamaRuntime *b, const int 
     return ESP_OK;
 }
 
-int generate_greedy_batch(LlamaRuntime &rt, const uint32_t *const *prompts, const int *prompt_counts, int n_seq, int max_tokens,
+int generate_greedy_batch(DecoderRuntime &rt, const uint32_t *const *prompts, const int *prompt_counts, int n_seq, int max_tokens,
                           std::vector<std::vector<uint32_t>> *out, double *decode_ms) {
     out->assign(n_seq, {});
     int eff = 0, rc = batch_budget(rt, nullptr, prompt_counts, n_seq, max_tokens, &eff);

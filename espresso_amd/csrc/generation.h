@@ -1,5 +1,5 @@
-// Greedy generation loops over LlamaRuntime: the plain incremental loop and the exact two-token
-// draft/verify loop.
+// Generation loops: the plain greedy and sampled loops over any DecoderRuntime, and the exact two-token draft/verify loop over
+// LlamaRuntime (which can take a rejected proposal back).
 #pragma once
 
 #include <cstdint>
@@ -16,7 +16,7 @@ struct GenerationTiming {
 
 // generateIncrementalExactCPULlama at temperature 0 (RealModelInferenceEngine.swift:6192-6431).
 // effectiveMaxTokens = min(maxTokens, maxSeq - promptLen) (:1425-1426).
-int generate_greedy(LlamaRuntime &rt, const uint32_t *prompt, int prompt_count, int max_tokens,
+int generate_greedy(DecoderRuntime &rt, const uint32_t *prompt, int prompt_count, int max_tokens,
                     std::vector<uint32_t> *out, GenerationTiming *timing);
 
 // sampleToken (RealModelInferenceEngine.swift:8036-8068).  `unit` in [0, 1) plays Double.random(in: 0..<total) / total.
@@ -36,7 +36,7 @@ struct SplitMix64 {
 };
 // generate(prompt:maxTokens:temperature:) with temperature > 0 (:1405-1493 with :8070-8081): per token the full
 // logits come back from the GPU and the reference's sampling runs on the host.
-int generate_sampled(LlamaRuntime &rt, const uint32_t *prompt, int prompt_count, int max_tokens, float temperature,
+int generate_sampled(DecoderRuntime &rt, const uint32_t *prompt, int prompt_count, int max_tokens, float temperature,
                      uint64_t seed, std::vector<uint32_t> *out, GenerationTiming *timing);
 
 struct TwoTokenStats {
@@ -57,7 +57,7 @@ int generate_two_token(LlamaRuntime &full, LlamaRuntime &draft, const uint32_t *
 // `n_seq` independent sequences in lock step (sequence s uses KV cache s), greedy, fixed budget: every
 // sequence yields min(max_tokens, context left for the longest prompt) tokens.  Steps of more than two rows
 // run on the matrix cores.  The closest reference notion is lane/stream packing (ane_interop.h:270-289).
-int generate_greedy_batch(LlamaRuntime &rt, const uint32_t *const *prompts, const int *prompt_counts, int n_seq, int max_tokens,
+int generate_greedy_batch(DecoderRuntime &rt, const uint32_t *const *prompts, const int *prompt_counts, int n_seq, int max_tokens,
                           std::vector<std::vector<uint32_t>> *out, double *decode_ms);
 // The exact two-token loop over `n_seq` sequences: each target pass verifies (current, proposed) of every
 // sequence at once.  Every sequence's stream equals its stream from generate_greedy_batch.

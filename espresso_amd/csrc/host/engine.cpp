@@ -6,6 +6,7 @@
 
 #include "../generation.h"
 #include "json_min.h"
+#include "layered_loader.h"
 
 namespace esp {
 namespace {
@@ -101,6 +102,25 @@ int RealModelInferenceEngine::loadRuntime(const MultiModelConfig &config, const 
     return ESP_OK;
 }
 
+int RealModelInferenceEngine::loadLayered(const MultiModelConfig &config, const std::string &modelDir, const Environment &env,
+                                          std::unique_ptr<DecoderRuntime> *out) {
+    LayeredOptions o;
+    o.max_seq = config.maxSeq;
+    o.eos_token = config.hasEosToken ? (int)config.eosToken : -1;
+    auto get = [&](const char *k) { auto it = env.find(k); return it == env.end() ? std::string() : it->second; };
+    const std::string precision = get("ESPRESSO_HIP_PRECISION"), sequences = get("ESPRESSO_HIP_MAX_SEQUENCES");
+    if (!precision.empty() && precision != "bf16" && precision != "f32") return fail(ESP_ERR_INVALID_ARGUMENT, "ESPRESSO_HIP_PRECISION must be bf16 or f32, not %s", precision.c_str());
+    if (precision == "f32") o.precision = Precision::f32;
+    if (!sequences.empty()) o.max_sequences = std::atoi(sequences.c_str());
+    std::unique_ptr<LayeredRuntime> rt;
+    const int rc = load_layered_model(modelDir, o, &rt);
+    if (rc != ESP_OK) return rc;
+    if (rt->shape().vocab != config.vocab || rt->shape().d_model != config.dModel || (int)rt->config().layers.size() != config.nLayer)
+        return fail(ESP_ERR_INVALID_ARGUMENT, "config.json of %s does not match the given configuration", modelDir.c_str());
+    *out = std::move(rt);
+    return ESP_OK;
+}
+
 int RealModelInferenceEngine::build(const MultiModelConfig &config, const std::string &weightDir, const std::string &tokenizerDir,
                                     const Environment &environment, std::unique_ptr<RealModelInferenceEngine> *out) {
     auto t0 = std::chrono::steady_clock::now();
@@ -114,8 +134,14 @@ int RealModelInferenceEngine::build(const MultiModelConfig &config, const std::s
         if (!st.ok()) return fail(ESP_ERR_INVALID_ARGUMENT, "Failed to load tokenizer from %s: error %d (%ld, %ld) %s", tokenizerDir.c_str(),
                                   (int)st.error, st.detail, st.detail2, st.text.c_str());
     }
-    int rc = loadRuntime(config, weightDir, environment, &e->runtime_);
-    if (rc != ESP_OK) return rc;
+    int rc;
+    if (config.architecture == MultiModelConfig::Architecture::layered) {
+        if ((rc = loadLayered(config, weightDir, environment, &e->runtime_)) != ESP_OK) return rc;
+    } else {
+        std::unique_ptr<LlamaRuntime> llama;
+        if ((rc = loadRuntime(config, weightDir, environment, &llama)) != ESP_OK) return rc;
+        e->runtime_ = std::move(llama);
+    }
     e->build_ms_ = std::chrono::duration<double, std::milli>(std::chrono::steady_clock::now() - t0).count();
     *out = std::move(e);
     return ESP_OK;
@@ -186,12 +212,13 @@ int RealModelInferenceEngine::generate(const std::vector<TokenID> &promptTokens,
             return rc;
         out->exactHeadBackend = "hip_gemv_logits_host_sampling";
     } else if (!draftDir.empty()) {
+        if (!runtime_->as_llama()) return fail(ESP_ERR_UNSUPPORTED, "exact two-token draft needs a llama target: recurrent states cannot take a rejected token back");
         if (!draft_runtime_ || draft_dir_loaded_ != draftDir) {
             if ((rc = loadRuntime(draftConfig, draftDir, environment, &draft_runtime_)) != ESP_OK) return rc;
             draft_dir_loaded_ = draftDir;
         }
         TwoTokenStats st;
-        if ((rc = generate_two_token(*runtime_, *draft_runtime_, promptTokens.data(), (int)promptTokens.size(), maxTokens, true,
+        if ((rc = generate_two_token(*runtime_->as_llama(), *draft_runtime_, promptTokens.data(), (int)promptTokens.size(), maxTokens, true,
                                      &out->tokens, &st, &timing)) != ESP_OK)
             return rc;
         out->exactHeadBackend = "hip_exact_two_token_draft";
@@ -203,7 +230,7 @@ int RealModelInferenceEngine::generate(const std::vector<TokenID> &promptTokens,
     } else {
         if ((rc = generate_greedy(*runtime_, promptTokens.data(), (int)promptTokens.size(), maxTokens, &out->tokens, &timing)) != ESP_OK)
             return rc;
-        out->exactHeadBackend = "hip_gemv_argmax";
+        out->exactHeadBackend = runtime_->as_llama() ? "hip_gemv_argmax" : "hip_gemv_logits_argmax";
     }
     out->tokenLatenciesMs = timing.token_latencies_ms;
     out->firstTokenLatencyMs = timing.first_token_latency_ms;

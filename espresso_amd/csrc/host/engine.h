@@ -30,7 +30,9 @@ struct GenerationResult {
 
 class RealModelInferenceEngine {
   public:
-    // Loads the weight directory (packed sidecar, else float32 sidecar, else fp16 BLOBFILE, per tensor) into HBM.
+    // Loads the weight directory into HBM: packed sidecar, else float32 sidecar, else fp16 BLOBFILE per tensor (llama), or
+    // config.json and model.safetensors (architecture layered; ESPRESSO_HIP_PRECISION = bf16 | f32 and
+    // ESPRESSO_HIP_MAX_SEQUENCES in the environment choose the arithmetic and the number of sequence slots).
     // A non-empty tokenizerDir is searched in the reference's order (loadTokenizer, :7558-7613) and must hold a
     // tokenizer; an empty one leaves the engine with the token-id entry points only.
     static int build(const MultiModelConfig &config, const std::string &weightDir, const std::string &tokenizerDir,
@@ -45,7 +47,7 @@ class RealModelInferenceEngine {
     static int generateTokensForTesting(const MultiModelConfig &config, const std::string &weightDir,
                                         const std::vector<TokenID> &promptTokens, int maxTokens, std::vector<TokenID> *out);
     const MultiModelConfig &config() const { return config_; }
-    LlamaRuntime &runtime() { return *runtime_; }
+    DecoderRuntime &runtime() { return *runtime_; }
     double buildTimeMs() const { return build_ms_; }
 
     // resolveExactTwoTokenDraft (:5324-5390): returns 0 and an empty draftWeightDir when no draft is configured
@@ -56,9 +58,11 @@ class RealModelInferenceEngine {
     RealModelInferenceEngine() = default;
     static int loadRuntime(const MultiModelConfig &config, const std::string &weightDir, const Environment &environment,
                            std::unique_ptr<LlamaRuntime> *out);
+    static int loadLayered(const MultiModelConfig &config, const std::string &modelDir, const Environment &environment,
+                           std::unique_ptr<DecoderRuntime> *out);
     MultiModelConfig config_;
     std::string weight_dir_;
-    std::unique_ptr<LlamaRuntime> runtime_;
+    std::unique_ptr<DecoderRuntime> runtime_;
     std::unique_ptr<LlamaRuntime> draft_runtime_;
     std::unique_ptr<Tokenizer> tokenizer_;
     std::string draft_dir_loaded_;

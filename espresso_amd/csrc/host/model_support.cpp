@@ -198,7 +198,7 @@ std::string metadataJSON(const MultiModelConfig &c) {
       << ",\n  \"nKVHead\": " << c.nKVHead << ",\n  \"dModel\": " << c.dModel << ",\n  \"headDim\": " << c.headDim
       << ",\n  \"hiddenDim\": " << c.hiddenDim << ",\n  \"vocab\": " << c.vocab << ",\n  \"maxSeq\": " << c.maxSeq
       << ",\n  \"normEps\": " << c.normEps << ",\n  \"ropeTheta\": " << c.ropeTheta << ",\n  \"architecture\": \""
-      << (c.architecture == MultiModelConfig::Architecture::gpt2 ? "gpt2" : "llama") << "\"";
+      << (c.architecture == MultiModelConfig::Architecture::gpt2 ? "gpt2" : c.architecture == MultiModelConfig::Architecture::layered ? "layered" : "llama") << "\"";
     if (c.hasEosToken) o << ",\n  \"eosToken\": " << c.eosToken;
     o << "\n}\n";
     return o.str();

@@ -14,7 +14,7 @@ using TokenID = uint32_t;  // Sources/ANETypes (TokenID = UInt32)
 
 // Sources/ModelSupport/MultiModelConfig.swift:3-55
 struct MultiModelConfig {
-    enum class Architecture { gpt2, llama };
+    enum class Architecture { gpt2, llama, layered };   // layered: config.json lists the layers (host/layered_config.h)
     std::string name;
     int nLayer = 0, nHead = 0, nKVHead = 0, dModel = 0, headDim = 0, hiddenDim = 0, vocab = 0, maxSeq = 0;
     float normEps = 1e-5f;

@@ -1112,7 +1112,7 @@ __global__ __launch_bounds__(kBlock) void greedy_tail_kernel(GreedyTailArgs a) {
         }
     }
     __syncthreads();
-    embed_row(a.table, a.table_is_f16, feed, a.d, a.hidden, kBlock);
+    if (a.table) embed_row(a.table, a.table_is_f16, feed, a.d, a.hidden, kBlock);   // without a table the trunk fetches its own rows
 }
 
 __global__ void set_ints_kernel(int *dst0, int v0, int *dst1, int v1) {

@@ -1,0 +1,109 @@
+// Embedding, residual stream and RMS norms of the layered models (gfx950).  One workgroup per row; fp32 throughout.
+#include <hip/hip_runtime.h>
+
+#include "gemv_device.h"
+#include "layer_ops.h"
+#include "matrix_ops.h"
+
+namespace esp {
+namespace {
+
+using matrix::Op;
+
+constexpr int kBlock = 256;
+
+__global__ __launch_bounds__(kBlock) void embed_norm_kernel(const uint16_t *table, const int *tokens, const float *weight, float eps, int width, int ld, float *x) {
+    __shared__ float red[4];
+    const int m = blockIdx.x;
+    const uint16_t *row = table + (size_t)tokens[m] * width;
+    float s = 0.0f;
+    for (int i = threadIdx.x; i < width; i += kBlock) { const float v = matrix::bf16_bits_to_float(row[i]); s += v * v; }
+    const float inv = 1.0f / sqrtf(detail::workgroup_sum(s, red) / (float)width + eps);
+    for (int i = threadIdx.x; i < ld; i += kBlock)
+        x[(size_t)m * ld + i] = i < width ? matrix::bf16_bits_to_float(row[i]) * inv * weight[i] : 0.0f;
+}
+
+struct ResidualNormArgs {
+    float *x, *final_x;
+    int width, ld, splits;
+    const float *planes;
+    size_t plane;
+    float mult, eps;
+    const float *norm1, *norm2;
+    void *out1, *out2;
+};
+
+__device__ __forceinline__ void store4(float *p, float4 v) { *reinterpret_cast<float4 *>(p) = v; }
+__device__ __forceinline__ void store4(uint16_t *p, float4 v) { *reinterpret_cast<uint2 *>(p) = make_uint2(matrix::pack_bf16(v.x, v.y), matrix::pack_bf16(v.z, v.w)); }
+
+template <typename T>
+__global__ __launch_bounds__(kBlock) void residual_norm_kernel(ResidualNormArgs a) {
+    __shared__ float red[4];
+    const size_t row = (size_t)blockIdx.x * a.ld;
+    float s = 0.0f;
+    constexpr int kHeld = 8;   // float4 per thread kept in registers: rows up to 8192 wide are read once
+    const int n4 = a.ld / 4;
+    float4 held[kHeld];
+    auto value = [&](int i) {
+        float4 v = reinterpret_cast<const float4 *>(a.x + row)[i];
+        if (a.splits > 0) {
+            float4 t = reinterpret_cast<const float4 *>(a.planes + row)[i];
+            for (int k = 1; k < a.splits; k++) {
+                const float4 u = reinterpret_cast<const float4 *>(a.planes + k * a.plane + row)[i];
+                t.x += u.x; t.y += u.y; t.z += u.z; t.w += u.w;
+            }
+            v.x += a.mult * t.x; v.y += a.mult * t.y; v.z += a.mult * t.z; v.w += a.mult * t.w;
+        }
+        return v;
+    };
+    float *dst = (a.final_x ? a.final_x : a.x) + row;
+#pragma unroll
+    for (int c = 0; c < kHeld; c++) {
+        const int i = threadIdx.x + c * kBlock;
+        if (i < n4) {
+            held[c] = value(i);
+            s += held[c].x * held[c].x + held[c].y * held[c].y + held[c].z * held[c].z + held[c].w * held[c].w;
+            if (a.splits > 0) store4(dst + 4 * i, held[c]);
+        }
+    }
+    for (int i = threadIdx.x + kHeld * kBlock; i < n4; i += kBlock) {   // wider rows: the rest is read back for the norms
+        const float4 v = value(i);
+        s += v.x * v.x + v.y * v.y + v.z * v.z + v.w * v.w;
+        if (a.splits > 0) store4(dst + 4 * i, v);
+    }
+    if (!a.norm1) return;
+    const float inv = 1.0f / sqrtf(detail::workgroup_sum(s, red) / (float)a.width + a.eps);
+    auto emit = [&](int i, const float4 &v) {
+        const float4 g = reinterpret_cast<const float4 *>(a.norm1)[i];
+        store4(static_cast<T *>(a.out1) + row + 4 * i, make_float4(v.x * inv * g.x, v.y * inv * g.y, v.z * inv * g.z, v.w * inv * g.w));
+        if (a.norm2) {
+            const float4 h = reinterpret_cast<const float4 *>(a.norm2)[i];
+            store4(static_cast<T *>(a.out2) + row + 4 * i, make_float4(v.x * inv * h.x, v.y * inv * h.y, v.z * inv * h.z, v.w * inv * h.w));
+        }
+    };
+#pragma unroll
+    for (int c = 0; c < kHeld; c++) {
+        const int i = threadIdx.x + c * kBlock;
+        if (i < n4) emit(i, held[c]);
+    }
+    for (int i = threadIdx.x + kHeld * kBlock; i < n4; i += kBlock) emit(i, reinterpret_cast<const float4 *>(dst)[i]);
+}
+
+}  // namespace
+
+hipError_t launch_embed_norm(const uint16_t *table, const int *tokens, const float *weight, float eps, int rows, int width, int ld, float *x, hipStream_t s) {
+    if (!table || rows < 1 || width < 1 || ld < width) return hipErrorInvalidValue;
+    hipLaunchKernelGGL(embed_norm_kernel, dim3(rows), dim3(kBlock), 0, s, table, tokens, weight, eps, width, ld, x);
+    return hipGetLastError();
+}
+
+hipError_t launch_residual_norm(const ResidualNorm &p, Precision type, hipStream_t s) {
+    if (!p.x || p.rows < 1 || p.ld % 64 || p.width > p.ld || (p.splits > 0 && !p.planes) || (p.norm1 && !p.out1) || (p.norm2 && !p.out2)) return hipErrorInvalidValue;
+    if (p.splits == 0 && p.final_x) return hipErrorInvalidValue;
+    ResidualNormArgs a{p.x, p.final_x, p.width, p.ld, p.splits, p.planes, p.plane, p.mult, p.eps, p.norm1, p.norm2, p.out1, p.out2};
+    if (type == Precision::bf16) hipLaunchKernelGGL((residual_norm_kernel<uint16_t>), dim3(p.rows), dim3(kBlock), 0, s, a);
+    else hipLaunchKernelGGL((residual_norm_kernel<float>), dim3(p.rows), dim3(kBlock), 0, s, a);
+    return hipGetLastError();
+}
+
+}  // namespace esp

@@ -1,6 +1,5 @@
 #include "llama_runtime.h"
 
-#include <atomic>
 #include <cmath>
 #include <cstdlib>
 #include <cstring>
@@ -25,12 +24,6 @@ float half_to_float_host(uint16_t h) {
     return out;
 }
 
-template <typename T>
-void free_device(T *&p) {
-    if (p) (void)hipFree(p);
-    p = nullptr;
-}
-
 }  // namespace
 
 int LlamaRuntime::create(const LlamaConfig &c, LlamaRuntime **out) {
@@ -48,12 +41,9 @@ int LlamaRuntime::create(const LlamaConfig &c, LlamaRuntime **out) {
         return fail(ESP_ERR_INVALID_ARGUMENT, "llama config: max_sequences must be 1..%d", kMaxStepRows);
     int rc = ensure_init();
     if (rc != ESP_OK) return rc;
-    static std::atomic<unsigned long long> next_id{1};
     LlamaRuntime *rt = new LlamaRuntime();
-    rt->id_ = next_id.fetch_add(1);
     rt->c_ = c;
     rt->h_layers_.resize(c.n_layer);
-    rt->visible_.assign(c.max_sequences, 0);
     *out = rt;
     return ESP_OK;
 }
@@ -68,64 +58,12 @@ LlamaRuntime::~LlamaRuntime() {
         free_device(L.k_cache); free_device(L.v_cache);
     }
     free_device(rope_cos_); free_device(rope_sin_);
-    free_device(hidden_); free_device(qkv_); free_device(q_); free_device(gu_); free_device(logits_);
-    free_device(last_hidden_); free_device(xn_); free_device(ctx_); free_device(act_);
+    free_device(qkv_); free_device(q_); free_device(gu_);
+    free_device(xn_); free_device(ctx_); free_device(act_);
     free_device(xn_lo_); free_device(ctx_lo_); free_device(act_lo_); free_device(xn_sums_); free_device(ctx_sums_); free_device(act_sums_);
-    free_device(d_tokens_); free_device(d_pos_); free_device(d_seq_); free_device(d_out_tokens_);
-    free_device(d_visible_); free_device(d_log_); free_device(d_log_count_);
     free_device(attn_scratch_);
     free_device(gemm_workspace_);
-    free_device(argmax_scratch_.part_value); free_device(argmax_scratch_.part_index);
-    for (hipGraphExec_t g : step_graphs_) if (g) (void)hipGraphExecDestroy(g);
-    for (hipGraphExec_t g : multi_graphs_) if (g) (void)hipGraphExecDestroy(g);
     release_loop_session();
-    for (TimedLaunch &t : timed_) { (void)hipEventDestroy(t.start); (void)hipEventDestroy(t.stop); }
-    for (hipEvent_t e : event_pool_) (void)hipEventDestroy(e);
-}
-
-hipEvent_t LlamaRuntime::take_event() {
-    if (!event_pool_.empty()) {
-        hipEvent_t e = event_pool_.back();
-        event_pool_.pop_back();
-        return e;
-    }
-    hipEvent_t e = nullptr;
-    if (hipEventCreate(&e) != hipSuccess) return nullptr;
-    return e;
-}
-
-int LlamaRuntime::time_begin(int kernel_class) {
-    if (!timing_enabled_) return ESP_OK;
-    TimedLaunch t{kernel_class, take_event(), take_event()};
-    if (!t.start || !t.stop) return fail(ESP_ERR_OUT_OF_MEMORY, "hipEventCreate failed");
-    ESP_HIP_TRY(hipEventRecord(t.start, context().stream));
-    timed_.push_back(t);
-    return ESP_OK;
-}
-
-int LlamaRuntime::time_end() {
-    if (!timing_enabled_) return ESP_OK;
-    ESP_HIP_TRY(hipEventRecord(timed_.back().stop, context().stream));
-    return ESP_OK;
-}
-
-int LlamaRuntime::collect_kernel_times(double total_us[K_CLASS_COUNT], long launches[K_CLASS_COUNT], bool reset) {
-    ESP_HIP_TRY(hipStreamSynchronize(context().stream));
-    for (TimedLaunch &t : timed_) {
-        float ms = 0.0f;
-        ESP_HIP_TRY(hipEventElapsedTime(&ms, t.start, t.stop));
-        time_total_us_[t.kernel_class] += (double)ms * 1e3;
-        time_launches_[t.kernel_class] += 1;
-        event_pool_.push_back(t.start);
-        event_pool_.push_back(t.stop);
-    }
-    timed_.clear();
-    for (int k = 0; k < K_CLASS_COUNT; k++) {
-        if (total_us) total_us[k] = time_total_us_[k];
-        if (launches) launches[k] = time_launches_[k];
-        if (reset) { time_total_us_[k] = 0; time_launches_[k] = 0; }
-    }
-    return ESP_OK;
 }
 
 // Launches the GEMV of one class for every layer in turn (the head: the same matrix), `iters` rounds, between
@@ -390,13 +328,11 @@ int LlamaRuntime::finalize() {
         ESP_HIP_TRY(hipMemcpy(rope_sin_, sn.data(), sn.size() * 4, hipMemcpyHostToDevice));
     }
     // ---- activations ----
-    const size_t R = kPrefillBlockRows > kMaxStepRows ? kPrefillBlockRows : kMaxStepRows, RS = kMaxStepRows;
-    if ((rc = device_alloc(&hidden_, R * d)) != ESP_OK) return rc;
+    const size_t R = kPrefillBlockRows > kMaxStepRows ? kPrefillBlockRows : kMaxStepRows;
+    if ((rc = allocate_common((int)R, d)) != ESP_OK) return rc;
     if ((rc = device_alloc(&qkv_, R * (ad + 2 * kd))) != ESP_OK) return rc;
     if ((rc = device_alloc(&q_, R * ad)) != ESP_OK) return rc;
     if ((rc = device_alloc(&gu_, R * 2 * hd)) != ESP_OK) return rc;
-    if ((rc = device_alloc(&logits_, RS * c_.vocab)) != ESP_OK) return rc;
-    if ((rc = device_alloc(&last_hidden_, (size_t)c_.max_sequences * d)) != ESP_OK) return rc;
     if ((rc = device_alloc(&xn_, R * (size_t)(d > hd ? d : hd))) != ESP_OK) return rc;
     if ((rc = device_alloc(&ctx_, R * ad)) != ESP_OK) return rc;
     if ((rc = device_alloc(&act_, R * hd)) != ESP_OK) return rc;
@@ -408,20 +344,6 @@ int LlamaRuntime::finalize() {
         if ((rc = device_alloc(&ctx_sums_, R * (size_t)(ad / 16))) != ESP_OK) return rc;
         if ((rc = device_alloc(&act_sums_, R * (size_t)(hd / 16))) != ESP_OK) return rc;
     }
-    if ((rc = device_alloc(&d_tokens_, R)) != ESP_OK) return rc;
-    if ((rc = device_alloc(&d_pos_, R)) != ESP_OK) return rc;
-    if ((rc = device_alloc(&d_seq_, R)) != ESP_OK) return rc;
-    if ((rc = device_alloc(&d_out_tokens_, R)) != ESP_OK) return rc;
-    if ((rc = device_alloc(&d_visible_, (size_t)c_.max_sequences)) != ESP_OK) return rc;
-    if ((rc = device_alloc(&d_log_, (size_t)c_.max_seq)) != ESP_OK) return rc;
-    if ((rc = device_alloc(&d_log_count_, 3)) != ESP_OK) return rc;   // tokens logged, stopped, stop enabled (greedy_tail_kernel)
-    step_graphs_.assign(c_.max_sequences, nullptr);
-    multi_graphs_.assign(c_.max_sequences, nullptr);
-    // one (value, index) pair per workgroup of the head GEMV and row: a workgroup owns eight rows, or the grid is persistent
-    head_partial_capacity_ = (c_.vocab + 7) / 8 > 4096 ? (c_.vocab + 7) / 8 : 4096;
-    const size_t argmax_slots = (size_t)2 * head_partial_capacity_ > (size_t)kArgmaxScratchSlots ? (size_t)2 * head_partial_capacity_ : (size_t)kArgmaxScratchSlots;
-    if ((rc = device_alloc(&argmax_scratch_.part_value, argmax_slots)) != ESP_OK) return rc;
-    if ((rc = device_alloc(&argmax_scratch_.part_index, argmax_slots)) != ESP_OK) return rc;
     {
         const size_t per_row = (size_t)c_.n_kv_head * kAttentionMaxSplits * (c_.n_head / c_.n_kv_head) * (c_.head_dim + 2);
         if ((rc = device_alloc(&attn_scratch_, R * per_row)) != ESP_OK) return rc;
@@ -439,54 +361,22 @@ int LlamaRuntime::finalize() {
         const char *sa = getenv("ESPRESSO_HIP_SPLIT_ACTIVATIONS");   // "0": activations rounded to fp16 once
         if (sa && sa[0] == '0') split_activations_ = false;
     }
-    finalized_ = true;
-    return reset();
+    return finish_finalize();
 }
 
-int LlamaRuntime::reset() {
-    if (!finalized_) return fail(ESP_ERR_INVALID_ARGUMENT, "runtime is not finalized");
-    Context &ctx = context();
+int LlamaRuntime::clear_state() {
     const size_t cache_bytes = (size_t)c_.max_sequences * c_.kv_dim() * c_.max_seq * (c_.kv_format == FMT_F16 ? 2 : 4);
     for (Layer &L : layers_) {
-        ESP_HIP_TRY(hipMemsetAsync(L.k_cache, 0, cache_bytes, ctx.stream));
-        ESP_HIP_TRY(hipMemsetAsync(L.v_cache, 0, cache_bytes, ctx.stream));
+        ESP_HIP_TRY(hipMemsetAsync(L.k_cache, 0, cache_bytes, context().stream));
+        ESP_HIP_TRY(hipMemsetAsync(L.v_cache, 0, cache_bytes, context().stream));
     }
-    ESP_HIP_TRY(hipMemsetAsync(last_hidden_, 0, (size_t)c_.max_sequences * c_.d_model * 4, ctx.stream));
-    ESP_HIP_TRY(hipStreamSynchronize(ctx.stream));
-    std::fill(visible_.begin(), visible_.end(), 0);
     return ESP_OK;
-}
-
-int LlamaRuntime::visible(int seq) const {
-    return seq >= 0 && seq < c_.max_sequences ? visible_[seq] : -1;
-}
-
-int LlamaRuntime::set_visible(int seq, int count) {
-    if (seq < 0 || seq >= c_.max_sequences || count < 0 || count > c_.max_seq)
-        return fail(ESP_ERR_OUT_OF_RANGE, "set_visible(seq %d, count %d) out of range", seq, count);
-    visible_[seq] = count;
-    return ESP_OK;
-}
-
-int LlamaRuntime::forward_rows(const StepRows &rows) {
-    if (!finalized_) return fail(ESP_ERR_INVALID_ARGUMENT, "runtime is not finalized");
-    if (rows.count < 1 || rows.count > kMaxStepRows) return fail(ESP_ERR_INVALID_ARGUMENT, "forward_rows: %d rows", rows.count);
-    for (int i = 0; i < rows.count; i++) {
-        if (rows.token[i] < 0 || rows.token[i] >= c_.vocab)
-            return fail(ESP_ERR_OUT_OF_RANGE, "token %d is outside vocab %d", rows.token[i], c_.vocab);   // (:687-689)
-        if (rows.pos[i] < 0 || rows.pos[i] >= c_.max_seq)
-            return fail(ESP_ERR_OUT_OF_RANGE, "position %d exceeds context %d", rows.pos[i], c_.max_seq);  // (:673-677)
-        if (rows.seq[i] < 0 || rows.seq[i] >= c_.max_sequences)
-            return fail(ESP_ERR_OUT_OF_RANGE, "sequence %d of %d", rows.seq[i], c_.max_sequences);
-    }
-    ESP_HIP_TRY(launch_set_rows(rows, d_tokens_, d_pos_, d_seq_, context().stream));
-    return enqueue_trunk(rows.count);
 }
 
 // The trunk over `M` rows whose (token, position, sequence) already sit in d_tokens_/d_pos_/d_seq_.
 int LlamaRuntime::enqueue_trunk(int M, bool embedded, float *final_out) {
     hipStream_t s = context().stream;
-    const int d = c_.d_model, ad = c_.attention_dim(), kd = c_.kv_dim(), hd = c_.hidden_dim;
+    const int d = c_.d_model, ad = c_.attention_dim(), kd = c_.kv_dim();
     const bool kv16 = c_.kv_format == FMT_F16;
     int rc = ESP_OK;
     if (!embedded) ESP_HIP_TRY(launch_embed(embedding_, embedding_f16_, d_tokens_, M, d, hidden_, s));
@@ -566,20 +456,6 @@ int LlamaRuntime::enqueue_trunk(int M, bool embedded, float *final_out) {
     return ESP_OK;
 }
 
-void LlamaRuntime::drop_captured_graphs() {
-    for (auto &g : step_graphs_) if (g) { (void)hipGraphExecDestroy(g); g = nullptr; }
-    for (auto &g : multi_graphs_) if (g) { (void)hipGraphExecDestroy(g); g = nullptr; }
-    graph_epoch_++;
-}
-
-// esp_set_tuning changes which kernels launch_gemv picks: graphs captured before it would keep replaying the old ones.
-void LlamaRuntime::sync_tuning() {
-    const unsigned e = gemv_tuning_epoch();
-    if (e == tuning_epoch_) return;
-    tuning_epoch_ = e;
-    drop_captured_graphs();
-}
-
 void LlamaRuntime::set_split_activations(bool enabled) {
     if (enabled == split_activations_) return;
     split_activations_ = enabled;
@@ -601,55 +477,6 @@ void LlamaRuntime::release_loop_session() {
     ss = DeviceLoopSession{};
 }
 
-int LlamaRuntime::keep_row(int row, int seq) {
-    if (row < 0 || row >= kPrefillBlockRows || seq < 0 || seq >= c_.max_sequences)
-        return fail(ESP_ERR_OUT_OF_RANGE, "keep_row(%d, %d)", row, seq);
-    ESP_HIP_TRY(launch_copy_rows(hidden_ + (size_t)row * c_.d_model, last_hidden_ + (size_t)seq * c_.d_model, 1, c_.d_model,
-                                 context().stream));
-    return ESP_OK;
-}
-
-int LlamaRuntime::advance(int seq, uint32_t token) {
-    if (seq < 0 || seq >= c_.max_sequences) return fail(ESP_ERR_OUT_OF_RANGE, "sequence %d of %d", seq, c_.max_sequences);
-    if (visible_[seq] >= c_.max_seq)
-        return fail(ESP_ERR_OUT_OF_RANGE, "runtime position %d exceeds context %d", visible_[seq], c_.max_seq);
-    if (token >= (uint32_t)c_.vocab) return fail(ESP_ERR_OUT_OF_RANGE, "token %u is outside vocab %d", token, c_.vocab);
-    StepRows rows{};
-    rows.count = 1; rows.token[0] = (int)token; rows.pos[0] = visible_[seq]; rows.seq[0] = seq;
-    int rc = forward_rows(rows);
-    if (rc != ESP_OK) return rc;
-    if ((rc = keep_row(0, seq)) != ESP_OK) return rc;
-    visible_[seq] += 1;
-    return ESP_OK;
-}
-
-int LlamaRuntime::prefill(int seq, const uint32_t *tokens, int count) {
-    if (count <= 0 || !tokens) return fail(ESP_ERR_INVALID_ARGUMENT, "Prompt tokens must not be empty");
-    if (seq < 0 || seq >= c_.max_sequences) return fail(ESP_ERR_OUT_OF_RANGE, "sequence %d of %d", seq, c_.max_sequences);
-    visible_[seq] = 0;
-    if (matrix_prefill_ && count >= kMatrixPrefillMinTokens && matrix_prefill_supported()) {
-        // long prompts: blocks of rows through the MFMA kernels (one pass over the weights per block)
-        if (count > c_.max_seq) return fail(ESP_ERR_OUT_OF_RANGE, "runtime position %d exceeds context %d", c_.max_seq, c_.max_seq);
-        for (int i = 0; i < count; i++)
-            if (tokens[i] >= (uint32_t)c_.vocab) return fail(ESP_ERR_OUT_OF_RANGE, "token %u is outside vocab %d", tokens[i], c_.vocab);
-        int rc = ESP_OK;
-        for (int base = 0; base < count && rc == ESP_OK; base += kPrefillBlockRows) {
-            const int rows = count - base < kPrefillBlockRows ? count - base : kPrefillBlockRows;
-            rc = prefill_block(seq, tokens + base, rows, base);
-            if (rc == ESP_OK && base + rows == count) rc = keep_row(rows - 1, seq);
-        }
-        if (rc != ESP_OK) return rc;
-        ESP_HIP_TRY(hipStreamSynchronize(context().stream));
-        visible_[seq] = count;
-        return ESP_OK;
-    }
-    for (int i = 0; i < count; i++) {
-        int rc = advance(seq, tokens[i]);
-        if (rc != ESP_OK) return rc;
-    }
-    return ESP_OK;
-}
-
 bool LlamaRuntime::matrix_prefill_supported() const {
     auto ok = [](const DeviceMatrix &m) { return m.format != FMT_F32 && m.cols % 64 == 0; };
     for (const Layer &L : layers_)
@@ -661,17 +488,9 @@ bool LlamaRuntime::matrix_prefill_supported() const {
 // a block of rows, every projection as one dequant-fused MFMA GEMM.  Rows of the block see each other's
 // keys and values causally because the whole block's K/V is written before its attention runs.
 int LlamaRuntime::prefill_block(int seq, const uint32_t *tokens, int rows, int base) {
-    hipStream_t s = context().stream;
-    const int d = c_.d_model, ad = c_.attention_dim(), kd = c_.kv_dim(), hd = c_.hidden_dim;
-    const bool kv16 = c_.kv_format == FMT_F16;
-    std::vector<int> h_tok(rows), h_pos(rows), h_seq(rows, seq);
-    for (int i = 0; i < rows; i++) { h_tok[i] = (int)tokens[i]; h_pos[i] = base + i; }
-    ESP_HIP_TRY(hipMemcpyAsync(d_tokens_, h_tok.data(), sizeof(int) * rows, hipMemcpyHostToDevice, s));
-    ESP_HIP_TRY(hipMemcpyAsync(d_pos_, h_pos.data(), sizeof(int) * rows, hipMemcpyHostToDevice, s));
-    ESP_HIP_TRY(hipMemcpyAsync(d_seq_, h_seq.data(), sizeof(int) * rows, hipMemcpyHostToDevice, s));
-    ESP_HIP_TRY(hipStreamSynchronize(s));   // the host vectors go out of scope
-    ESP_HIP_TRY(launch_embed(embedding_, embedding_f16_, d_tokens_, rows, d, hidden_, s));
-    (void)ad; (void)kd; (void)hd; (void)kv16;
+    const int rc = upload_block_rows(seq, tokens, rows, base);
+    if (rc != ESP_OK) return rc;
+    ESP_HIP_TRY(launch_embed(embedding_, embedding_f16_, d_tokens_, rows, c_.d_model, hidden_, context().stream));
     return enqueue_layers_matrix(rows, true);
 }
 
@@ -689,7 +508,7 @@ bool LlamaRuntime::split_blocks_supported() const {
 
 int LlamaRuntime::enqueue_layers_split(int rows) {
     hipStream_t s = context().stream;
-    const int d = c_.d_model, ad = c_.attention_dim(), kd = c_.kv_dim(), hd = c_.hidden_dim;
+    const int d = c_.d_model, ad = c_.attention_dim(), kd = c_.kv_dim();
     const size_t cache_seq_stride = (size_t)kd * c_.max_seq;
     SplitRowsView xn{xn_, xn_lo_, xn_sums_}, ctx{ctx_, ctx_lo_, ctx_sums_}, act{act_, act_lo_, act_sums_};
     // RMSNorm of hidden_ (or of the split-K planes a projection left, added to hidden_ first) into split rows
@@ -738,7 +557,7 @@ int LlamaRuntime::enqueue_layers_split(int rows) {
 int LlamaRuntime::enqueue_layers_matrix(int rows, bool one_sequence_consecutive) {
     if (one_sequence_consecutive && split_blocks_supported()) return enqueue_layers_split(rows);
     hipStream_t s = context().stream;
-    const int d = c_.d_model, ad = c_.attention_dim(), kd = c_.kv_dim(), hd = c_.hidden_dim;
+    const int d = c_.d_model, ad = c_.attention_dim(), kd = c_.kv_dim();
     const bool kv16 = c_.kv_format == FMT_F16;
     const size_t cache_seq_stride = (size_t)kd * c_.max_seq;
     GemmParams g;
@@ -824,208 +643,31 @@ int LlamaRuntime::run_head(const float *hidden_rows, int count, bool want_logits
     return ESP_OK;
 }
 
-int LlamaRuntime::select_greedy(int seq, uint32_t *token) {
-    if (!finalized_) return fail(ESP_ERR_INVALID_ARGUMENT, "runtime is not finalized");
-    if (seq < 0 || seq >= c_.max_sequences || !token) return fail(ESP_ERR_OUT_OF_RANGE, "select_greedy(seq %d)", seq);
-    int rc = run_head(last_hidden_ + (size_t)seq * c_.d_model, 1);
-    if (rc != ESP_OK) return rc;
-    int t = 0;
-    ESP_HIP_TRY(hipMemcpyAsync(&t, d_out_tokens_, sizeof(int), hipMemcpyDeviceToHost, context().stream));
-    ESP_HIP_TRY(hipStreamSynchronize(context().stream));
-    *token = (uint32_t)t;
-    return ESP_OK;
-}
-
-int LlamaRuntime::head_rows(int count, uint32_t *tokens) {
-    if (!finalized_) return fail(ESP_ERR_INVALID_ARGUMENT, "runtime is not finalized");
-    if (count < 1 || count > kMaxStepRows || !tokens) return fail(ESP_ERR_INVALID_ARGUMENT, "head_rows(%d)", count);
-    int rc = run_head(hidden_, count);
-    if (rc != ESP_OK) return rc;
-    int t[kMaxStepRows];
-    ESP_HIP_TRY(hipMemcpyAsync(t, d_out_tokens_, sizeof(int) * count, hipMemcpyDeviceToHost, context().stream));
-    ESP_HIP_TRY(hipStreamSynchronize(context().stream));
-    for (int i = 0; i < count; i++) tokens[i] = (uint32_t)t[i];
-    return ESP_OK;
-}
-
-// head(last hidden of seq) -> argmax -> feed row 0 -> trunk -> keep row 0, captured once per sequence.
-// Both step graphs of a sequence, at its first replayed step (a one-off of a few milliseconds per runtime, outside any later call).
-int LlamaRuntime::capture_step_graph(int seq) {
-    const int rc = capture_steps(seq, 1, &step_graphs_[seq]);
-    return rc != ESP_OK ? rc : capture_steps(seq, kStepsPerGraph, &multi_graphs_[seq]);
-}
-
-// Replays `steps` greedy steps: graphs of kStepsPerGraph steps while that many are left, single steps for the rest.  Every boundary between two graph launches costs about 3.5 us on the device, whatever the graphs hold
-// (6-layer model: 8.1 k tok/s with one step per graph, 8.35 k with four, 8.45 k with sixteen; 8B: 736 / 738.5 / 738.5).
-int LlamaRuntime::replay_steps(int seq, int steps) {
+// Head GEMV with the arg-max in its epilogue, then one launch that picks the token among the workgroups' candidates, feeds it and
+// fetches its embedding; the last layer writes the new hidden state where the next step's head reads it: 2 + 5 per layer launches
+// (3 + 5 per layer when the head has to store its logits).
+int LlamaRuntime::enqueue_greedy_token(int seq) {
     hipStream_t s = context().stream;
-    int i = 0;
-    if (multi_graphs_[seq])
-        for (; i + kStepsPerGraph <= steps; i += kStepsPerGraph) ESP_HIP_TRY(hipGraphLaunch(multi_graphs_[seq], s));
-    for (; i < steps; i++) ESP_HIP_TRY(hipGraphLaunch(step_graphs_[seq], s));
-    return ESP_OK;
-}
-
-int LlamaRuntime::capture_steps(int seq, int count, hipGraphExec_t *out) {
-    hipStream_t s = context().stream;
-    hipGraph_t graph = nullptr;
-    ESP_HIP_TRY(hipStreamSynchronize(s));
-    ESP_HIP_TRY(hipStreamBeginCapture(s, hipStreamCaptureModeThreadLocal));
-    int rc = ESP_OK;
-    float *kept = last_hidden_ + (size_t)seq * c_.d_model;
-    for (int step = 0; step < count && rc == ESP_OK; step++) {
-        // head GEMV with the arg-max in its epilogue, then one launch that picks the token among the workgroups' candidates,
-        // feeds it and fetches its embedding; the last layer writes the new hidden state where the next step's head reads
-        // it: 2 + 5 per layer launches (3 + 5 per layer when the head has to store its logits)
-        GemvParams g;
-        g.w = lm_head_; g.norm_x = kept; g.norm_w = final_norm_; g.norm_eps = c_.norm_eps; g.batch = 1;
-        hipError_t e;
-        if (head_fuses_argmax()) {
-            int blocks = 0;
-            g.epilogue = EPI_ARGMAX;
-            g.argmax_value = argmax_scratch_.part_value; g.argmax_index = argmax_scratch_.part_index; g.argmax_capacity = head_partial_capacity_;
-            g.argmax_blocks = &blocks;
-            e = launch_gemv(g, s);
-            if (e == hipSuccess)
-                e = launch_greedy_tail(argmax_scratch_, blocks, d_out_tokens_, seq, d_visible_, d_tokens_, d_pos_, d_seq_, d_log_, d_log_count_,
-                                       c_.max_seq, embedding_, embedding_f16_, c_.d_model, hidden_, c_.eos_token, s);
-        } else {
-            g.y = logits_; g.epilogue = EPI_STORE_F32;
-            e = launch_gemv(g, s);
-            if (e == hipSuccess)
-                e = launch_greedy_step_tail(logits_, c_.vocab, d_out_tokens_, argmax_scratch_, seq, d_visible_, d_tokens_, d_pos_, d_seq_, d_log_,
-                                            d_log_count_, c_.max_seq, embedding_, embedding_f16_, c_.d_model, hidden_, c_.eos_token, s);
-        }
-        if (e != hipSuccess) rc = fail_hip(e, "greedy step head");
-        if (rc == ESP_OK) rc = enqueue_trunk(1, true, kept);
+    GemvParams g;
+    g.w = lm_head_; g.norm_x = device_last_hidden(seq); g.norm_w = final_norm_; g.norm_eps = c_.norm_eps; g.batch = 1;
+    hipError_t e;
+    if (head_fuses_argmax()) {
+        int blocks = 0;
+        g.epilogue = EPI_ARGMAX;
+        g.argmax_value = argmax_scratch_.part_value; g.argmax_index = argmax_scratch_.part_index; g.argmax_capacity = head_partial_capacity_;
+        g.argmax_blocks = &blocks;
+        e = launch_gemv(g, s);
+        if (e == hipSuccess)
+            e = launch_greedy_tail(argmax_scratch_, blocks, d_out_tokens_, seq, d_visible_, d_tokens_, d_pos_, d_seq_, d_log_, d_log_count_,
+                                   c_.max_seq, embedding_, embedding_f16_, c_.d_model, hidden_, c_.eos_token, s);
+    } else {
+        g.y = logits_; g.epilogue = EPI_STORE_F32;
+        e = launch_gemv(g, s);
+        if (e == hipSuccess)
+            e = launch_greedy_step_tail(logits_, c_.vocab, d_out_tokens_, argmax_scratch_, seq, d_visible_, d_tokens_, d_pos_, d_seq_, d_log_,
+                                        d_log_count_, c_.max_seq, embedding_, embedding_f16_, c_.d_model, hidden_, c_.eos_token, s);
     }
-    hipError_t e = hipStreamEndCapture(s, &graph);
-    if (rc != ESP_OK) { if (graph) (void)hipGraphDestroy(graph); return rc; }
-    if (e != hipSuccess) return fail_hip(e, "hipStreamEndCapture");
-    hipGraphExec_t exec = nullptr;
-    e = hipGraphInstantiate(&exec, graph, nullptr, nullptr, 0);
-    (void)hipGraphDestroy(graph);
-    if (e != hipSuccess) return fail_hip(e, "hipGraphInstantiate");
-    *out = exec;
-    return ESP_OK;
-}
-
-int LlamaRuntime::continue_greedy(int seq, int steps, uint32_t *out_tokens) {
-    if (!finalized_) return fail(ESP_ERR_INVALID_ARGUMENT, "runtime is not finalized");
-    sync_tuning();
-    if (seq < 0 || seq >= c_.max_sequences) return fail(ESP_ERR_OUT_OF_RANGE, "sequence %d of %d", seq, c_.max_sequences);
-    if (steps < 0) return fail(ESP_ERR_INVALID_ARGUMENT, "steps must be >= 0");
-    if (visible_[seq] + steps > c_.max_seq)
-        return fail(ESP_ERR_OUT_OF_RANGE, "runtime position %d + %d steps exceeds context %d", visible_[seq], steps, c_.max_seq);
-    if (steps == 0) return ESP_OK;
-    hipStream_t s = context().stream;
-    int rc;
-    if (!use_graph_ || timing_enabled_) {
-        for (int i = 0; i < steps; i++) {
-            uint32_t t = 0;
-            if ((rc = select_greedy(seq, &t)) != ESP_OK) return rc;
-            if (out_tokens) out_tokens[i] = t;
-            if ((rc = advance(seq, t)) != ESP_OK) return rc;
-        }
-        return ESP_OK;
-    }
-    if (!step_graphs_[seq]) {
-        // one eager step first: it configures every kernel's LDS limit outside the capture
-        uint32_t t = 0;
-        if ((rc = select_greedy(seq, &t)) != ESP_OK) return rc;
-        if (out_tokens) out_tokens[0] = t;
-        if ((rc = advance(seq, t)) != ESP_OK) return rc;
-        if ((rc = capture_step_graph(seq)) != ESP_OK) return rc;
-        if (out_tokens) out_tokens += 1;
-        steps -= 1;
-        if (steps == 0) return ESP_OK;
-    }
-    ESP_HIP_TRY(launch_set_ints(d_visible_ + seq, visible_[seq], d_log_count_, 0, s));
-    ESP_HIP_TRY(launch_set_ints(d_log_count_ + 1, 0, d_log_count_ + 2, 0, s));   // not stopped, and no stop at the stop token
-    if ((rc = replay_steps(seq, steps)) != ESP_OK) return rc;
-    std::vector<int> log(steps);
-    ESP_HIP_TRY(hipMemcpyAsync(log.data(), d_log_, sizeof(int) * steps, hipMemcpyDeviceToHost, s));
-    ESP_HIP_TRY(hipStreamSynchronize(s));
-    visible_[seq] += steps;
-    if (out_tokens) for (int i = 0; i < steps; i++) out_tokens[i] = (uint32_t)log[i];
-    return ESP_OK;
-}
-
-// continue_greedy that ends with the stop token: the token is emitted and not consumed, as in the reference loop (:6385-6388).  The
-// replays run in chunks; the step graph itself notices the stop token, and replays after it change nothing.
-int LlamaRuntime::continue_greedy_until_stop(int seq, int steps, uint32_t *out_tokens, int *produced) {
-    if (!finalized_) return fail(ESP_ERR_INVALID_ARGUMENT, "runtime is not finalized");
-    if (seq < 0 || seq >= c_.max_sequences || !out_tokens || !produced) return fail(ESP_ERR_OUT_OF_RANGE, "continue_greedy_until_stop(seq %d)", seq);
-    *produced = 0;
-    sync_tuning();
-    if (steps < 0) return fail(ESP_ERR_INVALID_ARGUMENT, "steps must be >= 0");
-    if (visible_[seq] + steps > c_.max_seq)
-        return fail(ESP_ERR_OUT_OF_RANGE, "runtime position %d + %d steps exceeds context %d", visible_[seq], steps, c_.max_seq);
-    const int eos = c_.eos_token;
-    hipStream_t s = context().stream;
-    int rc;
-    auto eager_step = [&](bool *stopped) {
-        uint32_t t = 0;
-        int r = select_greedy(seq, &t);
-        if (r != ESP_OK) return r;
-        out_tokens[(*produced)++] = t;
-        *stopped = eos >= 0 && t == (uint32_t)eos;
-        return *stopped ? ESP_OK : advance(seq, t);
-    };
-    bool stopped = false;
-    if (!use_graph_ || timing_enabled_) {
-        while (*produced < steps && !stopped)
-            if ((rc = eager_step(&stopped)) != ESP_OK) return rc;
-        return ESP_OK;
-    }
-    if (steps > 0) {
-        // The first step always runs from the host.  A replay that finds the stop token re-embeds the row that sits in
-        // d_tokens_/d_pos_/d_seq_[0] and lets the trunk recompute it, which changes nothing only when that row is the one this
-        // sequence consumed last; after a prompt block or another sequence's pass those arrays hold something else.  advance()
-        // leaves exactly that row there (and the eager step configures every kernel's LDS limit outside a capture).
-        if ((rc = eager_step(&stopped)) != ESP_OK) return rc;
-        if (stopped) return ESP_OK;
-        if (!step_graphs_[seq] && (rc = capture_step_graph(seq)) != ESP_OK) return rc;
-    }
-    if (*produced >= steps) return ESP_OK;
-    const int first = *produced, want = steps - first;
-    ESP_HIP_TRY(launch_set_ints(d_visible_ + seq, visible_[seq], d_log_count_, 0, s));
-    ESP_HIP_TRY(launch_set_ints(d_log_count_ + 1, 0, d_log_count_ + 2, 1, s));
-    int state[2] = {0, 0};   // tokens logged, stopped
-    for (int launched = 0; launched < want && !state[1];) {
-        const int chunk = want - launched < 32 ? want - launched : 32;
-        if ((rc = replay_steps(seq, chunk)) != ESP_OK) return rc;
-        launched += chunk;
-        ESP_HIP_TRY(hipMemcpyAsync(state, d_log_count_, sizeof(state), hipMemcpyDeviceToHost, s));
-        ESP_HIP_TRY(hipStreamSynchronize(s));
-    }
-    const int logged = state[0] < want ? state[0] : want;
-    std::vector<int> log(logged > 0 ? logged : 1);
-    if (logged > 0) {
-        ESP_HIP_TRY(hipMemcpyAsync(log.data(), d_log_, sizeof(int) * logged, hipMemcpyDeviceToHost, s));
-        ESP_HIP_TRY(hipStreamSynchronize(s));
-    }
-    for (int i = 0; i < logged; i++) out_tokens[first + i] = (uint32_t)log[i];
-    *produced = first + logged;
-    visible_[seq] += logged - (state[1] ? 1 : 0);   // every logged token was consumed, except a stop token
-    return ESP_OK;
-}
-
-int LlamaRuntime::read_last_hidden(int seq, float *out) {
-    if (!finalized_ || seq < 0 || seq >= c_.max_sequences || !out) return fail(ESP_ERR_INVALID_ARGUMENT, "read_last_hidden");
-    ESP_HIP_TRY(hipMemcpyAsync(out, last_hidden_ + (size_t)seq * c_.d_model, (size_t)c_.d_model * 4, hipMemcpyDeviceToHost,
-                               context().stream));
-    ESP_HIP_TRY(hipStreamSynchronize(context().stream));
-    return ESP_OK;
-}
-
-int LlamaRuntime::read_logits(int seq, float *out) {
-    if (!finalized_ || seq < 0 || seq >= c_.max_sequences || !out) return fail(ESP_ERR_INVALID_ARGUMENT, "read_logits");
-    int rc = run_head(last_hidden_ + (size_t)seq * c_.d_model, 1, true);
-    if (rc != ESP_OK) return rc;
-    ESP_HIP_TRY(hipMemcpyAsync(out, logits_, (size_t)c_.vocab * 4, hipMemcpyDeviceToHost, context().stream));
-    ESP_HIP_TRY(hipStreamSynchronize(context().stream));
-    return ESP_OK;
+    return e == hipSuccess ? ESP_OK : fail_hip(e, "greedy step head");
 }
 
 }  // namespace esp

@@ -85,16 +85,19 @@ def _ptr(a):
     return a.ctypes.data_as(C.c_void_p)
 
 
+ARCHITECTURES = ("gpt2", "llama", "layered")
+
+
 def config_struct(cfg: llama.MultiModelConfig) -> ModelConfigStruct:
     return ModelConfigStruct(cfg.name.encode()[:63], cfg.n_layer, cfg.n_head, cfg.n_kv_head, cfg.d_model, cfg.head_dim, cfg.hidden_dim,
-                             cfg.vocab, cfg.max_seq, cfg.norm_eps, cfg.rope_theta, cfg.eos_token, 0 if cfg.architecture == "gpt2" else 1)
+                             cfg.vocab, cfg.max_seq, cfg.norm_eps, cfg.rope_theta, cfg.eos_token, ARCHITECTURES.index(cfg.architecture))
 
 
 def config_from_struct(s: ModelConfigStruct) -> llama.MultiModelConfig:
     return llama.MultiModelConfig(n_layer=s.n_layer, n_head=s.n_head, n_kv_head=s.n_kv_head, d_model=s.d_model, head_dim=s.head_dim,
                                   hidden_dim=s.hidden_dim, vocab=s.vocab, max_seq=s.max_seq, norm_eps=s.norm_eps,
                                   rope_theta=s.rope_theta, eos_token=s.eos_token, name=s.name.decode(),
-                                  architecture="gpt2" if s.architecture == 0 else "llama")
+                                  architecture=ARCHITECTURES[s.architecture])
 
 
 # ---- registry and head strategy ----------------------------------------------
@@ -159,6 +162,22 @@ def load_metadata(path: str) -> llama.MultiModelConfig:
     s = ModelConfigStruct()
     _lib.check(_L().esp_model_config_load_metadata(path.encode(), C.byref(s)))
     return config_from_struct(s)
+
+
+def load_model_config(model_dir: str, max_seq: int) -> llama.MultiModelConfig:
+    """The configuration of a model directory: config.json of a registered layered architecture, else metadata.json."""
+    L, s = _L(), ModelConfigStruct()
+    L.esp_model_config_load_dir.restype = C.c_int
+    L.esp_model_config_load_dir.argtypes = [C.c_char_p, C.c_int, C.POINTER(ModelConfigStruct)]
+    _lib.check(L.esp_model_config_load_dir(model_dir.encode(), max_seq, C.byref(s)))
+    return config_from_struct(s)
+
+
+def layered_architectures() -> list[str]:
+    """Names of the registered layered architectures."""
+    L = _L()
+    L.esp_layered_architecture_at.restype = C.c_char_p
+    return [L.esp_layered_architecture_at(i).decode() for i in range(L.esp_layered_architecture_count())]
 
 
 def write_metadata(cfg: llama.MultiModelConfig, path: str) -> None:
@@ -328,6 +347,7 @@ class RealModelInferenceEngine:
         """A non-owning view of the engine's runtime."""
         rt = llama.LlamaRuntime.__new__(llama.LlamaRuntime)
         rt.cfg, rt._L, rt._h = self.cfg, _L(), _L().esp_engine_runtime(self._h)
+        rt.engine = self                       # the view keeps its owner alive
         rt.close = lambda: None
         return rt
 

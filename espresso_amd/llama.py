@@ -30,7 +30,7 @@ class MultiModelConfig:
     rope_theta: float = 10000.0
     eos_token: int = -1
     name: str = "llama"
-    architecture: str = "llama"   # or "gpt2" (registry entries only: the runtime runs the llama family)
+    architecture: str = "llama"   # or "layered" (config.json lists the layers), or "gpt2" (registry entries only)
 
     @property
     def attention_dim(self) -> int:
@@ -113,6 +113,28 @@ class LlamaRuntime:
         out = np.empty(self.cfg.vocab, dtype=np.float32)
         _lib.check(self._L.esp_llama_read_logits(self._h, sequence, _ptr(out)))
         return out
+
+    def append(self, tokens, want=(), sequence: int = 0) -> np.ndarray:
+        """The sequence's next tokens; returns the logits [len(want), vocab] at the (ascending) places `want` among them."""
+        t, w = np.ascontiguousarray(tokens, dtype=np.uint32), np.ascontiguousarray(want, dtype=np.int32)
+        out = np.empty((w.size, self.cfg.vocab), dtype=np.float32)
+        _lib.check(self._L.esp_llama_append(self._h, sequence, _ptr(t), t.size, _ptr(w), w.size, _ptr(out)))
+        return out
+
+    def acquire_sequence(self) -> int:
+        s = C.c_int(-1)
+        _lib.check(self._L.esp_llama_acquire_sequence(self._h, C.byref(s)))
+        return int(s.value)
+
+    def release_sequence(self, sequence: int) -> None:
+        _lib.check(self._L.esp_llama_release_sequence(self._h, sequence))
+
+    def generate_sampled(self, prompt, max_tokens: int, temperature: float, seed: int) -> list[int]:
+        p = np.ascontiguousarray(prompt, dtype=np.uint32)
+        out = np.zeros(max(max_tokens, 1), dtype=np.uint32)
+        n, st = C.c_int(0), _lib.GenerationStatsStruct()
+        _lib.check(self._L.esp_llama_generate_sampled(self._h, _ptr(p), p.size, max_tokens, temperature, seed, _ptr(out), C.byref(n), C.byref(st)))
+        return out[:n.value].tolist()
 
     def generate(self, prompt, max_tokens: int):
         p = np.ascontiguousarray(prompt, dtype=np.uint32)

@@ -174,6 +174,13 @@ int esp_llama_set_visible_token_count(ESPLlamaRuntime *runtime, int sequence, in
 /* lastHidden [d_model] and the full-vocabulary logits of the current state [vocab], fp32. */
 int esp_llama_read_last_hidden(ESPLlamaRuntime *runtime, int sequence, float *out);
 int esp_llama_read_logits(ESPLlamaRuntime *runtime, int sequence, float *out);
+/* The next `count` tokens of a sequence, from the caches and recurrent state its earlier tokens left (a prompt may arrive in portions
+ * cut anywhere).  `want` lists, ascending, the places among these tokens whose logits go to `logits` ([want_count][vocab]); both may
+ * be null.  esp_llama_prefill is the same from an empty sequence. */
+int esp_llama_append(ESPLlamaRuntime *runtime, int sequence, const uint32_t *tokens, int count, const int *want, int want_count, float *logits);
+/* Sequence slots for requests that come and go: takes the lowest free slot (an empty sequence), gives one back. */
+int esp_llama_acquire_sequence(ESPLlamaRuntime *runtime, int *sequence);
+int esp_llama_release_sequence(ESPLlamaRuntime *runtime, int sequence);
 
 typedef struct ESPGenerationStats {
     int32_t generated;
@@ -185,6 +192,9 @@ typedef struct ESPGenerationStats {
  * else it receives one latency per generated token (GenerationResult.tokenLatenciesMs, :17-55). */
 int esp_llama_generate(ESPLlamaRuntime *runtime, const uint32_t *prompt, int prompt_count, int max_tokens,
                        uint32_t *out_tokens, int *out_count, ESPGenerationStats *stats, double *token_latencies_ms);
+/* Sampled generation at temperature > 0 (esp_sample_token on every step's logits, draws from a SplitMix64 of `seed`). */
+int esp_llama_generate_sampled(ESPLlamaRuntime *runtime, const uint32_t *prompt, int prompt_count, int max_tokens, float temperature,
+                               uint64_t seed, uint32_t *out_tokens, int *out_count, ESPGenerationStats *stats);
 
 typedef struct ESPTwoTokenStats {
     /* one pass = one batched verify of [current token, proposed token] by the target model; committed
@@ -266,12 +276,18 @@ typedef struct ESPModelConfig {
     int32_t n_layer, n_head, n_kv_head, d_model, head_dim, hidden_dim, vocab, max_seq;
     float norm_eps, rope_theta;
     int32_t eos_token;     /* -1: none */
-    int32_t architecture;  /* 0 gpt2, 1 llama */
+    int32_t architecture;  /* 0 gpt2, 1 llama, 2 layered (config.json lists the layers) */
 } ESPModelConfig;
 /* metadata.json as GGUFModelLoader writes it (GGUFModelLoader.swift:203-222) and the engine validates it
  * (RealModelInferenceEngine.swift:7658-7694). */
 int esp_model_config_load_metadata(const char *metadata_json_path, ESPModelConfig *out);
 int esp_model_config_write_metadata(const ESPModelConfig *config, const char *metadata_json_path);
+/* The configuration of a model directory, whatever its kind: a config.json that names a registered layered architecture (its weights
+ * in model.safetensors; architecture = 2, and max_seq is the caller's choice), else metadata.json as above. */
+int esp_model_config_load_dir(const char *model_dir, int max_seq, ESPModelConfig *out);
+/* Names of the registered layered architectures. */
+int esp_layered_architecture_count(void);
+const char *esp_layered_architecture_at(int index);
 
 /* ModelRegistry (Sources/ModelSupport/ModelRegistry.swift): esp_model_registry_count() named configurations in name
  * order; esp_model_registry_config(name, &out) = ModelRegistry.config(named:), ESP_ERR_INVALID_ARGUMENT when unknown. */
