@@ -217,6 +217,10 @@ int DecoderRuntime::append(int seq, const uint32_t *tokens, int count, const int
     for (int i = 0; i < want_count; i++)
         if (want[i] < 0 || want[i] >= count || (i > 0 && want[i] <= want[i - 1]))
             return fail(ESP_ERR_OUT_OF_RANGE, "append: wanted places must ascend within 0..%d", count - 1);
+    const int start = visible_[seq];   // every token is checked before the first one changes any state
+    if (start + count > max_seq) return fail(ESP_ERR_OUT_OF_RANGE, "runtime position %d exceeds context %d", max_seq, max_seq);
+    for (int i = 0; i < count; i++)
+        if (tokens[i] >= (uint32_t)vocab) return fail(ESP_ERR_OUT_OF_RANGE, "token %u is outside vocab %d", tokens[i], vocab);
     hipStream_t s = context().stream;
     int given = 0;   // wanted rows delivered so far
     auto deliver = [&](const float *rows, int n) -> int {
@@ -229,10 +233,6 @@ int DecoderRuntime::append(int seq, const uint32_t *tokens, int count, const int
     };
     if (matrix_prefill_ && count >= matrix_prefill_min_tokens() && matrix_prefill_supported()) {
         // blocks of rows through the MFMA kernels (one pass over the weights per block)
-        const int start = visible_[seq];
-        if (start + count > max_seq) return fail(ESP_ERR_OUT_OF_RANGE, "runtime position %d exceeds context %d", max_seq, max_seq);
-        for (int i = 0; i < count; i++)
-            if (tokens[i] >= (uint32_t)vocab) return fail(ESP_ERR_OUT_OF_RANGE, "token %u is outside vocab %d", tokens[i], vocab);
         for (int off = 0; off < count; off += block_rows_) {
             const int rows = count - off < block_rows_ ? count - off : block_rows_;
             if ((rc = prefill_block(seq, tokens + off, rows, start + off)) != ESP_OK) return rc;
