@@ -338,6 +338,61 @@ def run_two_token_8b(steps: int) -> dict:
     return out
 
 
+def run_layered(names, steps: int, prompt: int = 512) -> dict:
+    """Layered models (retention and latent attention, bf16 weights) beside llama models of equal width, feed-forward, vocabulary and
+    depth with fp16 weights: six random-init layers each, prefill of one block-aligned prompt (the second walk, every kernel warm)
+    and greedy decode at batch 1 behind it, as captured graphs.  step_weight_bytes: what a decode step reads of weights."""
+    import espresso_amd.layered as layered
+    import espresso_amd.llama as ll
+    import espresso_amd.synthetic as syn
+    from espresso_amd import _lib
+
+    def measure(rt, vocab):
+        tokens = np.random.default_rng(7).integers(0, vocab, prompt).astype(np.uint32)
+        walks = []
+        for _ in range(4):
+            rt.last_hidden()
+            t0 = time.perf_counter()
+            rt.prefill(tokens)
+            rt.last_hidden()
+            walks.append(time.perf_counter() - t0)
+        ll.continue_greedy(rt, 24)
+        rt.last_hidden()
+        t0 = time.perf_counter()
+        ll.continue_greedy(rt, steps)
+        rt.last_hidden()
+        per_step = (time.perf_counter() - t0) / steps
+        return {"prefill_ms": round(min(walks[1:]) * 1e3, 3), "prefill_tok_s": round(prompt / min(walks[1:])), "decode_us": round(per_step * 1e6, 1),
+                "decode_tok_s": round(1.0 / per_step, 1), "step_weight_bytes": rt.weight_bytes,
+                "step_weight_gbps": round(rt.weight_bytes / per_step / 1e9, 1), "frac_hbm_peak": round(rt.weight_bytes / per_step / 1e9 / HBM_PEAK_GBPS, 3)}
+
+    results = {}
+    for name in names:
+        config, llama = syn.LAYERED_SIZES[name]
+        rt = layered.LayeredRuntime(config, max_seq=llama["max_seq"], seed=5)
+        own = measure(rt, config["vocab"])
+        own["sequence_state_bytes"] = layered.sequence_bytes(rt)
+        ll.set_graph_replay(rt, False)
+        layered.set_kernel_timing(rt, True)
+        tokens = np.arange(prompt, dtype=np.uint32) % config["vocab"]
+        for phase, run, count in (("prefill", lambda: rt.prefill(tokens), 1), ("decode", lambda: ll.continue_greedy(rt, 16), 16)):
+            run()
+            layered.kernel_times(rt)
+            run()
+            t = layered.kernel_times(rt)
+            own[phase + "_kernel_us"] = {k: round(v["total_us"] / count, 1) for k, v in t.items() if v["brackets"]}
+        rt.close()
+        peer, _ = syn.build_runtime(ll.MultiModelConfig(**llama), _lib.FORMAT_F16, seed=3, kv_format=_lib.FORMAT_F16)
+        other = measure(peer, llama["vocab"])
+        peer.close()
+        results[name] = {"layered": own, "llama_f16": other,
+                         "prefill_ratio_per_weight": round((own["prefill_tok_s"] * own["step_weight_bytes"]) / (other["prefill_tok_s"] * other["step_weight_bytes"]), 3),
+                         "decode_ratio_per_weight": round(own["step_weight_gbps"] / other["step_weight_gbps"], 3)}
+    return {"metric": "layered model prefill and decode tok/s (6 layers, bf16) beside llama f16 of equal size", "unit": "tok/s", "n_gpus": 1, "data": "synthetic",
+            "prompt_tokens": prompt, "steps": steps, "results": results,
+            "note": "kernel_us: an event pair around each layer's launches of a class, launches one by one (no graph); event overhead included"}
+
+
 def run_stamps() -> dict:
     """Where the time of one Q4_K GEMV launch goes: every wavefront of one launch inside a back-to-back train over copies
     of the matrix that exceed the caches (weights from HBM, code and activations warm) records 100 MHz wall-clock stamps at its start, after the activations are
@@ -398,6 +453,8 @@ def main() -> None:
     ap.add_argument("--microbench", action="store_true", help="weight-GEMV microbenchmark (Q4_K / Q4_0, batch 1, 2, 8) instead of decode")
     ap.add_argument("--stamps", action="store_true", help="per-wavefront time stamps inside one Q4_K GEMV launch, per decode shape and kernel")
     ap.add_argument("--two-token", action="store_true", help="exact two-token draft/verify decode on the 6-layer model instead of plain decode")
+    ap.add_argument("--layered", nargs="*", metavar="SIZE", default=None,
+                    help="layered models (retention and latent attention) beside llama f16 models of equal size: d768, d2048, d4096 (default all)")
     args = ap.parse_args()
     if args.gpus != 1:
         raise SystemExit("bench.py measures one GPU: this path is a batch-1 decode on a single MI355X; run with --gpus 1")
@@ -410,6 +467,9 @@ def main() -> None:
         out = run_two_token(args.steps or 240)
         out["llama3-8b-q4k"] = run_two_token_8b(args.steps or 240)
         print(json.dumps(out))
+        return
+    if args.layered is not None:
+        print(json.dumps(run_layered(args.layered or ["d768", "d2048", "d4096"], args.steps or 128)))
         return
     if args.stamps:
         print(json.dumps(run_stamps()))

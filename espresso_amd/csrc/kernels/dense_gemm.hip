@@ -36,21 +36,27 @@ struct DenseGemmArgs {
 };
 
 // Eight consecutive values of an operand row on their way to LDS.
+typedef uint32_t uintx4 __attribute__((ext_vector_type(4)));
+typedef float floatx4 __attribute__((ext_vector_type(4)));
+typedef float floatx8 __attribute__((ext_vector_type(8)));
 template <typename T>
-struct Piece;
+struct PieceOf { typedef uintx4 type; };
 template <>
-struct Piece<uint16_t> { uint4 v; };
-template <>
-struct Piece<float> { float4 v0, v1; };
-__device__ __forceinline__ void fetch_piece(const uint16_t *p, Piece<uint16_t> &d) { d.v = *reinterpret_cast<const uint4 *>(p); }
-__device__ __forceinline__ void fetch_piece(const float *p, Piece<float> &d) { d.v0 = reinterpret_cast<const float4 *>(p)[0]; d.v1 = reinterpret_cast<const float4 *>(p)[1]; }
-__device__ __forceinline__ void store_piece(const Piece<uint16_t> &d, uint16_t *lds) { *reinterpret_cast<uint4 *>(lds) = d.v; }
-__device__ __forceinline__ void store_piece(const Piece<float> &d, float *lds) { reinterpret_cast<float4 *>(lds)[0] = d.v0; reinterpret_cast<float4 *>(lds)[1] = d.v1; }
-__device__ __forceinline__ void store_piece(const Piece<uint16_t> &d, float *lds) {
-    float f[8];
-    matrix::unpack_bf16(d.v, f);
-    reinterpret_cast<float4 *>(lds)[0] = make_float4(f[0], f[1], f[2], f[3]);
-    reinterpret_cast<float4 *>(lds)[1] = make_float4(f[4], f[5], f[6], f[7]);
+struct PieceOf<float> { typedef floatx8 type; };
+__device__ __forceinline__ uintx4 fetch_piece(const uint16_t *p) { return *reinterpret_cast<const uintx4 *>(p); }
+__device__ __forceinline__ floatx8 fetch_piece(const float *p) {
+    const floatx4 a = reinterpret_cast<const floatx4 *>(p)[0], b = reinterpret_cast<const floatx4 *>(p)[1];
+    return __builtin_shufflevector(a, b, 0, 1, 2, 3, 4, 5, 6, 7);
+}
+__device__ __forceinline__ void store_piece(uintx4 d, uint16_t *lds) { *reinterpret_cast<uintx4 *>(lds) = d; }
+__device__ __forceinline__ void store_piece(floatx8 d, float *lds) {
+    reinterpret_cast<floatx4 *>(lds)[0] = __builtin_shufflevector(d, d, 0, 1, 2, 3);
+    reinterpret_cast<floatx4 *>(lds)[1] = __builtin_shufflevector(d, d, 4, 5, 6, 7);
+}
+__device__ __forceinline__ void store_piece(uintx4 d, float *lds) {
+    const uintx4 lo = d << 16, hi = d & 0xFFFF0000u;
+    reinterpret_cast<floatx4 *>(lds)[0] = __builtin_bit_cast(floatx4, __builtin_shufflevector(lo, hi, 0, 4, 1, 5));
+    reinterpret_cast<floatx4 *>(lds)[1] = __builtin_bit_cast(floatx4, __builtin_shufflevector(lo, hi, 2, 6, 3, 7));
 }
 
 template <typename TA, typename TB, int WM, int WN, int TM, int TN>
@@ -58,7 +64,7 @@ __global__ __launch_bounds__(64 * WM * WN) void dense_gemm_kernel(DenseGemmArgs 
     using E = typename std::conditional<std::is_same<TA, float>::value || std::is_same<TB, float>::value, float, uint16_t>::type;
     constexpr int THREADS = 64 * WM * WN, BM = 32 * WM * TM, BN = 32 * WN * TN;
     constexpr int KT = 128 / sizeof(E), LDK = 144 / sizeof(E), NCH = KT / 8;   // values per tile row, per LDS row; pieces per tile row
-    constexpr int XA = BM * NCH / THREADS, XB = BN * NCH / THREADS, DEPTH = 2;
+    constexpr int XA = BM * NCH / THREADS, XB = BN * NCH / THREADS;
     static_assert(XA >= 1 && XB >= 1, "tile too small for the copy loop");
     __shared__ E at[2][BM * LDK];
     __shared__ E bt[2][BN * LDK];
@@ -79,8 +85,10 @@ __global__ __launch_bounds__(64 * WM * WN) void dense_gemm_kernel(DenseGemmArgs 
 #pragma unroll
         for (int j = 0; j < TN; j++) acc[i][j] = matrix::zero_accumulator();
 
-    Piece<TA> pa[DEPTH][XA];
-    Piece<TB> pb[DEPTH][XB];
+    typedef typename PieceOf<TA>::type PA;
+    typedef typename PieceOf<TB>::type PB;
+    PA pa0[XA], pa1[XA];   // even and odd tiles
+    PB pb0[XB], pb1[XB];
     const TA *ar[XA];
     const TB *br[XB];
 #pragma unroll
@@ -93,53 +101,57 @@ __global__ __launch_bounds__(64 * WM * WN) void dense_gemm_kernel(DenseGemmArgs 
         const int piece = tid + i * THREADS, row = n0 + piece / NCH;
         br[i] = bp + (size_t)(row < a.n ? row : a.n - 1) * a.ldb + (piece % NCH) * 8;
     }
-    auto fetch = [&](int S, int tile) {   // S is a constant after unrolling; tiles past the end repeat the last one
+    auto fetch = [&](PA (&pa)[XA], PB (&pb)[XB], int tile) {   // tiles past the end repeat the last one
         const size_t k = (size_t)(tile < t_last ? tile : t_last) * KT;
 #pragma unroll
-        for (int i = 0; i < XA; i++) fetch_piece(ar[i] + k, pa[S][i]);
+        for (int i = 0; i < XA; i++) pa[i] = fetch_piece(ar[i] + k);
 #pragma unroll
-        for (int i = 0; i < XB; i++) fetch_piece(br[i] + k, pb[S][i]);
+        for (int i = 0; i < XB; i++) pb[i] = fetch_piece(br[i] + k);
     };
-    auto stage = [&](int S, int buf) {
+    auto stage = [&](const PA (&pa)[XA], const PB (&pb)[XB], int buf) {
 #pragma unroll
         for (int i = 0; i < XA; i++) {
             const int piece = tid + i * THREADS;
-            store_piece(pa[S][i], at[buf] + piece / NCH * LDK + (piece % NCH) * 8);
+            store_piece(pa[i], at[buf] + piece / NCH * LDK + (piece % NCH) * 8);
         }
 #pragma unroll
         for (int i = 0; i < XB; i++) {
             const int piece = tid + i * THREADS;
-            store_piece(pb[S][i], bt[buf] + piece / NCH * LDK + (piece % NCH) * 8);
+            store_piece(pb[i], bt[buf] + piece / NCH * LDK + (piece % NCH) * 8);
         }
     };
-    fetch(0, t_begin);
-    fetch(1, t_begin + 1);
-    stage(0, 0);
-    fetch(0, t_begin + 2);
+    fetch(pa0, pb0, t_begin);
+    fetch(pa1, pb1, t_begin + 1);
+    stage(pa0, pb0, 0);
+    fetch(pa0, pb0, t_begin + 2);
     __syncthreads();
-    for (int t0 = t_begin; t0 < t_end; t0 += 2) {
+    auto multiply = [&](int buf) {
 #pragma unroll
-        for (int u = 0; u < 2; u++) {
-            if (t0 + u < t_end) {
+        for (int ks = 0; ks < KT / 16; ks++) {
+            const int kk = ks * 16 + 8 * (lane >> 5);
+            typename Op<E>::frag af[TM], bf[TN];
 #pragma unroll
-                for (int ks = 0; ks < KT / 16; ks++) {
-                    const int kk = ks * 16 + 8 * (lane >> 5);
-                    typename Op<E>::frag af[TM], bf[TN];
+            for (int i = 0; i < TM; i++) af[i] = Op<E>::load(at[buf] + ((wm * TM + i) * 32 + (lane & 31)) * LDK + kk);
 #pragma unroll
-                    for (int i = 0; i < TM; i++) af[i] = Op<E>::load(at[u] + ((wm * TM + i) * 32 + (lane & 31)) * LDK + kk);
+            for (int j = 0; j < TN; j++) bf[j] = Op<E>::load(bt[buf] + ((wn * TN + j) * 32 + (lane & 31)) * LDK + kk);
 #pragma unroll
-                    for (int j = 0; j < TN; j++) bf[j] = Op<E>::load(bt[u] + ((wn * TN + j) * 32 + (lane & 31)) * LDK + kk);
+            for (int i = 0; i < TM; i++)
 #pragma unroll
-                    for (int i = 0; i < TM; i++)
-#pragma unroll
-                        for (int j = 0; j < TN; j++) acc[i][j] = Op<E>::mma(af[i], bf[j], acc[i][j]);
-                }
-                stage(u ^ 1, u ^ 1);
-                fetch(u ^ 1, t0 + u + 3);
-                __syncthreads();
-            }
+                for (int j = 0; j < TN; j++) acc[i][j] = Op<E>::mma(af[i], bf[j], acc[i][j]);
         }
+    };
+    int t0 = t_begin;
+    for (; t0 + 1 < t_end; t0 += 2) {
+        multiply(0);
+        stage(pa1, pb1, 1);
+        fetch(pa1, pb1, t0 + 3);
+        __syncthreads();
+        multiply(1);
+        stage(pa0, pb0, 0);
+        fetch(pa0, pb0, t0 + 4);
+        __syncthreads();
     }
+    if (t0 < t_end) multiply(0);
 
     const int half = lane >> 5;
 #pragma unroll

@@ -4,8 +4,8 @@
 //
 // The kernels are bound by HBM: a weight is read once with 128-bit loads and costs a shift and a fused multiply-add.
 //   * a workgroup of eight wavefronts stages the whole activation row in LDS (fp32, the two halves of every eight values in planes
-//     of their own, so that a lane's two 128-bit reads are free of bank conflicts) and then walks units of 32 weight rows, four per
-//     wavefront; two workgroups fit a compute unit, which keeps 64 KB of weights on their way to it;
+//     of their own, so that a lane's two 128-bit reads are free of bank conflicts) and then walks units of weight rows: four rows per
+//     wavefront, two or one where the matrix has too few rows to give every compute unit work (the loads run further ahead then);
 //   * what surrounds the product lives in the staging and the epilogue: RMS norm (its scale factors out of the dot product), the
 //     per-head norm and gate of a retention output, SiLU(gate) * up, the residual sum, the soft cap of the logits;
 //   * the input side of a parallel layer is one launch over two activation rows: workgroups are dealt to the mixer's rows (norm1)
@@ -21,7 +21,7 @@ namespace {
 
 using detail::wave_sum;
 
-constexpr int kGemvThreads = 512, kGemvWaves = 8, kRowsPerWave = 4, kUnitRows = kGemvWaves * kRowsPerWave;
+constexpr int kGemvThreads = 512, kGemvWaves = 8, kRowAlign = 32;
 constexpr int kStep = 512;   // columns a wavefront takes per step: 64 lanes x 8
 enum GemvKind : int { KIND_IN, KIND_OUT, KIND_HEAD };
 
@@ -39,13 +39,17 @@ struct DenseGemvArgs {
     float mult, cap;
     const float *residual;
     int vocab;
+    float *best_value;                  // KIND_HEAD: the workgroup's largest logit and its lowest row
+    int *best_index;
 };
 
 // The place of column k in the staged row: groups of eight, the two fours of a group in separate planes.
 __device__ __forceinline__ int staged_at(int k, int k_pad) { return (k >> 3) * 4 + (k & 3) + ((k & 4) ? k_pad / 2 : 0); }
 
-template <int KIND>
+// RPW weight rows per wavefront, AHEAD steps of loads in flight
+template <int KIND, int RPW, int AHEAD>
 __global__ __launch_bounds__(kGemvThreads) void dense_gemv_kernel(DenseGemvArgs a) {
+    constexpr int kUnitRows = kGemvWaves * RPW;
     extern __shared__ float xs[];   // [k_pad], then [heads]
     __shared__ float red[kGemvWaves];
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
@@ -100,50 +104,81 @@ __global__ __launch_bounds__(kGemvThreads) void dense_gemv_kernel(DenseGemvArgs 
     const int stride = KIND == KIND_IN ? (second ? (int)gridDim.x - a.blocks_a : a.blocks_a) : (int)gridDim.x;
     const int units = second ? a.units_b : a.units_a, base_row = second ? a.mix_rows : 0;
     const int steps = a.k_pad / kStep;
+    float best = -INFINITY;
+    int best_row = 0x7FFFFFFF;
     for (int u = first; u < units; u += stride) {
-        const int row0 = base_row + u * kUnitRows + wave * kRowsPerWave;
+        const int row0 = base_row + u * kUnitRows + wave * RPW;
         const uint16_t *wr = a.w + (size_t)row0 * a.ld;
-        float acc[kRowsPerWave] = {0.f, 0.f, 0.f, 0.f};
-        uint4 next[kRowsPerWave];
-        auto fetch = [&](int step) {
+        float acc[RPW];
+#pragma unroll
+        for (int r = 0; r < RPW; r++) acc[r] = 0.0f;
+        uint4 ring[AHEAD][RPW];
+        auto fetch = [&](uint4 (&slot)[RPW], int step) {
             const int k = step * kStep + lane * 8, kc = k < a.ld ? k : 0;   // columns past the end meet staged zeros
 #pragma unroll
-            for (int r = 0; r < kRowsPerWave; r++) next[r] = *reinterpret_cast<const uint4 *>(wr + (size_t)r * a.ld + kc);
+            for (int r = 0; r < RPW; r++) slot[r] = *reinterpret_cast<const uint4 *>(wr + (size_t)r * a.ld + kc);
         };
-        fetch(0);
-        for (int step = 0; step < steps; step++) {
-            uint4 cur[kRowsPerWave];
-#pragma unroll
-            for (int r = 0; r < kRowsPerWave; r++) cur[r] = next[r];
-            if (step + 1 < steps) fetch(step + 1);
+        auto use = [&](const uint4 (&slot)[RPW], int step) {
             const float4 x0 = reinterpret_cast<const float4 *>(xs)[step * 64 + lane];
             const float4 x1 = reinterpret_cast<const float4 *>(xs + a.k_pad / 2)[step * 64 + lane];
             const float x[8] = {x0.x, x0.y, x0.z, x0.w, x1.x, x1.y, x1.z, x1.w};
 #pragma unroll
-            for (int r = 0; r < kRowsPerWave; r++) {
+            for (int r = 0; r < RPW; r++) {
                 float w[8];
-                matrix::unpack_bf16(cur[r], w);
+                matrix::unpack_bf16(slot[r], w);
 #pragma unroll
                 for (int i = 0; i < 8; i++) acc[r] = __builtin_fmaf(w[i], x[i], acc[r]);
             }
+        };
+#pragma unroll
+        for (int i = 0; i < AHEAD; i++) fetch(ring[i], i);   // steps past the end read the row's first columns; never used
+        int step = 0;
+        for (; step + AHEAD <= steps; step += AHEAD) {
+#pragma unroll
+            for (int i = 0; i < AHEAD; i++) {
+                use(ring[i], step + i);
+                fetch(ring[i], step + i + AHEAD);
+            }
         }
 #pragma unroll
-        for (int r = 0; r < kRowsPerWave; r++) acc[r] = wave_sum(acc[r]) * scale;
+        for (int i = 0; i < AHEAD; i++)
+            if (step + i < steps) use(ring[i], step + i);
+#pragma unroll
+        for (int r = 0; r < RPW; r++) acc[r] = wave_sum(acc[r]) * scale;
         if (lane != 0) continue;
         if constexpr (KIND == KIND_IN) {
             if (!second) {
-                *reinterpret_cast<float4 *>(a.y + row0) = make_float4(acc[0], acc[1], acc[2], acc[3]);
+#pragma unroll
+                for (int r = 0; r < RPW; r++) a.y[row0 + r] = acc[r];
             } else {
                 const int i = (row0 - a.mix_rows) / 2;
-                *reinterpret_cast<float2 *>(a.act_out + i) = make_float2(matrix::silu(acc[0]) * acc[1], matrix::silu(acc[2]) * acc[3]);
+#pragma unroll
+                for (int r = 0; r + 1 < RPW; r += 2) a.act_out[i + r / 2] = matrix::silu(acc[r]) * acc[r + 1];
             }
         } else if constexpr (KIND == KIND_OUT) {
-            const float4 x = *reinterpret_cast<const float4 *>(a.residual + row0);
-            *reinterpret_cast<float4 *>(a.y + row0) = make_float4(x.x + a.mult * acc[0], x.y + a.mult * acc[1], x.z + a.mult * acc[2], x.w + a.mult * acc[3]);
+#pragma unroll
+            for (int r = 0; r < RPW; r++) a.y[row0 + r] = a.residual[row0 + r] + a.mult * acc[r];
         } else {
 #pragma unroll
-            for (int r = 0; r < kRowsPerWave; r++)
-                if (row0 + r < a.vocab) a.y[row0 + r] = a.cap > 0.0f ? a.cap * tanhf(acc[r] / a.cap) : acc[r];
+            for (int r = 0; r < RPW; r++) {
+                if (row0 + r >= a.vocab) continue;
+                const float v = a.cap > 0.0f ? a.cap * tanhf(acc[r] / a.cap) : acc[r];
+                if (a.y) a.y[row0 + r] = v;
+                if (v > best) { best = v; best_row = row0 + r; }   // rows ascend: the first of equal logits stays
+            }
+        }
+    }
+    if constexpr (KIND == KIND_HEAD) {
+        __shared__ float bv[kGemvWaves];
+        __shared__ int bi[kGemvWaves];
+        if (!a.best_value) return;
+        if (lane == 0) { bv[wave] = best; bi[wave] = best_row; }
+        __syncthreads();
+        if (tid == 0) {
+            for (int w = 1; w < kGemvWaves; w++)
+                if (bv[w] > best || (bv[w] == best && bi[w] < best_row)) { best = bv[w]; best_row = bi[w]; }
+            a.best_value[blockIdx.x] = best;
+            a.best_index[blockIdx.x] = best_row;
         }
     }
 }
@@ -157,55 +192,64 @@ int resident_workgroups() {
     return n;
 }
 
-template <int KIND>
-hipError_t run(const DenseGemvArgs &a, int grid, hipStream_t s) {
+template <int KIND, int RPW, int AHEAD>
+hipError_t run(DenseGemvArgs a, int grid, hipStream_t s) {
     const size_t lds = (size_t)(a.k_pad + a.heads) * 4;
     if (lds > 150 * 1024 || grid < 1) return hipErrorInvalidValue;
     static size_t allowed = 0;
     if (lds > 48 * 1024 && lds > allowed) {
-        const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void *>(&dense_gemv_kernel<KIND>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+        const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void *>(&dense_gemv_kernel<KIND, RPW, AHEAD>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
         if (e != hipSuccess) return e;
         allowed = lds;
     }
-    hipLaunchKernelGGL((dense_gemv_kernel<KIND>), dim3(grid), dim3(kGemvThreads), lds, s, a);
+    hipLaunchKernelGGL((dense_gemv_kernel<KIND, RPW, AHEAD>), dim3(grid), dim3(kGemvThreads), lds, s, a);
     return hipGetLastError();
 }
 int round_up(int v, int to) { return (v + to - 1) / to * to; }
+int at_most(int units) { return units < resident_workgroups() ? units : resident_workgroups(); }
 
 }  // namespace
 
 hipError_t launch_dense_gemv_in(const DenseGemvIn &p, hipStream_t s) {
-    if (!p.w.w || p.w.ld % 64 || p.mix_rows % kUnitRows || p.w.rows % kUnitRows || p.w.rows < p.mix_rows || p.mix_rows < kUnitRows) return hipErrorInvalidValue;
+    if (!p.w.w || p.w.ld % 64 || p.mix_rows % kRowAlign || p.w.rows % kRowAlign || p.w.rows < p.mix_rows || p.mix_rows < kRowAlign) return hipErrorInvalidValue;
     DenseGemvArgs a{};
-    a.w = p.w.w; a.ld = p.w.ld; a.k_pad = round_up(p.w.ld, kStep);
-    a.units_a = p.mix_rows / kUnitRows; a.units_b = (p.w.rows - p.mix_rows) / kUnitRows; a.mix_rows = p.mix_rows;
-    const int units = a.units_a + a.units_b, wanted = units < resident_workgroups() ? units : resident_workgroups();
+    a.w = p.w.w; a.ld = p.w.ld; a.k_pad = round_up(p.w.ld, kStep); a.mix_rows = p.mix_rows;
+    a.x = p.x; a.norm_a = p.norm1; a.norm_b = p.norm2; a.width = p.width; a.eps = p.eps; a.y = p.y; a.act_out = p.act;
+    const int unit = p.w.rows >= resident_workgroups() * kGemvWaves * 4 ? kGemvWaves * 4 : kGemvWaves * 2;   // (gate, up) pairs stay together
+    a.units_a = p.mix_rows / unit; a.units_b = (p.w.rows - p.mix_rows) / unit;
+    const int units = a.units_a + a.units_b, wanted = at_most(units);
     a.blocks_a = (int)((long long)wanted * a.units_a / units);
     if (a.blocks_a < 1) a.blocks_a = 1;
     int grid = wanted;
     if (a.units_b == 0) a.blocks_a = grid;
     else if (a.blocks_a >= grid) grid = a.blocks_a + 1;
-    a.x = p.x; a.norm_a = p.norm1; a.norm_b = p.norm2; a.width = p.width; a.eps = p.eps; a.y = p.y; a.act_out = p.act;
-    return run<KIND_IN>(a, grid, s);
+    return unit == kGemvWaves * 4 ? run<KIND_IN, 4, 2>(a, grid, s) : run<KIND_IN, 2, 3>(a, grid, s);
 }
 
 hipError_t launch_dense_gemv_out(const DenseGemvOut &p, hipStream_t s) {
-    if (!p.w.w || p.w.ld % 64 || p.rows % kUnitRows || p.w.rows < p.rows || p.mix_cols % 32 || p.act_cols % 32 || p.act_at < p.mix_cols || p.act_at + p.act_cols > p.w.ld || p.rows < kUnitRows)
+    if (!p.w.w || p.w.ld % 64 || p.rows % kRowAlign || p.w.rows < p.rows || p.mix_cols % 32 || p.act_cols % 32 || p.act_at < p.mix_cols || p.act_at + p.act_cols > p.w.ld || p.rows < kRowAlign)
         return hipErrorInvalidValue;
     if (p.squares && (p.vdim_p <= 0 || p.mix_cols % p.vdim_p || !p.gate)) return hipErrorInvalidValue;
     DenseGemvArgs a{};
-    a.w = p.w.w; a.ld = p.w.ld; a.k_pad = round_up(p.w.ld, kStep); a.units_a = p.rows / kUnitRows;
+    a.w = p.w.w; a.ld = p.w.ld; a.k_pad = round_up(p.w.ld, kStep);
     a.mix = p.mix; a.act = p.act; a.squares = p.squares; a.gate = p.gate; a.mix_cols = p.mix_cols; a.act_at = p.act_at; a.act_cols = p.act_cols; a.parts = p.parts;
     a.heads = p.squares ? p.mix_cols / p.vdim_p : 0; a.vdim = p.vdim; a.vdim_p = p.vdim_p; a.eps = p.eps; a.mult = p.mult; a.residual = p.residual; a.y = p.out;
-    return run<KIND_OUT>(a, a.units_a < resident_workgroups() ? a.units_a : resident_workgroups(), s);
+    const int cus = resident_workgroups() / 2;   // long rows: a workgroup per compute unit
+    if (p.rows >= cus * kGemvWaves * 4) { a.units_a = p.rows / (kGemvWaves * 4); return run<KIND_OUT, 4, 2>(a, at_most(a.units_a), s); }
+    if (p.rows >= cus * kGemvWaves * 2) { a.units_a = p.rows / (kGemvWaves * 2); return run<KIND_OUT, 2, 4>(a, at_most(a.units_a), s); }
+    a.units_a = p.rows / kGemvWaves;
+    return run<KIND_OUT, 1, 6>(a, at_most(a.units_a), s);
 }
 
+int dense_gemv_head_workgroups(const DenseMatrix &w) { return at_most(w.rows / (kGemvWaves * 4)); }
+
 hipError_t launch_dense_gemv_head(const DenseGemvHead &p, hipStream_t s) {
-    if (!p.w.w || p.w.ld % 64 || p.w.rows % kUnitRows || p.vocab > p.w.rows || p.vocab < 1) return hipErrorInvalidValue;
+    if (!p.w.w || p.w.ld % 64 || p.w.rows % kRowAlign || p.vocab > p.w.rows || p.vocab < 1 || (!p.logits && !p.best_value) || (p.best_value && !p.best_index)) return hipErrorInvalidValue;
     DenseGemvArgs a{};
-    a.w = p.w.w; a.ld = p.w.ld; a.k_pad = round_up(p.w.ld, kStep); a.units_a = p.w.rows / kUnitRows;
+    a.w = p.w.w; a.ld = p.w.ld; a.k_pad = round_up(p.w.ld, kStep); a.units_a = p.w.rows / (kGemvWaves * 4);
     a.x = p.x; a.norm_a = p.norm; a.width = p.width; a.eps = p.eps; a.vocab = p.vocab; a.cap = p.cap; a.y = p.logits;
-    return run<KIND_HEAD>(a, a.units_a < resident_workgroups() ? a.units_a : resident_workgroups(), s);
+    a.best_value = p.best_value; a.best_index = p.best_index;
+    return run<KIND_HEAD, 4, 2>(a, dense_gemv_head_workgroups(p.w), s);
 }
 
 }  // namespace esp

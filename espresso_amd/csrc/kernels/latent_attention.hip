@@ -4,13 +4,13 @@
 //   cached row: [latent c (rank_p) | rotated key part (rot_p)], one per token, at position % ring
 //   score_h(i, j) = ((q_h . W_uk_h c_j) + q_rot_h . k_rot_j) scale,   value_h(j) = W_uv_h c_j
 //
-// Decode (launch_latent_step, three launches): the query goes through W_uk^T once instead of every key through W_uk, so a head's
+// Decode (launch_latent_step, three launches; the first also stores the row's own latent): the query goes through W_uk^T once instead of every key through W_uk, so a head's
 // query is a row of rank_p + rot_p values against the cached rows themselves, and the weighted sum stays in the latent space until
 // one product with W_uv.  All heads share the cached rows: 32 heads are the 32 columns of the matrix-core tile.  Slices of the
 // window go to different workgroups, which leave (maximum, sum, weighted latents); the merge adds the sink once.
 //
 // Prompt blocks (launch_latent_block): keys and values of the visible span are products of the gathered latents (done by the
-// caller as two dense products, values transposed), then attention in tiles of 64 keys: a wavefront owns 32 queries; scores are
+// caller as two dense products, values transposed), then attention in tiles of 64 keys: a wavefront owns 32 queries and half of every tile; scores are
 // computed transposed (keys as rows), so a lane holds one query's column, the softmax needs one exchange between the lane halves,
 // and the weights are the B operand of the value product without passing through LDS.
 // With bf16 operands queries of the decode form and softmax weights enter the products as a high and a low bf16.
@@ -33,24 +33,48 @@ __device__ __forceinline__ float rotated_pairs(const float *x, int i, int dims, 
     return (i & 1) ? v * c + u * s : u * c - v * s;
 }
 
+// Row m's latent (normed) and rotated key part into the cache, by a workgroup of 256 threads.
+template <typename T>
+__device__ __forceinline__ void store_latent(const LatentShape &l, const float *mixed, const int *pos, const int *seq, int m, float *red) {
+    const int p = pos[m], width = l.rank_p + l.rot_p;
+    const float *c = mixed + (size_t)m * l.ld_mix + l.dkv_at;
+    constexpr int kHeld = 4;
+    static_assert(kHeld * 256 >= kLatentMaxRank, "a latent is held in registers");
+    float held[kHeld], s = 0.0f;
+#pragma unroll
+    for (int k = 0; k < kHeld; k++) {
+        const int i = threadIdx.x + k * 256;
+        held[k] = i < l.rank_p ? c[i] : 0.0f;
+    }
+#pragma unroll
+    for (int k = 0; k < kHeld; k++) s += held[k] * held[k];
+    const float inv = 1.0f / sqrtf(detail::workgroup_sum(s, red) / (float)l.kv_rank + l.eps);
+    T *row = static_cast<T *>(l.cache) + ((size_t)seq[m] * l.ring + p % l.ring) * width;
+#pragma unroll
+    for (int k = 0; k < kHeld; k++) {
+        const int i = threadIdx.x + k * 256;
+        if (i < l.rank_p) row[i] = Op<T>::from_float(held[k] * inv * l.latent_norm[i]);
+    }
+    const size_t at = (size_t)p * (l.rot_dims / 2);
+    for (int i = threadIdx.x; i < l.rot_p; i += 256) row[l.rank_p + i] = Op<T>::from_float(rotated_pairs(c + l.rank_p, i, l.rot_dims, l.cos + at, l.sin + at));
+}
+
 template <typename T>
 __global__ __launch_bounds__(256) void latent_store_kernel(LatentShape l, const float *mixed, const int *pos, const int *seq) {
     __shared__ float red[4];
-    const int m = blockIdx.x, p = pos[m], width = l.rank_p + l.rot_p;
-    const float *c = mixed + (size_t)m * l.ld_mix + l.dkv_at;
-    float s = 0.0f;
-    for (int i = threadIdx.x; i < l.rank_p; i += 256) s += c[i] * c[i];
-    const float inv = 1.0f / sqrtf(detail::workgroup_sum(s, red) / (float)l.kv_rank + l.eps);
-    T *row = static_cast<T *>(l.cache) + ((size_t)seq[m] * l.ring + p % l.ring) * width;
-    const size_t at = (size_t)p * (l.rot_dims / 2);
-    for (int i = threadIdx.x; i < width; i += 256)
-        row[i] = Op<T>::from_float(i < l.rank_p ? c[i] * inv * l.latent_norm[i] : rotated_pairs(c + l.rank_p, i - l.rank_p, l.rot_dims, l.cos + at, l.sin + at));
+    store_latent<T>(l, mixed, pos, seq, blockIdx.x, red);
 }
 
-// absorbed[m][h] = scale * [W_uk_h^T q_h | rotated part]; grid (chunks of 128 ranks, heads, rows)
+// absorbed[m][h] = scale * [W_uk_h^T q_h | rotated part]; grid (chunks of 128 ranks, heads, rows), and one more workgroup per row
+// (y = heads, x = 0) that stores the row's own latent where the layer has one.
+template <typename T>
 __global__ __launch_bounds__(256) void latent_absorb_kernel(LatentShape l, LatentStep p) {
     extern __shared__ float lds[];   // q [dim_p], partial sums [16][128]
     const int tid = threadIdx.x, c0 = blockIdx.x * 128, h = blockIdx.y, m = blockIdx.z, qk = l.dim_p + l.rot_p;
+    if (h == l.heads) {
+        if (blockIdx.x == 0) store_latent<T>(l, p.mixed, p.pos, p.seq, m, lds);
+        return;
+    }
     const float *q = p.mixed + (size_t)m * l.ld_mix + h * qk;
     float *out = p.absorbed + ((size_t)m * l.heads + h) * (l.rank_p + l.rot_p);
     for (int i = tid; i < l.dim_p; i += 256) lds[i] = q[i];
@@ -63,12 +87,19 @@ __global__ __launch_bounds__(256) void latent_absorb_kernel(LatentShape l, Laten
     float acc[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
     if (col < l.rank_p) {
         const uint16_t *w = l.uk + (size_t)h * l.dim_p * l.rank_p + col;
-        for (int d = g; d < l.dim_p; d += 16) {
-            float f[8];
-            matrix::unpack_bf16(*reinterpret_cast<const uint4 *>(w + (size_t)d * l.rank_p), f);
-            const float x = lds[d];
+        for (int d0 = g; d0 < l.dim_p; d0 += 16 * 4) {   // four rows of W_uk in flight
+            uint4 v[4];
 #pragma unroll
-            for (int i = 0; i < 8; i++) acc[i] = __builtin_fmaf(f[i], x, acc[i]);
+            for (int u = 0; u < 4; u++) v[u] = *reinterpret_cast<const uint4 *>(w + (size_t)(d0 + 16 * u < l.dim_p ? d0 + 16 * u : g) * l.rank_p);
+#pragma unroll
+            for (int u = 0; u < 4; u++) {
+                if (d0 + 16 * u >= l.dim_p) continue;
+                float f[8];
+                matrix::unpack_bf16(v[u], f);
+                const float x = lds[d0 + 16 * u];
+#pragma unroll
+                for (int i = 0; i < 8; i++) acc[i] = __builtin_fmaf(f[i], x, acc[i]);
+            }
         }
     }
     float *sums = lds + l.dim_p;
@@ -87,54 +118,100 @@ __global__ __launch_bounds__(256) void latent_absorb_kernel(LatentShape l, Laten
 __device__ __forceinline__ int first_seen(int pos, int window) { return pos - window + 1 > 0 ? pos - window + 1 : 0; }
 
 template <typename T>
-struct PartialLayout {   // LDS of latent_partial_kernel
+struct PartialLayout {   // LDS of latent_partial_kernel: a tile of 32 cached rows, the scores of four wavefronts
     static constexpr int kPad = 16 / sizeof(T);
-    static size_t bytes(int width, bool queries) { return (size_t)32 * (width + kPad) * sizeof(T) + (size_t)4 * 32 * 33 * 4 + (queries ? (size_t)32 * (width + 4) * 4 : 0); }
+    static size_t bytes(int width) { return (size_t)32 * (width + kPad) * sizeof(T) + (size_t)4 * 32 * 33 * 4; }
 };
+typedef uint32_t uintx4 __attribute__((ext_vector_type(4)));
 
-// grid (splits, groups of 32 heads, rows); NT: tiles of 32 ranks per wavefront
-template <typename T, int NT>
-__global__ __launch_bounds__(256) void latent_partial_kernel(LatentShape l, LatentStep p, int queries_in_lds) {
+// Products and exponentials of scores: bf16 models use the hardware's exponential directly.
+template <typename T>
+__device__ __forceinline__ float weight_exp(float x) {
+    if constexpr (Op<T>::kSplit) return __expf(x);
+    else return expf(x);
+}
+
+// grid (splits, groups of 32 heads, rows).  NT: tiles of 32 ranks per wavefront.  KS: rows of up to 64 KS values have their queries
+// and the next tile in registers (KS steps of 16 per wavefront, KS pieces of eight per thread); 0: any width, from memory as needed.
+template <typename T, int NT, int KS>
+__global__ __launch_bounds__(256) void latent_partial_kernel(LatentShape l, LatentStep p) {
     extern __shared__ char smem[];
-    const int width = l.rank_p + l.rot_p, ldc = width + PartialLayout<T>::kPad, ldq = width + 4;
+    constexpr int kVec = sizeof(T) / 2;   // 128-bit words per piece
+    const int width = l.rank_p + l.rot_p, ldc = width + PartialLayout<T>::kPad;
     T *tile = reinterpret_cast<T *>(smem);
-    float *scores = reinterpret_cast<float *>(tile + 32 * ldc), *queries = scores + 4 * 32 * 33;
+    float *scores = reinterpret_cast<float *>(tile + 32 * ldc);
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, half = lane >> 5, col = lane & 31;
     const int split = blockIdx.x, m = blockIdx.z, pos = p.pos[m];
     const int lo = first_seen(pos, l.window), tiles = (pos - lo) / 32 + 1;
     if (split >= tiles) return;
     const int head = blockIdx.y * 32 + col, head_in = head < l.heads ? head : l.heads - 1;   // columns past the heads repeat the last one
-    const float *q_row = p.absorbed + ((size_t)m * l.heads + head_in) * width;
-    if (queries_in_lds) {
-        for (int i = tid * 4; i < 32 * width; i += 256 * 4) {
-            const int hh = i / width, k = i % width, hs = blockIdx.y * 32 + hh < l.heads ? blockIdx.y * 32 + hh : l.heads - 1;
-            *reinterpret_cast<float4 *>(queries + hh * ldq + k) = *reinterpret_cast<const float4 *>(p.absorbed + ((size_t)m * l.heads + hs) * width + k);
-        }
-        q_row = queries + col * ldq;
-    }
+    const float *q_row = p.absorbed + ((size_t)m * l.heads + head_in) * width + 8 * half;
     const T *cache = static_cast<const T *>(l.cache) + (size_t)p.seq[m] * l.ring * width;
+    const int pieces = width / 8, steps = width / 16;
+    auto row_piece = [&](int k0, int i) {   // piece i of the tile at k0; rows past the query repeat it and are masked below
+        const int row = i / pieces, part = i % pieces, key = k0 + row < pos ? k0 + row : pos;
+        return reinterpret_cast<const uintx4 *>(cache + (size_t)(key % l.ring) * width + part * 8);
+    };
+    auto tile_piece = [&](int i) { return reinterpret_cast<uintx4 *>(tile + i / pieces * ldc + i % pieces * 8); };
+    uintx4 ahead[KS ? KS * kVec : 1];
+    auto fetch = [&](int t) {
+        if constexpr (KS > 0) {
+#pragma unroll
+            for (int k = 0; k < KS; k++) {
+                const int i = tid + k * 256;
+                const uintx4 *src = row_piece(lo + t * 32, i < 32 * pieces ? i : 0);
+#pragma unroll
+                for (int v = 0; v < kVec; v++) ahead[k * kVec + v] = src[v];
+            }
+        }
+    };
+    fetch(split);
+    float qv[KS ? KS : 1][8];
+    if constexpr (KS > 0) {
+#pragma unroll
+        for (int k = 0; k < KS; k++) {
+            const int ks = wave + 4 * k < steps ? wave + 4 * k : 0;
+            const float4 q0 = reinterpret_cast<const float4 *>(q_row + ks * 16)[0], q1 = reinterpret_cast<const float4 *>(q_row + ks * 16)[1];
+            qv[k][0] = q0.x; qv[k][1] = q0.y; qv[k][2] = q0.z; qv[k][3] = q0.w; qv[k][4] = q1.x; qv[k][5] = q1.y; qv[k][6] = q1.z; qv[k][7] = q1.w;
+        }
+    }
     float top = -INFINITY, sum = 0.0f;
     floatx16 acc[NT];
 #pragma unroll
     for (int i = 0; i < NT; i++) acc[i] = matrix::zero_accumulator();
-    const int pieces = width / 8;
     for (int t = split; t < tiles; t += p.splits) {
         const int k0 = lo + t * 32;
         __syncthreads();
-        for (int i = tid; i < 32 * pieces; i += 256) {
-            const int row = i / pieces, part = i % pieces, key = k0 + row < pos ? k0 + row : pos;   // rows past the query repeat it; masked below
-            const uint4 *src = reinterpret_cast<const uint4 *>(cache + (size_t)(key % l.ring) * width + part * 8);
-            uint4 *dst = reinterpret_cast<uint4 *>(tile + row * ldc + part * 8);
-            dst[0] = src[0];
-            if constexpr (sizeof(T) == 4) dst[1] = src[1];
+        if constexpr (KS > 0) {
+#pragma unroll
+            for (int k = 0; k < KS; k++) {
+                const int i = tid + k * 256;
+                if (i < 32 * pieces) {
+#pragma unroll
+                    for (int v = 0; v < kVec; v++) tile_piece(i)[v] = ahead[k * kVec + v];
+                }
+            }
+            if (t + p.splits < tiles) fetch(t + p.splits);
+        } else {
+            for (int i = tid; i < 32 * pieces; i += 256) {
+                const uintx4 *src = row_piece(k0, i);
+#pragma unroll
+                for (int v = 0; v < kVec; v++) tile_piece(i)[v] = src[v];
+            }
         }
         __syncthreads();
         floatx16 s = matrix::zero_accumulator();
-        for (int ks = wave; ks < width / 16; ks += 4) {
-            const float *qp = q_row + ks * 16 + 8 * half;
-            const float4 q0 = reinterpret_cast<const float4 *>(qp)[0], q1 = reinterpret_cast<const float4 *>(qp)[1];
-            const float f[8] = {q0.x, q0.y, q0.z, q0.w, q1.x, q1.y, q1.z, q1.w};
-            s = matrix::mma_values<T>(Op<T>::load(tile + col * ldc + ks * 16 + 8 * half), f, s);
+        const T *key_row = tile + col * ldc + 8 * half;
+        if constexpr (KS > 0) {
+#pragma unroll
+            for (int k = 0; k < KS; k++)
+                if (wave + 4 * k < steps) s = matrix::mma_values<T>(Op<T>::load(key_row + (wave + 4 * k) * 16), qv[k], s);
+        } else {
+            for (int ks = wave; ks < steps; ks += 4) {
+                const float4 q0 = reinterpret_cast<const float4 *>(q_row + ks * 16)[0], q1 = reinterpret_cast<const float4 *>(q_row + ks * 16)[1];
+                const float f[8] = {q0.x, q0.y, q0.z, q0.w, q1.x, q1.y, q1.z, q1.w};
+                s = matrix::mma_values<T>(Op<T>::load(key_row + ks * 16), f, s);
+            }
         }
 #pragma unroll
         for (int r = 0; r < 16; r++) scores[(wave * 32 + matrix::accumulator_row(r, half)) * 33 + col] = s[r];
@@ -148,10 +225,10 @@ __global__ __launch_bounds__(256) void latent_partial_kernel(LatentShape l, Late
             best = fmaxf(best, w[r]);
         }
         best = fmaxf(fmaxf(best, __shfl_xor(best, 32)), top);
-        const float keep = expf(top - best);
+        const float keep = weight_exp<T>(top - best);
         float add = 0.0f;
 #pragma unroll
-        for (int r = 0; r < 16; r++) { w[r] = expf(w[r] - best); add += w[r]; }
+        for (int r = 0; r < 16; r++) { w[r] = weight_exp<T>(w[r] - best); add += w[r]; }
         add += __shfl_xor(add, 32);
         sum = sum * keep + add;
         top = best;
@@ -187,44 +264,65 @@ __global__ __launch_bounds__(256) void latent_partial_kernel(LatentShape l, Late
     if (wave == 0 && half == 0) *reinterpret_cast<float2 *>(p.partial_ml + at * 2) = make_float2(top, sum);
 }
 
-// Slices of a head merged with its sink, then 32 rows of W_uv and the gate; grid (vdim_p / 32, heads, rows)
+// Slices of a head merged with its sink, then 32 rows of W_uv and the gate; grid (vdim_p / 32, heads, rows).  splits <= 64: a lane
+// of the first wavefront each.
 template <typename T>
 __global__ __launch_bounds__(256) void latent_merge_kernel(LatentShape l, LatentStep p) {
-    extern __shared__ float lds[];   // merged latents [rank_p], weights [splits]
+    extern __shared__ float lds[];   // merged latents [rank_p], weights [64]
     const int tid = threadIdx.x, h = blockIdx.y, m = blockIdx.z, pos = p.pos[m];
     const int tiles = (pos - first_seen(pos, l.window)) / 32 + 1, live = tiles < p.splits ? tiles : p.splits;
     const size_t first = (size_t)m * p.splits * l.heads + h;   // slice s: first + s * heads
-    const float sink = l.sink[h];
-    float top = sink, sum = 0.0f;
-    for (int s = 0; s < live; s++) top = fmaxf(top, p.partial_ml[(first + (size_t)s * l.heads) * 2]);
-    for (int s = 0; s < live; s++) {
-        const float2 ml = *reinterpret_cast<const float2 *>(p.partial_ml + (first + (size_t)s * l.heads) * 2);
-        const float w = expf(ml.x - top);
-        sum += w * ml.y;
-        if (tid == 0) lds[l.rank_p + s] = w;
+    if (tid < 64) {
+        const float sink = l.sink[h];
+        const float2 ml = *reinterpret_cast<const float2 *>(p.partial_ml + (first + (size_t)(tid < live ? tid : 0) * l.heads) * 2);
+        float top = fmaxf(ml.x, sink);
+#pragma unroll
+        for (int x = 32; x >= 1; x >>= 1) top = fmaxf(top, __shfl_xor(top, x));
+        const float w = tid < live ? expf(ml.x - top) : 0.0f;
+        const float sum = detail::wave_sum(w * ml.y) + expf(sink - top);
+        lds[l.rank_p + tid] = w / sum;
     }
-    const float inv = 1.0f / (sum + expf(sink - top));
-    __syncthreads();
-    for (int r = tid; r < l.rank_p; r += 256) {
-        float v = 0.0f;
-        for (int s = 0; s < live; s++) v += lds[l.rank_p + s] * p.partial[(first + (size_t)s * l.heads) * l.rank_p + r];
-        lds[r] = v * inv;
-    }
-    __syncthreads();
+    // W_uv's row and the gate are on their way meanwhile
     const int e = tid & 7, j = blockIdx.x * 32 + (tid >> 3);
     const uint16_t *w = l.uv + ((size_t)h * l.vdim_p + j) * l.rank_p;
+    constexpr int kHeld = 8;
+    uint4 row[kHeld];
+#pragma unroll
+    for (int i = 0; i < kHeld; i++) row[i] = *reinterpret_cast<const uint4 *>(w + (e * 8 + i * 64 < l.rank_p ? e * 8 + i * 64 : 0));
+    const float gate = p.mixed[(size_t)m * l.ld_mix + l.gate_at + h];
+    __syncthreads();
+    for (int r = tid * 4; r < l.rank_p; r += 256 * 4) {
+        float4 v = make_float4(0.f, 0.f, 0.f, 0.f);
+        for (int s0 = 0; s0 < live; s0 += 8) {   // eight slices in flight
+            float4 x[8];
+#pragma unroll
+            for (int u = 0; u < 8; u++) x[u] = *reinterpret_cast<const float4 *>(p.partial + (first + (size_t)(s0 + u < live ? s0 + u : 0) * l.heads) * l.rank_p + r);
+#pragma unroll
+            for (int u = 0; u < 8; u++) {
+                if (s0 + u >= live) continue;
+                const float f = lds[l.rank_p + s0 + u];
+                v.x += f * x[u].x; v.y += f * x[u].y; v.z += f * x[u].z; v.w += f * x[u].w;
+            }
+        }
+        *reinterpret_cast<float4 *>(lds + r) = v;
+    }
+    __syncthreads();
     float o = 0.0f;
-    for (int r = e * 8; r < l.rank_p; r += 64) {
+    auto add = [&](const uint4 &piece, int r) {
         float f[8];
-        matrix::unpack_bf16(*reinterpret_cast<const uint4 *>(w + r), f);
+        matrix::unpack_bf16(piece, f);
 #pragma unroll
         for (int i = 0; i < 8; i++) o = __builtin_fmaf(f[i], lds[r + i], o);
-    }
+    };
+#pragma unroll
+    for (int i = 0; i < kHeld; i++)
+        if (e * 8 + i * 64 < l.rank_p) add(row[i], e * 8 + i * 64);
+    for (int r = e * 8 + kHeld * 64; r < l.rank_p; r += 64) add(*reinterpret_cast<const uint4 *>(w + r), r);
     o += detail::dpp_term<0xB1, 0xF>(o);
     o += detail::dpp_term<0x4E, 0xF>(o);
     o += detail::dpp_term<0x141, 0xF>(o);
     if (e != 0) return;
-    o *= matrix::sigmoid(p.mixed[(size_t)m * l.ld_mix + l.gate_at + h]);
+    o *= matrix::sigmoid(gate);
     if (p.mix) p.mix[(size_t)m * l.heads * l.vdim_p + h * l.vdim_p + j] = o;
     else static_cast<T *>(p.act)[(size_t)m * p.ld_act + h * l.vdim_p + j] = Op<T>::from_float(o);
 }
@@ -254,91 +352,109 @@ __global__ __launch_bounds__(256) void latent_queries_kernel(LatentShape l, Late
     }
 }
 
-constexpr int kQueries = 128, kKeys = 64, kValues = 128;   // per workgroup and tile
+constexpr int kQueries = 64, kKeys = 64, kValues = 128;   // per workgroup and tile
 template <typename T>
 struct BlockLayout {
     static constexpr int kPad = 16 / sizeof(T);
-    static size_t bytes(int qk) { return ((size_t)kKeys * (qk + kPad) + (size_t)kValues * (kKeys + kPad)) * sizeof(T); }
+    static size_t bytes(int qk) {
+        const size_t tiles = ((size_t)kKeys * (qk + kPad) + (size_t)kValues * (kKeys + kPad)) * sizeof(T), merge = (size_t)2 * 64 * 66 * 4;
+        return tiles > merge ? tiles : merge;
+    }
 };
 
-// grid (blocks of 128 queries, heads, slices of 128 values); NQ: steps of 16 query dimensions held in registers, 0 = read again
+// grid (blocks of 64 queries, heads, slices of 128 values).  Wavefront w takes queries 32 (w % 2) .. and, of every tile of 64 keys, keys
+// 32 (w / 2) ..; the two halves' softmax states meet in LDS at the end.  NQ: steps of 16 query dimensions held in registers (the next
+// tile too), 0 = any number, read when needed.
 template <typename T, int NQ>
 __global__ __launch_bounds__(256) void latent_block_kernel(LatentShape l, LatentBlock p, int rows_p) {
     extern __shared__ char smem[];
-    constexpr int kPad = BlockLayout<T>::kPad, LDV = kKeys + kPad;
+    constexpr int kPad = BlockLayout<T>::kPad, LDV = kKeys + kPad, kVec = sizeof(T) / 2;
+    constexpr int PK = NQ ? NQ / 2 : 1, PV = kValues * kKeys / 8 / 256;   // pieces of eight per thread: keys (64 rows of 2 NQ pieces), values
     const int qk = l.dim_p + l.rot_p, ldk = qk + kPad;
     T *kt = reinterpret_cast<T *>(smem), *vt = kt + kKeys * ldk;
-    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, half = lane >> 5, col = lane & 31;
+    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, half = lane >> 5, col = lane & 31, qt = wave & 1, set = wave >> 1;
     const int h = blockIdx.y, q0 = blockIdx.x * kQueries, v0 = blockIdx.z * kValues;
     const int values = l.vdim_p - v0 < kValues ? l.vdim_p - v0 : kValues;
-    const int m = q0 + wave * 32 + col, at = p.base - p.first_key + m;   // this lane's query: row and place among the keys
-    const int wave_at = p.base - p.first_key + q0 + wave * 32;           // the wavefront's first query
+    const int m = q0 + qt * 32 + col, at = p.base - p.first_key + m;   // this lane's query: row and place among the keys
+    const int wave_at = p.base - p.first_key + q0 + qt * 32;           // the wavefront's first query
+    const int block_at = p.base - p.first_key + q0, seen = block_at - l.window + 1;
+    const int k_begin = seen > 0 ? seen / kKeys * kKeys : 0;
+    const int last = q0 + kQueries < p.rows ? q0 + kQueries : p.rows, k_end = p.base - p.first_key + last;
+    const int row_pieces = l.dim_p / 8, k_pieces = row_pieces + l.rot_p / 8;
+    const T *keys = static_cast<const T *>(p.k) + h * l.dim_p, *key_rot = static_cast<const T *>(p.key_rot);
+    const T *vals = static_cast<const T *>(p.vt) + ((size_t)h * l.vdim_p + v0) * p.keys_p;
+    auto key_piece = [&](int k0, int i) {
+        const int row = i / k_pieces, part = i % k_pieces;
+        return reinterpret_cast<const uintx4 *>(part < row_pieces ? keys + (size_t)(k0 + row) * l.heads * l.dim_p + part * 8 : key_rot + (size_t)(k0 + row) * l.rot_p + (part - row_pieces) * 8);
+    };
+    auto value_piece = [&](int k0, int i) { return reinterpret_cast<const uintx4 *>(vals + (size_t)(i / (kKeys / 8)) * p.keys_p + k0 + i % (kKeys / 8) * 8); };
+    auto key_place = [&](int i) { return reinterpret_cast<uintx4 *>(kt + i / k_pieces * ldk + i % k_pieces * 8); };
+    auto value_place = [&](int i) { return reinterpret_cast<uintx4 *>(vt + i / (kKeys / 8) * LDV + i % (kKeys / 8) * 8); };
+    const int n_key = kKeys * k_pieces, n_value = values * (kKeys / 8);
+    uintx4 ahead_k[PK], ahead_v[NQ ? PV : 1];   // bf16 only: one word per piece
+    auto fetch = [&](int k0) {
+        if constexpr (NQ > 0) {
+#pragma unroll
+            for (int i = 0; i < PK; i++) ahead_k[i] = *key_piece(k0, tid + i * 256 < n_key ? tid + i * 256 : 0);
+#pragma unroll
+            for (int i = 0; i < PV; i++) ahead_v[i] = *value_piece(k0, tid + i * 256 < n_value ? tid + i * 256 : 0);
+        }
+    };
+    fetch(k_begin);
     const T *q = static_cast<const T *>(p.q) + ((size_t)h * rows_p + (m < rows_p ? m : rows_p - 1)) * qk + 8 * half;
     typename Op<T>::frag qf[NQ ? NQ : 1];
     if constexpr (NQ > 0) {
 #pragma unroll
         for (int i = 0; i < NQ; i++) qf[i] = Op<T>::load(q + (i * 16 < qk ? i * 16 : 0));
     }
-    float top = l.sink[h], sum = 1.0f;   // the sink: one more term of the denominator, without a value
+    float top = l.sink[h], sum = set == 0 ? 1.0f : 0.0f;   // the sink: one more term of the denominator, without a value
     floatx16 out[4];
 #pragma unroll
     for (int i = 0; i < 4; i++) out[i] = matrix::zero_accumulator();
-    const int block_at = p.base - p.first_key + q0, seen = block_at - l.window + 1;
-    const int k_begin = seen > 0 ? seen / kKeys * kKeys : 0;
-    const int last = q0 + kQueries < p.rows ? q0 + kQueries : p.rows, k_end = p.base - p.first_key + last;
-    const int row_pieces = l.dim_p / 8, rot_pieces = l.rot_p / 8, k_pieces = row_pieces + rot_pieces;
-    const T *keys = static_cast<const T *>(p.k), *key_rot = static_cast<const T *>(p.key_rot), *vals = static_cast<const T *>(p.vt);
-    auto copy = [&](T *dst, const T *src) {
-        reinterpret_cast<uint4 *>(dst)[0] = reinterpret_cast<const uint4 *>(src)[0];
-        if constexpr (sizeof(T) == 4) reinterpret_cast<uint4 *>(dst)[1] = reinterpret_cast<const uint4 *>(src)[1];
-    };
     for (int k0 = k_begin; k0 < k_end; k0 += kKeys) {
         __syncthreads();
-        for (int i = tid; i < kKeys * k_pieces; i += 256) {
-            const int row = i / k_pieces, part = i % k_pieces;
-            copy(kt + row * ldk + part * 8, part < row_pieces ? keys + (size_t)(k0 + row) * l.heads * l.dim_p + h * l.dim_p + part * 8
-                                                               : key_rot + (size_t)(k0 + row) * l.rot_p + (part - row_pieces) * 8);
-        }
-        for (int i = tid; i < values * (kKeys / 8); i += 256) {
-            const int row = i / (kKeys / 8), part = i % (kKeys / 8);
-            copy(vt + row * LDV + part * 8, vals + ((size_t)h * l.vdim_p + v0 + row) * p.keys_p + k0 + part * 8);
-        }
-        __syncthreads();
-        if (k0 > wave_at + 31 || k0 + kKeys - 1 <= wave_at - l.window) continue;   // no query of this wavefront sees the tile
-        floatx16 s[2];
-        s[0] = s[1] = matrix::zero_accumulator();
-        const T *kp = kt + col * ldk + 8 * half;
         if constexpr (NQ > 0) {
 #pragma unroll
-            for (int i = 0; i < NQ; i++) {
-                if (i * 16 < qk) {
-                    s[0] = Op<T>::mma(Op<T>::load(kp + i * 16), qf[i], s[0]);
-                    s[1] = Op<T>::mma(Op<T>::load(kp + 32 * ldk + i * 16), qf[i], s[1]);
-                }
-            }
+            for (int i = 0; i < PK; i++)
+                if (tid + i * 256 < n_key) *key_place(tid + i * 256) = ahead_k[i];
+#pragma unroll
+            for (int i = 0; i < PV; i++)
+                if (tid + i * 256 < n_value) *value_place(tid + i * 256) = ahead_v[i];
+            if (k0 + kKeys < k_end) fetch(k0 + kKeys);
         } else {
-            for (int d = 0; d < qk; d += 16) {
-                const typename Op<T>::frag f = Op<T>::load(q + d);
-                s[0] = Op<T>::mma(Op<T>::load(kp + d), f, s[0]);
-                s[1] = Op<T>::mma(Op<T>::load(kp + 32 * ldk + d), f, s[1]);
+            for (int i = tid; i < n_key; i += 256) {
+#pragma unroll
+                for (int v = 0; v < kVec; v++) key_place(i)[v] = key_piece(k0, i)[v];
+            }
+            for (int i = tid; i < n_value; i += 256) {
+#pragma unroll
+                for (int v = 0; v < kVec; v++) value_place(i)[v] = value_piece(k0, i)[v];
             }
         }
-        float w[2][16], best = -INFINITY;
+        __syncthreads();
+        const int ks = k0 + set * 32;
+        if (ks > wave_at + 31 || ks + 31 <= wave_at - l.window) continue;   // no query of this wavefront sees these keys
+        floatx16 s = matrix::zero_accumulator();
+        const T *kp = kt + (set * 32 + col) * ldk + 8 * half;
+        if constexpr (NQ > 0) {
 #pragma unroll
-        for (int t = 0; t < 2; t++)
+            for (int i = 0; i < NQ; i++)
+                if (i * 16 < qk) s = Op<T>::mma(Op<T>::load(kp + i * 16), qf[i], s);
+        } else {
+            for (int d = 0; d < qk; d += 16) s = Op<T>::mma(Op<T>::load(kp + d), Op<T>::load(q + d), s);
+        }
+        float w[16], best = -INFINITY;
 #pragma unroll
-            for (int r = 0; r < 16; r++) {
-                const int gap = at - (k0 + t * 32 + matrix::accumulator_row(r, half));
-                w[t][r] = gap >= 0 && gap < l.window ? s[t][r] * l.scale : -INFINITY;
-                best = fmaxf(best, w[t][r]);
-            }
+        for (int r = 0; r < 16; r++) {
+            const int gap = at - (ks + matrix::accumulator_row(r, half));
+            w[r] = gap >= 0 && gap < l.window ? s[r] * l.scale : -INFINITY;
+            best = fmaxf(best, w[r]);
+        }
         best = fmaxf(fmaxf(best, __shfl_xor(best, 32)), top);
-        const float keep = expf(top - best);
+        const float keep = weight_exp<T>(top - best);
         float add = 0.0f;
 #pragma unroll
-        for (int t = 0; t < 2; t++)
-#pragma unroll
-            for (int r = 0; r < 16; r++) { w[t][r] = expf(w[t][r] - best); add += w[t][r]; }
+        for (int r = 0; r < 16; r++) { w[r] = weight_exp<T>(w[r] - best); add += w[r]; }
         add += __shfl_xor(add, 32);
         sum = sum * keep + add;
         top = best;
@@ -349,22 +465,33 @@ __global__ __launch_bounds__(256) void latent_block_kernel(LatentShape l, Latent
             for (int r = 0; r < 16; r++) out[i][r] *= keep;
         }
 #pragma unroll
-        for (int t = 0; t < 2; t++)
+        for (int st = 0; st < 2; st++) {
+            float f[8];
 #pragma unroll
-            for (int st = 0; st < 2; st++) {
-                float f[8];
+            for (int j = 0; j < 8; j++) f[j] = w[st * 8 + j];
 #pragma unroll
-                for (int j = 0; j < 8; j++) f[j] = w[t][st * 8 + j];
-#pragma unroll
-                for (int i = 0; i < 4; i++) {
-                    if (i * 32 >= values) continue;
-                    const T *vp = vt + (i * 32 + col) * LDV + t * 32 + st * 16 + 4 * half;
-                    out[i] = matrix::mma_values<T>(Op<T>::load_pair(vp, vp + 8), f, out[i]);
-                }
+            for (int i = 0; i < 4; i++) {
+                if (i * 32 >= values) continue;
+                const T *vp = vt + (i * 32 + col) * LDV + set * 32 + st * 16 + 4 * half;
+                out[i] = matrix::mma_values<T>(Op<T>::load_pair(vp, vp + 8), f, out[i]);
             }
+        }
     }
-    if (m >= p.rows) return;
-    const float factor = matrix::sigmoid(p.mixed[(size_t)m * l.ld_mix + l.gate_at + h]) / sum;
+    // the second half of the keys joins the first: per query tile 64 lanes x (64 sums, maximum, denominator), 66 words apart
+    __syncthreads();
+    float *meet = reinterpret_cast<float *>(smem) + (size_t)(qt * 64 + lane) * 66;
+    if (set == 1) {
+#pragma unroll
+        for (int i = 0; i < 4; i++)
+#pragma unroll
+            for (int r = 0; r < 16; r++) meet[i * 16 + r] = out[i][r];
+        meet[64] = top;
+        meet[65] = sum;
+    }
+    __syncthreads();
+    if (set == 1 || m >= p.rows) return;
+    const float all = fmaxf(top, meet[64]), mine = weight_exp<T>(top - all), theirs = weight_exp<T>(meet[64] - all);
+    const float factor = matrix::sigmoid(p.mixed[(size_t)m * l.ld_mix + l.gate_at + h]) / (sum * mine + meet[65] * theirs);
     T *dst = static_cast<T *>(p.act) + (size_t)m * p.ld_act + h * l.vdim_p + v0;
 #pragma unroll
     for (int i = 0; i < 4; i++) {
@@ -372,7 +499,7 @@ __global__ __launch_bounds__(256) void latent_block_kernel(LatentShape l, Latent
 #pragma unroll
         for (int g = 0; g < 4; g++)
 #pragma unroll
-            for (int k = 0; k < 4; k++) dst[i * 32 + g * 8 + 4 * half + k] = Op<T>::from_float(out[i][4 * g + k] * factor);
+            for (int k = 0; k < 4; k++) dst[i * 32 + g * 8 + 4 * half + k] = Op<T>::from_float((out[i][4 * g + k] * mine + meet[i * 16 + 4 * g + k] * theirs) * factor);
     }
 }
 
@@ -381,24 +508,27 @@ bool shape_ok(const LatentShape &l) {
            l.kv_rank <= l.rank_p && l.rot_dims <= l.rot_dim && l.rot_dims % 2 == 0 && l.window >= 1 && l.ring >= 1 && l.cache && l.rank_p <= kLatentMaxRank && l.dim_p <= 4096;
 }
 
-template <typename T, int NT>
+template <typename T, int NT, int KS>
 hipError_t run_partial(const LatentShape &l, const LatentStep &p, hipStream_t s) {
-    const int width = l.rank_p + l.rot_p;
-    const bool queries = PartialLayout<T>::bytes(width, true) <= 158 * 1024;   // otherwise they are read from memory for every tile
-    const size_t lds = PartialLayout<T>::bytes(width, queries);
+    const size_t lds = PartialLayout<T>::bytes(l.rank_p + l.rot_p);
     if (lds > 158 * 1024) return hipErrorInvalidValue;
-    const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void *>(&latent_partial_kernel<T, NT>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+    const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void *>(&latent_partial_kernel<T, NT, KS>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
     if (e != hipSuccess) return e;
-    hipLaunchKernelGGL((latent_partial_kernel<T, NT>), dim3(p.splits, (l.heads + 31) / 32, p.rows), dim3(256), lds, s, l, p, queries ? 1 : 0);
+    hipLaunchKernelGGL((latent_partial_kernel<T, NT, KS>), dim3(p.splits, (l.heads + 31) / 32, p.rows), dim3(256), lds, s, l, p);
     return hipGetLastError();
 }
 
 template <typename T>
 hipError_t run_step(const LatentShape &l, const LatentStep &p, hipStream_t s) {
-    hipLaunchKernelGGL(latent_absorb_kernel, dim3((l.rank_p + 127) / 128, l.heads, p.rows), dim3(256), (size_t)(l.dim_p + 16 * 128) * 4, s, l, p);
-    const hipError_t e = l.rank_p <= 128 ? run_partial<T, 1>(l, p, s) : l.rank_p <= 256 ? run_partial<T, 2>(l, p, s) : l.rank_p <= 512 ? run_partial<T, 4>(l, p, s) : run_partial<T, 8>(l, p, s);
+    const int width = l.rank_p + l.rot_p;
+    hipLaunchKernelGGL((latent_absorb_kernel<T>), dim3((l.rank_p + 127) / 128, l.heads + (l.dkv_at >= 0 ? 1 : 0), p.rows), dim3(256), (size_t)(l.dim_p + 16 * 128) * 4, s, l, p);
+    hipError_t e;
+    if (l.rank_p <= 128 && width <= 64 * 4) e = run_partial<T, 1, 4>(l, p, s);
+    else if (l.rank_p <= 256 && width <= 64 * 6) e = run_partial<T, 2, 6>(l, p, s);
+    else if (l.rank_p <= 512 && width <= 64 * 10) e = run_partial<T, 4, 10>(l, p, s);
+    else e = run_partial<T, 8, 0>(l, p, s);
     if (e != hipSuccess) return e;
-    hipLaunchKernelGGL((latent_merge_kernel<T>), dim3(l.vdim_p / 32, l.heads, p.rows), dim3(256), (size_t)(l.rank_p + p.splits) * 4, s, l, p);
+    hipLaunchKernelGGL((latent_merge_kernel<T>), dim3(l.vdim_p / 32, l.heads, p.rows), dim3(256), (size_t)(l.rank_p + 64) * 4, s, l, p);
     return hipGetLastError();
 }
 
@@ -434,7 +564,7 @@ hipError_t launch_latent_store(const LatentShape &l, const float *mixed, const i
 }
 
 hipError_t launch_latent_step(const LatentShape &l, const LatentStep &p, Precision type, hipStream_t s) {
-    if (!shape_ok(l) || p.rows < 1 || p.splits < 1 || (!p.mix && !p.act)) return hipErrorInvalidValue;
+    if (!shape_ok(l) || p.rows < 1 || p.splits < 1 || p.splits > 64 || (!p.mix && !p.act)) return hipErrorInvalidValue;
     return type == Precision::bf16 ? run_step<uint16_t>(l, p, s) : run_step<float>(l, p, s);
 }
 

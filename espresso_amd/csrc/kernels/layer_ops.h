@@ -55,8 +55,12 @@ struct DenseGemvHead {
     const float *x = nullptr, *norm = nullptr;
     int width = 0, vocab = 0;
     float eps = 0, cap = 0;
-    float *logits = nullptr;
+    float *logits = nullptr;            // [vocab], or null
+    // optional: every workgroup's largest logit and the lowest row that has it, dense_gemv_head_workgroups of them
+    float *best_value = nullptr;
+    int *best_index = nullptr;
 };
+int dense_gemv_head_workgroups(const DenseMatrix &w);
 hipError_t launch_dense_gemv_head(const DenseGemvHead &p, hipStream_t s);
 
 // ---- blocks of rows on the matrix cores (dense_gemm.hip) -----------------------------------------------
@@ -152,9 +156,10 @@ struct LatentShape {
     const uint16_t *uk, *uv;                 // [heads * dim_p][rank_p], [heads * vdim_p][rank_p]
     void *cache;                             // [sequence][ring][rank_p + rot_p]
 };
-// Rows' latents and rotated key parts into the cache (layers with dkv_at >= 0).
+// Rows' latents and rotated key parts into the cache (layers with dkv_at >= 0); for blocks, a step does it itself.
 hipError_t launch_latent_store(const LatentShape &l, const float *mixed, const int *pos, const int *seq, int rows, Precision type, hipStream_t s);
-// One query per row: queries through W_uk into the latent space, attention over the cached latents, values through W_uv.
+// One query per row (rows of different sequences): the row's own latent into the cache where the layer has one, queries through W_uk
+// into the latent space, attention over the cached latents, values through W_uv.
 constexpr int kLatentMaxRank = 1024;
 int latent_step_splits(const LatentShape &l);
 struct LatentStep {

@@ -16,10 +16,23 @@ __global__ __launch_bounds__(kBlock) void embed_norm_kernel(const uint16_t *tabl
     __shared__ float red[4];
     const int m = blockIdx.x;
     const uint16_t *row = table + (size_t)tokens[m] * width;
-    float s = 0.0f;
-    for (int i = threadIdx.x; i < width; i += kBlock) { const float v = matrix::bf16_bits_to_float(row[i]); s += v * v; }
+    constexpr int kHeld = 32;   // values per thread kept in registers: rows up to 8192 wide are read once
+    float held[kHeld], s = 0.0f;
+#pragma unroll
+    for (int c = 0; c < kHeld; c++) {
+        const int i = threadIdx.x + c * kBlock;
+        held[c] = i < width ? matrix::bf16_bits_to_float(row[i]) : 0.0f;
+    }
+#pragma unroll
+    for (int c = 0; c < kHeld; c++) s += held[c] * held[c];
+    for (int i = threadIdx.x + kHeld * kBlock; i < width; i += kBlock) { const float v = matrix::bf16_bits_to_float(row[i]); s += v * v; }
     const float inv = 1.0f / sqrtf(detail::workgroup_sum(s, red) / (float)width + eps);
-    for (int i = threadIdx.x; i < ld; i += kBlock)
+#pragma unroll
+    for (int c = 0; c < kHeld; c++) {
+        const int i = threadIdx.x + c * kBlock;
+        if (i < ld) x[(size_t)m * ld + i] = i < width ? held[c] * inv * weight[i] : 0.0f;
+    }
+    for (int i = threadIdx.x + kHeld * kBlock; i < ld; i += kBlock)
         x[(size_t)m * ld + i] = i < width ? matrix::bf16_bits_to_float(row[i]) * inv * weight[i] : 0.0f;
 }
 

@@ -45,6 +45,14 @@ __global__ __launch_bounds__(256) void retention_step_kernel(RetentionShape r, R
     __shared__ float red[4];
     const int part = blockIdx.x, h = blockIdx.y, m = blockIdx.z, tid = threadIdx.x;
     const int pos = p.pos[m], seq = p.seq[m];
+    const bool again = p.halt && *p.halt, fresh = pos == 0 && !again;
+    const int e = tid & 7, v = part * kStepRows + (tid >> 3);
+    float *state = r.state + (((size_t)seq * r.heads + h) * r.vdim_p + v) * r.dim_p + e * 4;
+    // up to eight pieces of the row are on their way while q and k are rotated
+    constexpr int kHeld = 8;
+    float4 held[kHeld];
+#pragma unroll
+    for (int i = 0; i < kHeld; i++) held[i] = *reinterpret_cast<const float4 *>(state + (i * 32 < r.dim_p ? i * 32 : 0));
     const float *row = p.mixed + (size_t)m * r.ld_mix;
     const float *cos = r.cos + (size_t)pos * (r.rot_dims / 2), *sin = r.sin + (size_t)pos * (r.rot_dims / 2);
     const float k_scale = 1.0f / sqrtf((float)r.dim);
@@ -52,28 +60,40 @@ __global__ __launch_bounds__(256) void retention_step_kernel(RetentionShape r, R
         lds[i] = rotated_half(row + h * r.dim_p, i, r.rot_dims, cos, sin);
         lds[r.dim_p + i] = rotated_half(row + (r.heads + h) * r.dim_p, i, r.rot_dims, cos, sin) * k_scale;
     }
-    __syncthreads();
-    const int e = tid & 7, v = part * kStepRows + (tid >> 3);
     const float value = row[2 * r.heads * r.dim_p + h * r.vdim_p + v], decay = r.decay[h];
-    float *state = r.state + (((size_t)seq * r.heads + h) * r.vdim_p + v) * r.dim_p;
-    const bool again = p.halt && *p.halt, fresh = pos == 0 && !again;
+    __syncthreads();
     float o = 0.0f;
-    for (int d0 = 0; d0 < r.dim_p; d0 += 32) {
-        const int d = d0 + e * 4;
-        float4 s = fresh ? make_float4(0.f, 0.f, 0.f, 0.f) : *reinterpret_cast<const float4 *>(state + d);
-        const float4 q = *reinterpret_cast<const float4 *>(lds + d), k = *reinterpret_cast<const float4 *>(lds + r.dim_p + d);
+    auto piece = [&](int d0, float4 s) {
+        if (fresh) s = make_float4(0.f, 0.f, 0.f, 0.f);
+        const float4 q = *reinterpret_cast<const float4 *>(lds + d0 + e * 4), k = *reinterpret_cast<const float4 *>(lds + r.dim_p + d0 + e * 4);
         if (!again) {
             s.x = decay * s.x + k.x * value; s.y = decay * s.y + k.y * value; s.z = decay * s.z + k.z * value; s.w = decay * s.w + k.w * value;
-            *reinterpret_cast<float4 *>(state + d) = s;
+            *reinterpret_cast<float4 *>(state + d0) = s;
         }
         o += s.x * q.x + s.y * q.y + s.z * q.z + s.w * q.w;
-    }
+    };
+#pragma unroll
+    for (int i = 0; i < kHeld; i++)
+        if (i * 32 < r.dim_p) piece(i * 32, held[i]);
+    for (int d0 = kHeld * 32; d0 < r.dim_p; d0 += 32) piece(d0, *reinterpret_cast<const float4 *>(state + d0));
     o += detail::dpp_term<0xB1, 0xF>(o);    // the eight lanes of a row
     o += detail::dpp_term<0x4E, 0xF>(o);
     o += detail::dpp_term<0x141, 0xF>(o);
     if (e == 0) p.o[(size_t)m * r.heads * r.vdim_p + h * r.vdim_p + v] = o;
     const float total = detail::workgroup_sum(e == 0 ? o * o : 0.0f, red);
     if (tid == 0) p.squares[((size_t)m * r.heads + h) * gridDim.x + part] = total;
+}
+
+template <typename T>
+__device__ __forceinline__ void store8(T *p, const float (&x)[8]);
+template <>
+__device__ __forceinline__ void store8<uint16_t>(uint16_t *p, const float (&x)[8]) {
+    *reinterpret_cast<uint4 *>(p) = make_uint4(matrix::pack_bf16(x[0], x[1]), matrix::pack_bf16(x[2], x[3]), matrix::pack_bf16(x[4], x[5]), matrix::pack_bf16(x[6], x[7]));
+}
+template <>
+__device__ __forceinline__ void store8<float>(float *p, const float (&x)[8]) {
+    reinterpret_cast<float4 *>(p)[0] = make_float4(x[0], x[1], x[2], x[3]);
+    reinterpret_cast<float4 *>(p)[1] = make_float4(x[4], x[5], x[6], x[7]);
 }
 
 struct BlockArgs {
@@ -84,40 +104,58 @@ struct BlockArgs {
     float *o;
 };
 
-// grid (chunks, heads, 2): z = 0 rotates q and k, z = 1 transposes v
+// grid (chunks, heads, slabs of 32 columns: first those of q and k, then those of v).  What is needed transposed goes through LDS.
 template <typename T>
 __global__ __launch_bounds__(256) void retention_prepare_kernel(BlockArgs a) {
+    __shared__ float slab[32][C + 1];
     const RetentionShape &r = a.r;
-    const int chunk = blockIdx.x, h = blockIdx.y, t0 = chunk * C, tid = threadIdx.x;
-    const int len = a.rows - t0 < C ? a.rows - t0 : C;
-    const size_t head_rows = (size_t)h * a.R;
-    if (blockIdx.z == 1) {
-        const float *v = a.mixed + 2 * r.heads * r.dim_p + h * r.vdim_p;
-        for (int i = tid; i < r.vdim_p * C; i += 256) {
-            const int t = i % C, d = i / C;   // neighbours write neighbouring tokens of one dimension
-            static_cast<T *>(a.vt)[((size_t)h * r.vdim_p + d) * a.R + t0 + t] = Op<T>::from_float(t < len ? v[(size_t)(t0 + t) * r.ld_mix + d] : 0.0f);
+    const int chunk = blockIdx.x, h = blockIdx.y, t0 = chunk * C, tid = threadIdx.x, slabs = r.dim_p / 32;
+    const int len = a.rows - t0 < C ? a.rows - t0 : C, c = tid & 31;
+    const bool values = (int)blockIdx.z >= slabs;
+    const int d = (values ? (int)blockIdx.z - slabs : (int)blockIdx.z) * 32 + c;
+    if (values) {
+        const float *v = a.mixed + 2 * r.heads * r.dim_p + h * r.vdim_p + d;
+#pragma unroll
+        for (int i = 0; i < C / 8; i++) {
+            const int t = (tid >> 5) + 8 * i;
+            slab[c][t] = t < len ? v[(size_t)(t0 + t) * r.ld_mix] : 0.0f;
         }
-        return;
+    } else {
+        const float k_scale = 1.0f / sqrtf((float)r.dim);
+        const float *powers = r.powers + h * (C + 1);
+#pragma unroll
+        for (int i = 0; i < C / 8; i++) {
+            const int t = (tid >> 5) + 8 * i;
+            float q = 0.0f, k = 0.0f;
+            if (t < len) {
+                const float *row = a.mixed + (size_t)(t0 + t) * r.ld_mix;
+                const size_t at = (size_t)(a.base + t0 + t) * (r.rot_dims / 2);
+                q = rotated_half(row + h * r.dim_p, d, r.rot_dims, r.cos + at, r.sin + at);
+                k = rotated_half(row + (r.heads + h) * r.dim_p, d, r.rot_dims, r.cos + at, r.sin + at) * k_scale;
+            }
+            const size_t o = ((size_t)h * a.R + t0 + t) * r.dim_p + d;
+            static_cast<T *>(a.q)[o] = Op<T>::from_float(q);
+            static_cast<T *>(a.k)[o] = Op<T>::from_float(k);
+            slab[c][t] = t < len ? k * powers[len - 1 - t] : 0.0f;
+        }
     }
-    const float k_scale = 1.0f / sqrtf((float)r.dim);
-    const float *powers = r.powers + h * (C + 1);
-    for (int i = tid; i < r.dim_p * C; i += 256) {
-        const int d = i % r.dim_p, t = i / r.dim_p;
-        float q = 0.0f, k = 0.0f;
-        if (t < len) {
-            const float *row = a.mixed + (size_t)(t0 + t) * r.ld_mix;
-            const size_t at = (size_t)(a.base + t0 + t) * (r.rot_dims / 2);
-            q = rotated_half(row + h * r.dim_p, d, r.rot_dims, r.cos + at, r.sin + at);
-            k = rotated_half(row + (r.heads + h) * r.dim_p, d, r.rot_dims, r.cos + at, r.sin + at) * k_scale;
+    __syncthreads();
+    // eight tokens of one column per thread
+    const int col = tid >> 3, part = (tid & 7) * 8;
+    const int first = (values ? (int)blockIdx.z - slabs : (int)blockIdx.z) * 32 + col;
+    float x[8];
+#pragma unroll
+    for (int i = 0; i < 8; i++) x[i] = slab[col][part + i];
+    if (values) {
+        store8<T>(static_cast<T *>(a.vt) + ((size_t)h * r.vdim_p + first) * a.R + t0 + part, x);
+    } else {
+        const size_t o = ((size_t)h * r.dim_p + first) * a.R + t0 + part;
+        store8<T>(static_cast<T *>(a.kt_hi) + o, x);
+        if constexpr (Op<T>::kSplit) {
+#pragma unroll
+            for (int i = 0; i < 8; i++) x[i] -= Op<T>::to_float(Op<T>::from_float(x[i]));
+            store8<T>(static_cast<T *>(a.kt_lo) + o, x);
         }
-        const size_t o = (head_rows + t0 + t) * r.dim_p + d;
-        static_cast<T *>(a.q)[o] = Op<T>::from_float(q);
-        static_cast<T *>(a.k)[o] = Op<T>::from_float(k);
-        const float w = t < len ? k * powers[len - 1 - t] : 0.0f;
-        const size_t ot = ((size_t)h * r.dim_p + d) * a.R + t0 + t;
-        const T hi = Op<T>::from_float(w);
-        static_cast<T *>(a.kt_hi)[ot] = hi;
-        if constexpr (Op<T>::kSplit) static_cast<T *>(a.kt_lo)[ot] = Op<T>::from_float(w - Op<T>::to_float(hi));
     }
 }
 
@@ -249,7 +287,7 @@ template <typename T>
 hipError_t run_block(const BlockArgs &a, hipStream_t s) {
     const RetentionShape &r = a.r;
     const int chunks = a.R / C;
-    hipLaunchKernelGGL((retention_prepare_kernel<T>), dim3(chunks, r.heads, 2), dim3(256), 0, s, a);
+    hipLaunchKernelGGL((retention_prepare_kernel<T>), dim3(chunks, r.heads, (r.dim_p + r.vdim_p) / 32), dim3(256), 0, s, a);
     hipLaunchKernelGGL((retention_states_kernel<T>), dim3((r.dim_p + 127) / 128, r.vdim_p / 32, r.heads), dim3(256), 0, s, a);
     hipLaunchKernelGGL((retention_outputs_kernel<T>), dim3(chunks, r.heads, (r.vdim_p + 127) / 128), dim3(256), 0, s, a);
     return hipGetLastError();

@@ -315,7 +315,7 @@ int LayeredRuntime::enqueue_trunk(int rows, bool, float *final_out) {
     return rows == 1 ? enqueue_step(final_out) : enqueue_block(rows, -1, 0, final_out);
 }
 
-// One row: three launches per retention layer, six per attention layer.
+// One row: three launches per retention layer, five per attention layer.
 int LayeredRuntime::enqueue_step(float *final_out) {
     hipStream_t s = context().stream;
     const float eps = (float)c_.norm_eps, mult = (float)c_.residual_mult;
@@ -342,7 +342,6 @@ int LayeredRuntime::enqueue_step(float *final_out) {
         } else {
             const LatentShape &l = L.latent;
             if ((rc = time_begin(K_LATENT)) != ESP_OK) return rc;
-            if (l.dkv_at >= 0) ESP_HIP_TRY(launch_latent_store(l, mixed_, d_pos_, d_seq_, 1, precision_, s));
             LatentStep st{mixed_, d_pos_, d_seq_, absorbed_, partial_, partial_ml_, L.splits, 1, mix32_, nullptr, 0};
             ESP_HIP_TRY(launch_latent_step(l, st, precision_, s));
             if ((rc = time_end()) != ESP_OK) return rc;
@@ -391,8 +390,8 @@ int LayeredRuntime::enqueue_block(int rows, int seq, int base, float *final_out)
         } else {
             const LatentShape &l = L.latent;
             if ((rc = time_begin(K_LATENT)) != ESP_OK) return rc;
-            if (l.dkv_at >= 0) ESP_HIP_TRY(launch_latent_store(l, mixed_, d_pos_, d_seq_, rows, precision_, s));
             if (seq >= 0) {
+                if (l.dkv_at >= 0) ESP_HIP_TRY(launch_latent_store(l, mixed_, d_pos_, d_seq_, rows, precision_, s));
                 LatentBlock b{};
                 b.mixed = mixed_; b.rows = rows; b.base = base; b.seq = seq;
                 latent_key_range(L, rows, base, &b);
@@ -445,7 +444,9 @@ int LayeredRuntime::run_head(const float *hidden_rows, int count, bool want_logi
     if ((rc = time_begin(K_HEAD)) != ESP_OK) return rc;
     if (count == 1) {
         DenseGemvHead h;
-        h.w = head_; h.x = hidden_rows; h.norm = final_norm_; h.width = c_.width; h.vocab = c_.vocab; h.eps = (float)c_.norm_eps; h.cap = (float)c_.logit_softcap; h.logits = logits_;
+        h.w = head_; h.x = hidden_rows; h.norm = final_norm_; h.width = c_.width; h.vocab = c_.vocab; h.eps = (float)c_.norm_eps; h.cap = (float)c_.logit_softcap;
+        if (want_logits) h.logits = logits_;
+        else { h.best_value = argmax_scratch_.part_value; h.best_index = argmax_scratch_.part_index; }
         ESP_HIP_TRY(launch_dense_gemv_head(h, s));
     } else {
         ResidualNorm n;
@@ -457,16 +458,20 @@ int LayeredRuntime::run_head(const float *hidden_rows, int count, bool want_logi
         ESP_HIP_TRY(launch_dense_gemm(g, s));
     }
     if ((rc = time_end()) != ESP_OK) return rc;
-    if (!want_logits) ESP_HIP_TRY(launch_argmax(logits_, count, c_.vocab, d_out_tokens_, nullptr, argmax_scratch_, s));
+    if (want_logits) return ESP_OK;
+    if (count == 1) ESP_HIP_TRY(launch_argmax_final(argmax_scratch_, dense_gemv_head_workgroups(head_), 1, d_out_tokens_, s));
+    else ESP_HIP_TRY(launch_argmax(logits_, count, c_.vocab, d_out_tokens_, nullptr, argmax_scratch_, s));
     return ESP_OK;
 }
 
 int LayeredRuntime::enqueue_greedy_token(int seq) {
     hipStream_t s = context().stream;
-    const int rc = run_head(device_last_hidden(seq), 1, true);
-    if (rc != ESP_OK) return rc;
-    ESP_HIP_TRY(launch_greedy_step_tail(logits_, c_.vocab, d_out_tokens_, argmax_scratch_, seq, d_visible_, d_tokens_, d_pos_, d_seq_, d_log_, d_log_count_, shape_.max_seq,
-                                        nullptr, false, c_.width, hidden_, shape_.eos_token, s));
+    DenseGemvHead h;
+    h.w = head_; h.x = device_last_hidden(seq); h.norm = final_norm_; h.width = c_.width; h.vocab = c_.vocab; h.eps = (float)c_.norm_eps; h.cap = (float)c_.logit_softcap;
+    h.best_value = argmax_scratch_.part_value; h.best_index = argmax_scratch_.part_index;
+    ESP_HIP_TRY(launch_dense_gemv_head(h, s));
+    ESP_HIP_TRY(launch_greedy_tail(argmax_scratch_, dense_gemv_head_workgroups(head_), d_out_tokens_, seq, d_visible_, d_tokens_, d_pos_, d_seq_, d_log_, d_log_count_,
+                                   shape_.max_seq, nullptr, false, c_.width, hidden_, shape_.eos_token, s));
     return ESP_OK;
 }
 

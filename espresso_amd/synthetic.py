@@ -62,3 +62,33 @@ STORIES_6L = dict(n_layer=6, n_head=12, n_kv_head=12, d_model=768, head_dim=64, 
                   max_seq=256, norm_eps=1e-5, rope_theta=10000.0, name="stories-6l-d768")
 LLAMA3_8B = dict(n_layer=32, n_head=32, n_kv_head=8, d_model=4096, head_dim=128, hidden_dim=14336, vocab=128256,
                  max_seq=1024, norm_eps=1e-5, rope_theta=500000.0, name="llama3-8b-arch")
+
+
+def layered_config(width: int, ff: int, vocab: int, attention: dict, retention: dict, layers: int = 6, window: int = 1024) -> dict:
+    """A config.json of a layered model: latent attention, two retention layers, latent attention over the first one's latents, two
+    retention layers, and so on."""
+    out = []
+    for i in range(layers):
+        mlp = {"kind": "dense", "ff": ff}
+        if i % 3:
+            heads = retention["heads"]
+            decay = [1.0 - 2.0 ** -(5.0 + 7.0 * h / max(heads - 1, 1)) for h in range(heads)]
+            out.append({"type": "retention", "mlp": mlp, "mixer": dict(retention, decay=decay, rot={"base": 1000000.0, "dims": retention["dim"]})})
+        else:
+            m = dict(attention, scale=(attention["dim"] + attention["rot_dim"]) ** -0.5, mask={"size": window},
+                     rot={"base": 10000.0, "dims": attention["rot_dim"], "scaling": {"factor": 4.0, "original": 4096, "fast": 32.0, "slow": 1.0}})
+            if i % 6 == 3:
+                m["kv_from"] = i - 3
+            out.append({"type": "latent_attention", "mlp": mlp, "mixer": m})
+    return {"architecture": "Ranavik", "vocab": vocab, "width": width, "residual_mult": 0.5, "logit_softcap": 30.0, "norm": {"eps": 1e-6}, "layers": out}
+
+
+# Layers of the size of real models, six of them, and the llama model of equal width, feed-forward, vocabulary and depth.
+LAYERED_SIZES = {
+    "d768": (layered_config(768, 2048, 32000, dict(heads=12, dim=64, vdim=64, rot_dim=32, kv_rank=256), dict(heads=6, dim=128, vdim=128)),
+             dict(n_layer=6, n_head=12, n_kv_head=12, d_model=768, head_dim=64, hidden_dim=2048, vocab=32000, max_seq=1024)),
+    "d2048": (layered_config(2048, 8192, 32000, dict(heads=16, dim=128, vdim=128, rot_dim=64, kv_rank=512), dict(heads=8, dim=256, vdim=256)),
+              dict(n_layer=6, n_head=32, n_kv_head=8, d_model=2048, head_dim=64, hidden_dim=8192, vocab=32000, max_seq=1024)),
+    "d4096": (layered_config(4096, 14336, 32000, dict(heads=32, dim=128, vdim=128, rot_dim=64, kv_rank=512), dict(heads=16, dim=256, vdim=256)),
+              dict(n_layer=6, n_head=32, n_kv_head=8, d_model=4096, head_dim=128, hidden_dim=14336, vocab=32000, max_seq=1024)),
+}
