@@ -179,14 +179,19 @@ __global__ __launch_bounds__(64 * WM * WN) void dense_gemm_kernel(DenseGemmArgs 
 }
 
 struct TileShape { int bm, bn; };
-TileShape tile_for(int m, bool f32) { return m <= 32 && !f32 ? TileShape{32, 128} : m <= 64 ? TileShape{64, 128} : TileShape{128, 128}; }
+// Tall tiles unless they leave compute units without one (a launch that may split k fills the chip that way instead).
+TileShape tile_for(int m, int n, bool f32, bool splits) {
+    if (m <= 32 && !f32) return TileShape{32, 128};
+    if (m <= 64 || (!splits && ((m + 127) / 128) * ((n + 127) / 128) < 200)) return TileShape{64, 128};
+    return TileShape{128, 128};
+}
 int ceil_div(int a, int b) { return (a + b - 1) / b; }
 
 template <typename TA, typename TB>
 hipError_t run(const DenseGemm &p, hipStream_t s) {
     constexpr bool f32 = std::is_same<TA, float>::value || std::is_same<TB, float>::value;
     constexpr int KT = f32 ? 32 : 64;
-    const TileShape t = tile_for(p.m, f32);
+    const TileShape t = tile_for(p.m, p.n, f32, p.out == GemmOut::planes);
     DenseGemmArgs a{};
     a.a = p.a; a.a2 = p.a2; a.b = p.b; a.lda = p.lda; a.ldb = p.ldb; a.m = p.m; a.n = p.n;
     a.tiles = p.k / KT;
@@ -210,7 +215,7 @@ hipError_t run(const DenseGemm &p, hipStream_t s) {
 
 // Enough workgroups for two per compute unit, at least four tiles of 64 per split, planes within the workspace.
 int gemm_planes_splits(int m, int n, int k, size_t workspace_floats) {
-    const TileShape t = tile_for(m, false);
+    const TileShape t = tile_for(m, n, false, true);
     const int tiles = ceil_div(m, t.bm) * ceil_div(n, t.bn), k_tiles = k / 64;
     int splits = 1;
     for (int s = 2; s <= 16; s++) {

@@ -117,10 +117,11 @@ __global__ __launch_bounds__(256) void latent_absorb_kernel(LatentShape l, Laten
 // Keys a query at `pos` sees: first, and how many.
 __device__ __forceinline__ int first_seen(int pos, int window) { return pos - window + 1 > 0 ? pos - window + 1 : 0; }
 
+constexpr int kPartialWaves = 8, kPartialThreads = 64 * kPartialWaves;
 template <typename T>
-struct PartialLayout {   // LDS of latent_partial_kernel: a tile of 32 cached rows, the scores of four wavefronts
+struct PartialLayout {   // LDS of latent_partial_kernel: a tile of 32 cached rows, the scores of its wavefronts
     static constexpr int kPad = 16 / sizeof(T);
-    static size_t bytes(int width) { return (size_t)32 * (width + kPad) * sizeof(T) + (size_t)4 * 32 * 33 * 4; }
+    static size_t bytes(int width) { return (size_t)32 * (width + kPad) * sizeof(T) + (size_t)kPartialWaves * 32 * 33 * 4; }
 };
 typedef uint32_t uintx4 __attribute__((ext_vector_type(4)));
 
@@ -131,10 +132,10 @@ __device__ __forceinline__ float weight_exp(float x) {
     else return expf(x);
 }
 
-// grid (splits, groups of 32 heads, rows).  NT: tiles of 32 ranks per wavefront.  KS: rows of up to 64 KS values have their queries
+// grid (splits, groups of 32 heads, rows).  NT: tiles of 32 ranks per wavefront.  KS: rows of up to 128 KS values have their queries
 // and the next tile in registers (KS steps of 16 per wavefront, KS pieces of eight per thread); 0: any width, from memory as needed.
 template <typename T, int NT, int KS>
-__global__ __launch_bounds__(256) void latent_partial_kernel(LatentShape l, LatentStep p) {
+__global__ __launch_bounds__(kPartialThreads) void latent_partial_kernel(LatentShape l, LatentStep p) {
     extern __shared__ char smem[];
     constexpr int kVec = sizeof(T) / 2;   // 128-bit words per piece
     const int width = l.rank_p + l.rot_p, ldc = width + PartialLayout<T>::kPad;
@@ -148,33 +149,35 @@ __global__ __launch_bounds__(256) void latent_partial_kernel(LatentShape l, Late
     const float *q_row = p.absorbed + ((size_t)m * l.heads + head_in) * width + 8 * half;
     const T *cache = static_cast<const T *>(l.cache) + (size_t)p.seq[m] * l.ring * width;
     const int pieces = width / 8, steps = width / 16;
-    auto row_piece = [&](int k0, int i) {   // piece i of the tile at k0; rows past the query repeat it and are masked below
-        const int row = i / pieces, part = i % pieces, key = k0 + row < pos ? k0 + row : pos;
-        return reinterpret_cast<const uintx4 *>(cache + (size_t)(key % l.ring) * width + part * 8);
+    constexpr int kRowThreads = kPartialThreads / 32;   // sixteen threads copy a row of the tile
+    const int row = tid / kRowThreads, part = tid % kRowThreads;
+    auto source_row = [&](int k0) {   // rows past the query repeat it and are masked below
+        const int key = k0 + row < pos ? k0 + row : pos;
+        return cache + (size_t)(key % l.ring) * width;
     };
-    auto tile_piece = [&](int i) { return reinterpret_cast<uintx4 *>(tile + i / pieces * ldc + i % pieces * 8); };
+    auto place = [&](int piece) { return reinterpret_cast<uintx4 *>(tile + row * ldc + piece * 8); };
     uintx4 ahead[KS ? KS * kVec : 1];
     auto fetch = [&](int t) {
         if constexpr (KS > 0) {
+            const T *src = source_row(lo + t * 32);
 #pragma unroll
             for (int k = 0; k < KS; k++) {
-                const int i = tid + k * 256;
-                const uintx4 *src = row_piece(lo + t * 32, i < 32 * pieces ? i : 0);
+                const int piece = part + k * kRowThreads;
 #pragma unroll
-                for (int v = 0; v < kVec; v++) ahead[k * kVec + v] = src[v];
+                for (int v = 0; v < kVec; v++) ahead[k * kVec + v] = reinterpret_cast<const uintx4 *>(src + (piece < pieces ? piece : 0) * 8)[v];
             }
         }
     };
-    fetch(split);
     float qv[KS ? KS : 1][8];
     if constexpr (KS > 0) {
 #pragma unroll
         for (int k = 0; k < KS; k++) {
-            const int ks = wave + 4 * k < steps ? wave + 4 * k : 0;
+            const int ks = wave + kPartialWaves * k < steps ? wave + kPartialWaves * k : 0;
             const float4 q0 = reinterpret_cast<const float4 *>(q_row + ks * 16)[0], q1 = reinterpret_cast<const float4 *>(q_row + ks * 16)[1];
             qv[k][0] = q0.x; qv[k][1] = q0.y; qv[k][2] = q0.z; qv[k][3] = q0.w; qv[k][4] = q1.x; qv[k][5] = q1.y; qv[k][6] = q1.z; qv[k][7] = q1.w;
         }
     }
+    fetch(split);
     float top = -INFINITY, sum = 0.0f;
     floatx16 acc[NT];
 #pragma unroll
@@ -185,18 +188,17 @@ __global__ __launch_bounds__(256) void latent_partial_kernel(LatentShape l, Late
         if constexpr (KS > 0) {
 #pragma unroll
             for (int k = 0; k < KS; k++) {
-                const int i = tid + k * 256;
-                if (i < 32 * pieces) {
+                if (part + k * kRowThreads < pieces) {
 #pragma unroll
-                    for (int v = 0; v < kVec; v++) tile_piece(i)[v] = ahead[k * kVec + v];
+                    for (int v = 0; v < kVec; v++) place(part + k * kRowThreads)[v] = ahead[k * kVec + v];
                 }
             }
             if (t + p.splits < tiles) fetch(t + p.splits);
         } else {
-            for (int i = tid; i < 32 * pieces; i += 256) {
-                const uintx4 *src = row_piece(k0, i);
+            const T *src = source_row(k0);
+            for (int i = part; i < pieces; i += kRowThreads) {
 #pragma unroll
-                for (int v = 0; v < kVec; v++) tile_piece(i)[v] = src[v];
+                for (int v = 0; v < kVec; v++) place(i)[v] = reinterpret_cast<const uintx4 *>(src + i * 8)[v];
             }
         }
         __syncthreads();
@@ -205,9 +207,9 @@ __global__ __launch_bounds__(256) void latent_partial_kernel(LatentShape l, Late
         if constexpr (KS > 0) {
 #pragma unroll
             for (int k = 0; k < KS; k++)
-                if (wave + 4 * k < steps) s = matrix::mma_values<T>(Op<T>::load(key_row + (wave + 4 * k) * 16), qv[k], s);
+                if (wave + kPartialWaves * k < steps) s = matrix::mma_values<T>(Op<T>::load(key_row + (wave + kPartialWaves * k) * 16), qv[k], s);
         } else {
-            for (int ks = wave; ks < steps; ks += 4) {
+            for (int ks = wave; ks < steps; ks += kPartialWaves) {
                 const float4 q0 = reinterpret_cast<const float4 *>(q_row + ks * 16)[0], q1 = reinterpret_cast<const float4 *>(q_row + ks * 16)[1];
                 const float f[8] = {q0.x, q0.y, q0.z, q0.w, q1.x, q1.y, q1.z, q1.w};
                 s = matrix::mma_values<T>(Op<T>::load(key_row + ks * 16), f, s);
@@ -220,7 +222,9 @@ __global__ __launch_bounds__(256) void latent_partial_kernel(LatentShape l, Late
 #pragma unroll
         for (int r = 0; r < 16; r++) {
             const int key = matrix::accumulator_row(r, half), at = key * 33 + col;
-            const float x = (scores[at] + scores[at + 32 * 33]) + (scores[at + 64 * 33] + scores[at + 96 * 33]);
+            float x = scores[at];
+#pragma unroll
+            for (int g = 1; g < kPartialWaves; g++) x += scores[at + g * 32 * 33];
             w[r] = k0 + key <= pos ? x : -INFINITY;
             best = fmaxf(best, w[r]);
         }
@@ -234,7 +238,7 @@ __global__ __launch_bounds__(256) void latent_partial_kernel(LatentShape l, Late
         top = best;
 #pragma unroll
         for (int i = 0; i < NT; i++) {
-            const int r0 = (wave + 4 * i) * 32;
+            const int r0 = (wave + kPartialWaves * i) * 32;
             if (r0 >= l.rank_p) continue;
 #pragma unroll
             for (int r = 0; r < 16; r++) acc[i][r] *= keep;
@@ -255,7 +259,7 @@ __global__ __launch_bounds__(256) void latent_partial_kernel(LatentShape l, Late
     const size_t at = ((size_t)m * p.splits + split) * l.heads + head;
 #pragma unroll
     for (int i = 0; i < NT; i++) {
-        const int r0 = (wave + 4 * i) * 32;
+        const int r0 = (wave + kPartialWaves * i) * 32;
         if (r0 >= l.rank_p) continue;
 #pragma unroll
         for (int g = 0; g < 4; g++)
@@ -514,7 +518,7 @@ hipError_t run_partial(const LatentShape &l, const LatentStep &p, hipStream_t s)
     if (lds > 158 * 1024) return hipErrorInvalidValue;
     const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void *>(&latent_partial_kernel<T, NT, KS>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
     if (e != hipSuccess) return e;
-    hipLaunchKernelGGL((latent_partial_kernel<T, NT, KS>), dim3(p.splits, (l.heads + 31) / 32, p.rows), dim3(256), lds, s, l, p);
+    hipLaunchKernelGGL((latent_partial_kernel<T, NT, KS>), dim3(p.splits, (l.heads + 31) / 32, p.rows), dim3(kPartialThreads), lds, s, l, p);
     return hipGetLastError();
 }
 
@@ -523,10 +527,9 @@ hipError_t run_step(const LatentShape &l, const LatentStep &p, hipStream_t s) {
     const int width = l.rank_p + l.rot_p;
     hipLaunchKernelGGL((latent_absorb_kernel<T>), dim3((l.rank_p + 127) / 128, l.heads + (l.dkv_at >= 0 ? 1 : 0), p.rows), dim3(256), (size_t)(l.dim_p + 16 * 128) * 4, s, l, p);
     hipError_t e;
-    if (l.rank_p <= 128 && width <= 64 * 4) e = run_partial<T, 1, 4>(l, p, s);
-    else if (l.rank_p <= 256 && width <= 64 * 6) e = run_partial<T, 2, 6>(l, p, s);
-    else if (l.rank_p <= 512 && width <= 64 * 10) e = run_partial<T, 4, 10>(l, p, s);
-    else e = run_partial<T, 8, 0>(l, p, s);
+    if (l.rank_p <= 256 && width <= 128 * 3) e = run_partial<T, 1, 3>(l, p, s);
+    else if (l.rank_p <= 512 && width <= 128 * 5) e = run_partial<T, 2, 5>(l, p, s);
+    else e = run_partial<T, 4, 0>(l, p, s);
     if (e != hipSuccess) return e;
     hipLaunchKernelGGL((latent_merge_kernel<T>), dim3(l.vdim_p / 32, l.heads, p.rows), dim3(256), (size_t)(l.rank_p + 64) * 4, s, l, p);
     return hipGetLastError();

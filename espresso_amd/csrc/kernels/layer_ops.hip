@@ -12,27 +12,39 @@ using matrix::Op;
 
 constexpr int kBlock = 256;
 
-__global__ __launch_bounds__(kBlock) void embed_norm_kernel(const uint16_t *table, const int *tokens, const float *weight, float eps, int width, int ld, float *x) {
-    __shared__ float red[4];
+constexpr int kEmbedBlock = 1024;
+__global__ __launch_bounds__(kEmbedBlock) void embed_norm_kernel(const uint16_t *table, const int *tokens, const float *weight, float eps, int width, int ld, float *x) {
+    __shared__ float red[kEmbedBlock / 64];
     const int m = blockIdx.x;
     const uint16_t *row = table + (size_t)tokens[m] * width;
-    constexpr int kHeld = 32;   // values per thread kept in registers: rows up to 8192 wide are read once
-    float held[kHeld], s = 0.0f;
+    constexpr int kHeld = 8;   // values per thread kept in registers: rows up to 8192 wide are read once, with every load in flight
+    uint16_t bits[kHeld];
+    float gain[kHeld], s = 0.0f;
 #pragma unroll
     for (int c = 0; c < kHeld; c++) {
-        const int i = threadIdx.x + c * kBlock;
-        held[c] = i < width ? matrix::bf16_bits_to_float(row[i]) : 0.0f;
+        const int i = threadIdx.x + c * kEmbedBlock, in = i < width ? i : width - 1;
+        bits[c] = row[in];
+        gain[c] = weight[in];
     }
-#pragma unroll
-    for (int c = 0; c < kHeld; c++) s += held[c] * held[c];
-    for (int i = threadIdx.x + kHeld * kBlock; i < width; i += kBlock) { const float v = matrix::bf16_bits_to_float(row[i]); s += v * v; }
-    const float inv = 1.0f / sqrtf(detail::workgroup_sum(s, red) / (float)width + eps);
 #pragma unroll
     for (int c = 0; c < kHeld; c++) {
-        const int i = threadIdx.x + c * kBlock;
-        if (i < ld) x[(size_t)m * ld + i] = i < width ? held[c] * inv * weight[i] : 0.0f;
+        const float v = matrix::bf16_bits_to_float(bits[c]);
+        s += (int)threadIdx.x + c * kEmbedBlock < width ? v * v : 0.0f;
     }
-    for (int i = threadIdx.x + kHeld * kBlock; i < ld; i += kBlock)
+    for (int i = threadIdx.x + kHeld * kEmbedBlock; i < width; i += kEmbedBlock) { const float v = matrix::bf16_bits_to_float(row[i]); s += v * v; }
+    s = detail::wave_sum(s);
+    if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = s;
+    __syncthreads();
+    float total = 0.0f;
+#pragma unroll
+    for (int w = 0; w < kEmbedBlock / 64; w++) total += red[w];
+    const float inv = 1.0f / sqrtf(total / (float)width + eps);
+#pragma unroll
+    for (int c = 0; c < kHeld; c++) {
+        const int i = threadIdx.x + c * kEmbedBlock;
+        if (i < ld) x[(size_t)m * ld + i] = i < width ? matrix::bf16_bits_to_float(bits[c]) * inv * gain[c] : 0.0f;
+    }
+    for (int i = threadIdx.x + kHeld * kEmbedBlock; i < ld; i += kEmbedBlock)
         x[(size_t)m * ld + i] = i < width ? matrix::bf16_bits_to_float(row[i]) * inv * weight[i] : 0.0f;
 }
 
@@ -106,7 +118,7 @@ __global__ __launch_bounds__(kBlock) void residual_norm_kernel(ResidualNormArgs 
 
 hipError_t launch_embed_norm(const uint16_t *table, const int *tokens, const float *weight, float eps, int rows, int width, int ld, float *x, hipStream_t s) {
     if (!table || rows < 1 || width < 1 || ld < width) return hipErrorInvalidValue;
-    hipLaunchKernelGGL(embed_norm_kernel, dim3(rows), dim3(kBlock), 0, s, table, tokens, weight, eps, width, ld, x);
+    hipLaunchKernelGGL(embed_norm_kernel, dim3(rows), dim3(kEmbedBlock), 0, s, table, tokens, weight, eps, width, ld, x);
     return hipGetLastError();
 }
 

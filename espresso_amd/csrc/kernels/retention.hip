@@ -181,6 +181,13 @@ __global__ __launch_bounds__(256) void retention_states_kernel(BlockArgs a) {
         const int len = a.rows - c * C < C ? a.rows - c * C : C;
         T *hi = static_cast<T *>(a.states_hi) + ((size_t)c * r.heads + h) * head, *lo = static_cast<T *>(a.states_lo) + ((size_t)c * r.heads + h) * head;
         const float factor = r.powers[h * (C + 1) + len];
+        typename Op<T>::frag v[C / 16], w[C / 16], x[C / 16];   // on their way while the state before the chunk is stored
+#pragma unroll
+        for (int ks = 0; ks < C / 16; ks++) {
+            v[ks] = Op<T>::load(vt + c * C + ks * 16);
+            w[ks] = Op<T>::load(kh + c * C + ks * 16);
+            if constexpr (Op<T>::kSplit) x[ks] = Op<T>::load(kl + c * C + ks * 16);
+        }
 #pragma unroll
         for (int i = 0; i < 16; i++) {
             const size_t o = tile + (size_t)matrix::accumulator_row(i, half) * r.dim_p;
@@ -191,9 +198,8 @@ __global__ __launch_bounds__(256) void retention_states_kernel(BlockArgs a) {
         }
 #pragma unroll
         for (int ks = 0; ks < C / 16; ks++) {
-            const typename Op<T>::frag v = Op<T>::load(vt + c * C + ks * 16);
-            acc = Op<T>::mma(v, Op<T>::load(kh + c * C + ks * 16), acc);
-            if constexpr (Op<T>::kSplit) acc = Op<T>::mma(v, Op<T>::load(kl + c * C + ks * 16), acc);
+            acc = Op<T>::mma(v[ks], w[ks], acc);
+            if constexpr (Op<T>::kSplit) acc = Op<T>::mma(v[ks], x[ks], acc);
         }
     }
 #pragma unroll
@@ -217,15 +223,29 @@ __global__ __launch_bounds__(256) void retention_outputs_kernel(BlockArgs a) {
     floatx16 score[2], out[2];
 #pragma unroll
     for (int i = 0; i < 2; i++) score[i] = out[i] = matrix::zero_accumulator();
-    for (int d = 0; d < r.dim_p; d += 16) {
-        const typename Op<T>::frag qf = Op<T>::load(q + d);
-        score[0] = Op<T>::mma(Op<T>::load(k + d), qf, score[0]);
-        if (qt) score[1] = Op<T>::mma(Op<T>::load(k + (size_t)32 * r.dim_p + d), qf, score[1]);
+    constexpr int kAhead = Op<T>::kSplit ? 2 : 1;   // steps of 16 dimensions whose loads are in flight together (dim_p is a multiple of 32)
+    const size_t k_next = qt ? (size_t)32 * r.dim_p : 0;
+    for (int d0 = 0; d0 < r.dim_p; d0 += 16 * kAhead) {
+        typename Op<T>::frag qf[kAhead], kf[kAhead][2], sf[kAhead][2], tf[kAhead][2];
 #pragma unroll
-        for (int i = 0; i < 2; i++) {
-            out[i] = Op<T>::mma(Op<T>::load(shi + i * next + d), qf, out[i]);
-            if constexpr (Op<T>::kSplit) out[i] = Op<T>::mma(Op<T>::load(slo + i * next + d), qf, out[i]);
+        for (int u = 0; u < kAhead; u++) {
+            const int d = d0 + 16 * u;
+            qf[u] = Op<T>::load(q + d);
+#pragma unroll
+            for (int i = 0; i < 2; i++) {
+                kf[u][i] = Op<T>::load(k + i * k_next + d);
+                sf[u][i] = Op<T>::load(shi + i * next + d);
+                if constexpr (Op<T>::kSplit) tf[u][i] = Op<T>::load(slo + i * next + d);
+            }
         }
+#pragma unroll
+        for (int u = 0; u < kAhead; u++)
+#pragma unroll
+            for (int i = 0; i < 2; i++) {
+                score[i] = Op<T>::mma(kf[u][i], qf[u], score[i]);
+                out[i] = Op<T>::mma(sf[u][i], qf[u], out[i]);
+                if constexpr (Op<T>::kSplit) out[i] = Op<T>::mma(tf[u][i], qf[u], out[i]);
+            }
     }
     const float *powers = r.powers + h * (C + 1);
     const float reach = powers[t_local + 1];
