@@ -25,16 +25,36 @@ def library_path() -> str:
     return _build.LIB_PATH
 
 
-def load_library() -> C.CDLL:
+class _Present:
+    """Declarations on a library that may be one component of the whole: symbols it does not have are skipped."""
+
+    class _Absent:
+        pass
+
+    def __init__(self, lib: C.CDLL):
+        self._lib = lib
+
+    def __getattr__(self, name: str):
+        return getattr(self._lib, name, None) or _Present._Absent()
+
+
+def load_library(component: str | None = None) -> C.CDLL:
+    """The library, built first if nothing is.  `component` (build.COMPONENTS): a caller that needs no more than that part takes the
+    whole library if it is there, and else builds and loads the part alone."""
     global _LIB
     if _LIB is not None:
         return _LIB
     path = library_path()
     if not os.path.exists(path):
-        _build.build()
+        if component is None:
+            _build.build()
+        else:
+            path = _build.component_path(component)
+            if not os.path.exists(path):
+                _build.build(component=component, jobs=os.cpu_count() and min(16, os.cpu_count()) or 8)
     lib = C.CDLL(path)
-    _declare(lib)
-    _declare_llama(lib)
+    _declare(_Present(lib))
+    _declare_llama(_Present(lib))
     _LIB = lib
     return lib
 

@@ -2,7 +2,7 @@
 
 Every source is compiled to an object of its own, several at a time, and the objects are linked into the shared
 library.  build() recompiles everything; build(incremental=True) keeps objects that are newer than their source and
-every header (a convenience while developing).
+every header (a convenience while developing); build(component=...) builds a part of the library that stands alone.
 """
 from __future__ import annotations
 
@@ -17,6 +17,16 @@ CSRC = os.path.join(HERE, "csrc")
 LIB_DIR = os.path.join(HERE, "lib")
 OBJ_DIR = os.path.join(HERE, "build")
 LIB_PATH = os.path.join(LIB_DIR, "libespresso_hip.so")
+
+# Parts of the library that can be built alone (a checkout with nothing built that serves one model): the sources under csrc/.
+COMPONENTS = {
+    "layered": [
+        "context.cpp", "decoder_runtime.cpp", "generation.cpp", "layered_runtime.cpp", "capi_runtime.cpp", "capi_engine.cpp", "capi_layered.cpp",
+        "host/engine.cpp", "host/runtime_registry.cpp", "host/layered_loader.cpp", "host/layered_config.cpp", "host/safetensors.cpp", "host/json_min.cpp",
+        "host/model_support.cpp", "host/tokenizer.cpp", "host/regex_min.cpp", "kernels/decode_ops.hip", "kernels/dense_gemv.hip", "kernels/dense_gemm.hip",
+        "kernels/layer_ops.hip", "kernels/retention.hip", "kernels/latent_attention.hip",
+    ],
+}
 
 # -packed-fp32-ops is switched off on purpose: packed fp32 VALU forms are not used in this library.
 HIPCC_FLAGS = [
@@ -50,13 +60,20 @@ def _run(cmd: list[str]) -> str:
     return err
 
 
-def build(verbose: bool = False, incremental: bool = False, jobs: int = 8) -> str:
+def component_path(component: str) -> str:
+    return os.path.join(LIB_DIR, f"libespresso_{component}.so")
+
+
+def build(verbose: bool = False, incremental: bool = False, jobs: int = 8, component: str | None = None) -> str:
+    """Builds the library (or one component of it) and returns its path."""
+    chosen = sources() if component is None else [os.path.join(CSRC, s) for s in COMPONENTS[component]]
+    path = LIB_PATH if component is None else component_path(component)
     os.makedirs(LIB_DIR, exist_ok=True)
     os.makedirs(OBJ_DIR, exist_ok=True)
     hipcc = os.environ.get("HIPCC", "/opt/rocm/bin/hipcc")
     newest_header = max(os.path.getmtime(h) for h in headers())
     todo = []
-    for src in sources():
+    for src in chosen:
         obj = _object_path(src)
         fresh = incremental and os.path.exists(obj) and os.path.getmtime(obj) > max(os.path.getmtime(src), newest_header)
         if not fresh:
@@ -67,10 +84,12 @@ def build(verbose: bool = False, incremental: bool = False, jobs: int = 8) -> st
                 print(" ".join(cmd))
                 if err.strip():
                     print(err, file=sys.stderr)
-    err = _run([hipcc, "--offload-arch=gfx950", "-shared", "-fPIC", "-o", LIB_PATH, *[_object_path(s) for s in sources()]])
+    part = f"{path}.{os.getpid()}"   # two processes may build at once
+    err = _run([hipcc, "--offload-arch=gfx950", "-shared", "-fPIC", "-Wl,-z,defs", "-o", part, *[_object_path(s) for s in chosen]])
+    os.replace(part, path)
     if verbose and err.strip():
         print(err, file=sys.stderr)
-    return LIB_PATH
+    return path
 
 
 if __name__ == "__main__":

@@ -1,51 +1,18 @@
-// C ABI: weight files, metadata, the GGUF front door, the engine and the exact two-token harness.
+// C ABI: weight files, the GGUF front door, tokenizers, bundles and the exact two-token harness.
 #include <algorithm>
 #include <chrono>
 #include <cstring>
 
-#include "generation.h"
-#include "host/engine.h"
+#include "capi_common.h"
 #include "host/gguf.h"
 #include "host/bundle.h"
 #include "host/harness.h"
-#include "host/layered_loader.h"
 #include "host/tokenizer.h"
 
 using namespace esp;
-
-struct ESPEngine {
-    std::unique_ptr<RealModelInferenceEngine> engine;
-    ESPLlamaRuntime runtime_handle{nullptr};
-};
+using namespace esp::capi;
 
 namespace {
-
-MultiModelConfig from_c(const ESPModelConfig &c) {
-    MultiModelConfig m;
-    m.name = std::string(c.name, strnlen(c.name, sizeof(c.name)));
-    m.nLayer = c.n_layer; m.nHead = c.n_head; m.nKVHead = c.n_kv_head; m.dModel = c.d_model; m.headDim = c.head_dim;
-    m.hiddenDim = c.hidden_dim; m.vocab = c.vocab; m.maxSeq = c.max_seq; m.normEps = c.norm_eps; m.ropeTheta = c.rope_theta;
-    m.hasEosToken = c.eos_token >= 0;
-    m.eosToken = c.eos_token >= 0 ? (TokenID)c.eos_token : 0;
-    m.architecture = c.architecture == 0 ? MultiModelConfig::Architecture::gpt2
-                     : c.architecture == 2 ? MultiModelConfig::Architecture::layered : MultiModelConfig::Architecture::llama;
-    return m;
-}
-
-void to_c(const MultiModelConfig &m, ESPModelConfig *c) {
-    std::memset(c, 0, sizeof(*c));
-    std::strncpy(c->name, m.name.c_str(), sizeof(c->name) - 1);
-    c->n_layer = m.nLayer; c->n_head = m.nHead; c->n_kv_head = m.nKVHead; c->d_model = m.dModel; c->head_dim = m.headDim;
-    c->hidden_dim = m.hiddenDim; c->vocab = m.vocab; c->max_seq = m.maxSeq; c->norm_eps = m.normEps; c->rope_theta = m.ropeTheta;
-    c->eos_token = m.hasEosToken ? (int32_t)m.eosToken : -1;
-    c->architecture = m.architecture == MultiModelConfig::Architecture::gpt2 ? 0 : m.architecture == MultiModelConfig::Architecture::layered ? 2 : 1;
-}
-
-Environment env_from(const char *const *keys, const char *const *values, int count) {
-    Environment e;
-    for (int i = 0; i < count; i++) if (keys && values && keys[i] && values[i]) e[keys[i]] = values[i];
-    return e;
-}
 
 // adapts the C callback table to the C++ protocol
 class CallbackModel : public ExactTwoTokenGeneratingLanguageModel {
@@ -122,60 +89,6 @@ int esp_layer_weight_path(int layer, const char *blob_dir, int slot, char *out, 
     if (s->size() + 1 > capacity) return fail(ESP_ERR_OUT_OF_RANGE, "layer_weight_path: buffer too small");
     std::memcpy(out, s->c_str(), s->size() + 1);
     return (int)s->size();
-}
-
-int esp_model_config_load_metadata(const char *path, ESPModelConfig *out) {
-    if (!path || !out) return fail(ESP_ERR_INVALID_ARGUMENT, "null pointer");
-    MultiModelConfig m;
-    std::string err;
-    if (!loadConfigFromMetadataFile(path, &m, &err)) return fail(ESP_ERR_IO, "%s", err.c_str());
-    to_c(m, out);
-    return ESP_OK;
-}
-
-int esp_model_config_write_metadata(const ESPModelConfig *config, const char *path) {
-    if (!path || !config) return fail(ESP_ERR_INVALID_ARGUMENT, "null pointer");
-    const std::string j = metadataJSON(from_c(*config));
-    return writeFile(path, j.data(), j.size()) ? ESP_OK : fail(ESP_ERR_IO, "cannot write %s", path);
-}
-
-int esp_model_config_load_dir(const char *model_dir, int max_seq, ESPModelConfig *out) {
-    if (!model_dir || !out) return fail(ESP_ERR_INVALID_ARGUMENT, "null argument");
-    MultiModelConfig m;
-    if (is_layered_model_dir(model_dir) || !fileExists(joinPath(model_dir, "metadata.json"))) {
-        const int rc = layered_model_config(model_dir, max_seq, &m);
-        if (rc != ESP_OK) return rc;
-    } else {
-        std::string err;
-        if (!loadConfigFromMetadataFile(joinPath(model_dir, "metadata.json"), &m, &err)) return fail(ESP_ERR_INVALID_ARGUMENT, "%s", err.c_str());
-    }
-    to_c(m, out);
-    return ESP_OK;
-}
-
-int esp_layered_architecture_count(void) { return (int)layered_architectures().size(); }
-const char *esp_layered_architecture_at(int index) {
-    return index >= 0 && index < (int)layered_architectures().size() ? layered_architectures()[index].name : nullptr;
-}
-
-int esp_model_registry_count(void) { return (int)ModelRegistry::all().size(); }
-int esp_model_registry_at(int index, ESPModelConfig *out) {
-    if (!out || index < 0 || index >= (int)ModelRegistry::all().size()) return fail(ESP_ERR_INVALID_ARGUMENT, "model registry: index %d", index);
-    to_c(ModelRegistry::all()[(size_t)index], out);
-    return ESP_OK;
-}
-int esp_model_registry_config(const char *name, ESPModelConfig *out) {
-    if (!name || !out) return fail(ESP_ERR_INVALID_ARGUMENT, "model registry: null argument");
-    const MultiModelConfig *c = ModelRegistry::config(name);
-    if (!c) return fail(ESP_ERR_INVALID_ARGUMENT, "model registry: no configuration named %s", name);
-    to_c(*c, out);
-    return ESP_OK;
-}
-int esp_classifier_strategy_select(const ESPModelConfig *config, int has_exact_float32_lm_head, char *out_label, size_t label_bytes) {
-    if (!config) return fail(ESP_ERR_INVALID_ARGUMENT, "classifier strategy: null config");
-    const ClassifierStrategy s = selectClassifierStrategy(from_c(*config), has_exact_float32_lm_head != 0);
-    if (out_label && label_bytes) { std::strncpy(out_label, exactHeadBackendLabel(s), label_bytes - 1); out_label[label_bytes - 1] = 0; }
-    return (int)s;
 }
 
 int esp_gguf_prepare(const char *gguf_path, const char *output_dir, const ESPPrepareOptions *o, ESPModelConfig *out_config,
@@ -266,66 +179,6 @@ int esp_gguf_cleanup(const char *weight_dir) {
 }
 
 int esp_gguf_default_cache_root(char *out, size_t out_bytes) { return copy_out(GGUFModelLoader::defaultPreparedArtifactCacheRoot(), out, out_bytes, "cache root"); }
-
-namespace {
-void fill_result(const GenerationResult &r, ESPGenerationResult *result) {
-    std::memset(result, 0, sizeof(*result));
-    result->token_count = (int32_t)r.tokens.size();
-    result->tokens_per_second = r.tokensPerSecond;
-    result->compile_time_ms = r.compileTimeMs;
-    result->first_token_latency_ms = r.firstTokenLatencyMs;
-    result->has_two_token_stats = r.hasTwoTokenStats ? 1 : 0;
-    result->committed_exact_tokens_per_pass = r.committedExactTokensPerPass;
-    result->accepted_future_tokens_per_pass = r.acceptedFutureTokensPerPass;
-    std::strncpy(result->exact_head_backend, r.exactHeadBackend.c_str(), sizeof(result->exact_head_backend) - 1);
-}
-}  // namespace
-
-ESPEngine *esp_engine_build(const ESPModelConfig *config, const char *weight_dir, const char *tokenizer_dir,
-                            const char *const *env_keys, const char *const *env_values, int env_count) {
-    if (!config || !weight_dir) { fail(ESP_ERR_INVALID_ARGUMENT, "null config or weight directory"); return nullptr; }
-    std::unique_ptr<RealModelInferenceEngine> e;
-    if (RealModelInferenceEngine::build(from_c(*config), weight_dir, tokenizer_dir ? tokenizer_dir : "",
-                                        env_from(env_keys, env_values, env_count), &e) != ESP_OK)
-        return nullptr;
-    ESPEngine *h = new ESPEngine();
-    h->engine = std::move(e);
-    h->runtime_handle.rt = &h->engine->runtime();
-    return h;
-}
-
-void esp_engine_free(ESPEngine *engine) { delete engine; }
-
-ESPLlamaRuntime *esp_engine_runtime(ESPEngine *engine) { return engine ? &engine->runtime_handle : nullptr; }
-
-int esp_engine_generate(ESPEngine *engine, const uint32_t *prompt_tokens, int prompt_count, int max_tokens, float temperature,
-                        const char *const *env_keys, const char *const *env_values, int env_count, uint32_t *out_tokens,
-                        ESPGenerationResult *result) {
-    if (!engine) return fail(ESP_ERR_INVALID_ARGUMENT, "null engine");
-    std::vector<TokenID> prompt;
-    if (prompt_tokens && prompt_count > 0) prompt.assign(prompt_tokens, prompt_tokens + prompt_count);
-    GenerationResult r;
-    int rc = engine->engine->generate(prompt, max_tokens, temperature, env_from(env_keys, env_values, env_count), &r);
-    if (rc != ESP_OK) return rc;
-    if (out_tokens) for (size_t i = 0; i < r.tokens.size(); i++) out_tokens[i] = r.tokens[i];
-    if (result) fill_result(r, result);
-    return ESP_OK;
-}
-
-int esp_engine_generate_text(ESPEngine *engine, const char *prompt_utf8, size_t prompt_bytes, int max_tokens, float temperature,
-                             const char *const *env_keys, const char *const *env_values, int env_count, uint32_t *out_tokens,
-                             char *out_text, size_t text_capacity, size_t *out_text_bytes, ESPGenerationResult *result) {
-    if (!engine || (!prompt_utf8 && prompt_bytes)) return fail(ESP_ERR_INVALID_ARGUMENT, "null engine or prompt");
-    GenerationResult r;
-    int rc = engine->engine->generateText(std::string(prompt_utf8 ? prompt_utf8 : "", prompt_bytes), max_tokens, temperature,
-                                          env_from(env_keys, env_values, env_count), &r);
-    if (rc != ESP_OK) return rc;
-    if (out_tokens) for (size_t i = 0; i < r.tokens.size(); i++) out_tokens[i] = r.tokens[i];
-    if (out_text_bytes) *out_text_bytes = r.text.size();
-    if (out_text && text_capacity) std::memcpy(out_text, r.text.data(), std::min(text_capacity, r.text.size()));
-    if (result) fill_result(r, result);
-    return ESP_OK;
-}
 
 int esp_run_gguf(const char *gguf_path, const char *tokenizer_dir, const char *prompt_utf8, size_t prompt_bytes, int max_tokens,
                  const char *const *env_keys, const char *const *env_values, int env_count, uint32_t *out_tokens, char *out_text,

@@ -25,7 +25,7 @@ float *g_scratch_ptr[kNoAllocMaxDevices] = {};
 }  // namespace
 
 namespace esp {
-int noalloc_setup(int device) {
+static int noalloc_setup(int device) {
     if (device < 0 || device >= kNoAllocMaxDevices) return fail(ESP_ERR_INVALID_ARGUMENT, "device %d outside 0..%d", device, kNoAllocMaxDevices - 1);
     if (g_scratch_ptr[device]) return ESP_OK;
     float *ptr = nullptr;
@@ -34,24 +34,10 @@ int noalloc_setup(int device) {
     g_scratch_ptr[device] = ptr;
     return ESP_OK;
 }
+static const DeviceSetup noalloc_scratch(noalloc_setup);
 }  // namespace esp
 
 extern "C" {
-
-int esp_init(void) { return ensure_init(); }
-
-int esp_device_info(char *name, size_t name_capacity, int *compute_units, size_t *hbm_bytes) {
-    int rc = ensure_init();
-    if (rc != ESP_OK) return rc;
-    const Context &c = context();
-    if (name && name_capacity) {
-        std::strncpy(name, c.props.gcnArchName, name_capacity - 1);
-        name[name_capacity - 1] = 0;
-    }
-    if (compute_units) *compute_units = c.props.multiProcessorCount;
-    if (hbm_bytes) *hbm_bytes = c.props.totalGlobalMem;
-    return ESP_OK;
-}
 
 size_t esp_format_bytes(int format, size_t elements) {
     if (!format_supported(format) || elements % format_block_elems(format) != 0) return 0;

@@ -2,14 +2,22 @@
 
 #include <cstdarg>
 #include <cstdio>
+#include <cstring>
 #include <mutex>
+#include <vector>
 
 namespace esp {
 namespace {
 thread_local std::string t_last_error;
 std::mutex g_init_mutex;
 Context g_context;
+std::vector<int (*)(int)> &setup_hooks() {
+    static std::vector<int (*)(int)> hooks;
+    return hooks;
+}
 }  // namespace
+
+DeviceSetup::DeviceSetup(int (*setup)(int device)) { setup_hooks().push_back(setup); }
 
 Context &context() { return g_context; }
 
@@ -48,87 +56,35 @@ int ensure_init() {
     ESP_HIP_TRY(hipGetDeviceProperties(&g_context.props, 0));
     ESP_HIP_TRY(hipStreamCreateWithFlags(&g_context.stream, hipStreamNonBlocking));
     g_context.device = 0;
-    {
-        const int rc = noalloc_setup(0);
+    for (int (*setup)(int) : setup_hooks()) {
+        const int rc = setup(0);
         if (rc != ESP_OK) return rc;
     }
     g_context.ready = true;
     return ESP_OK;
 }
 
-int matrix_upload(int format, const void *gguf_blocks, int rows, int cols, DeviceMatrix *out) {
-    *out = DeviceMatrix{};
-    if (!gguf_blocks || rows <= 0 || cols <= 0) return fail(ESP_ERR_INVALID_ARGUMENT, "matrix: null data or empty shape");
-    if (!(format == FMT_F32 || format == FMT_F16 || format == FMT_Q4_0 || format == FMT_Q8_0 || format == FMT_Q4_K))
-        return fail(ESP_ERR_UNSUPPORTED, "matrix: format %d has no GEMV kernel", format);
-    const int block = format == FMT_F16 ? 8 : format == FMT_F32 ? 4 : format_block_elems(format);
-    if (cols % block != 0) return fail(ESP_ERR_INVALID_ARGUMENT, "matrix: cols %d is not a multiple of %d", cols, block);
+}  // namespace esp
+
+extern "C" {
+
+using namespace esp;
+
+const char *esp_last_error(void) { return last_error_text(); }
+
+int esp_init(void) { return ensure_init(); }
+
+int esp_device_info(char *name, size_t name_capacity, int *compute_units, size_t *hbm_bytes) {
     int rc = ensure_init();
     if (rc != ESP_OK) return rc;
-    Context &c = context();
-    const size_t elems = (size_t)rows * cols;
-    const size_t src_bytes = format_bytes(format, elems);
-
-    DeviceMatrix m;
-    m.format = format; m.rows = rows; m.cols = cols;
-    switch (format) {
-    case FMT_Q8_0: m.qs_row_bytes = (size_t)cols; break;
-    case FMT_Q4_0: m.qs_row_bytes = (size_t)cols / 2; break;
-    case FMT_Q4_K: m.qs_row_bytes = (size_t)cols / 256 * 144; break;
-    case FMT_F32: m.qs_row_bytes = (size_t)cols * 4; break;
-    default: m.qs_row_bytes = (size_t)cols * 2; break;
+    const Context &c = context();
+    if (name && name_capacity) {
+        std::strncpy(name, c.props.gcnArchName, name_capacity - 1);
+        name[name_capacity - 1] = 0;
     }
-    if (m.qs_row_bytes % 16 != 0) return fail(ESP_ERR_INVALID_ARGUMENT, "matrix: row of %zu bytes is not 16-byte aligned", m.qs_row_bytes);
-    if ((rc = device_alloc(&m.qs, (size_t)rows * m.qs_row_bytes)) != ESP_OK) return rc;
-    const bool planes = format == FMT_Q8_0 || format == FMT_Q4_0;
-    if (planes && (rc = device_alloc(&m.scales, elems / 32)) != ESP_OK) { matrix_release(&m); return rc; }
-
-    hipError_t e;
-    if (planes) {
-        uint8_t *staging = nullptr;
-        if ((rc = device_alloc(&staging, src_bytes)) != ESP_OK) { matrix_release(&m); return rc; }
-        e = hipMemcpyAsync(staging, gguf_blocks, src_bytes, hipMemcpyHostToDevice, c.stream);
-        if (e == hipSuccess) e = launch_repack(format, staging, rows, cols, m, c.stream);
-        // Q4_0 matrices of the widths the matrix-core GEMV is built for also get the tiled copy it reads
-        if (e == hipSuccess && format == FMT_Q4_0 && gemv_wants_tiled_copy(format, cols)) {
-            const size_t tiled_bytes = (size_t)((rows + 15) / 16) * (cols / 512) * 4608;
-            if ((rc = device_alloc(&m.tiled, tiled_bytes)) != ESP_OK) { (void)hipFree(staging); matrix_release(&m); return rc; }
-            e = launch_q40_tile(m.qs, m.scales, rows, cols, m.tiled, c.stream);
-        }
-        if (e == hipSuccess && format == FMT_Q8_0 && gemv_wants_tiled_copy(format, cols)) {
-            const size_t tiled_bytes = (size_t)((rows + 15) / 16) * (cols / 256) * 4352;
-            if ((rc = device_alloc(&m.tiled, tiled_bytes)) != ESP_OK) { (void)hipFree(staging); matrix_release(&m); return rc; }
-            e = launch_q80_tile(m.qs, m.scales, rows, cols, m.tiled, c.stream);
-        }
-        if (e == hipSuccess) e = hipStreamSynchronize(c.stream);
-        (void)hipFree(staging);
-    } else {
-        e = hipMemcpyAsync(m.qs, gguf_blocks, src_bytes, hipMemcpyHostToDevice, c.stream);
-        // Q4_K matrices of the widths the matrix-core GEMV is built for also get the tiled copy it reads
-        if (e == hipSuccess && format == FMT_Q4_K && gemv_wants_tiled_copy(format, cols)) {
-            const size_t tiled_bytes = (size_t)((rows + 15) / 16) * (cols / 256) * 2304;
-            if ((rc = device_alloc(&m.tiled, tiled_bytes)) != ESP_OK) { matrix_release(&m); return rc; }
-            e = launch_q4k_tile(m.qs, rows, cols, m.tiled, c.stream);
-        }
-        if (e == hipSuccess && format == FMT_F16 && gemv_wants_tiled_copy(format, cols)) {
-            const size_t tiled_bytes = (size_t)((rows + 15) / 16) * (cols / 256) * 8192;
-            if ((rc = device_alloc(&m.tiled, tiled_bytes)) != ESP_OK) { matrix_release(&m); return rc; }
-            e = launch_f16_tile(m.qs, rows, cols, m.tiled, c.stream);
-        }
-        if (e == hipSuccess) e = hipStreamSynchronize(c.stream);
-    }
-    if (e != hipSuccess) { matrix_release(&m); return fail_hip(e, "matrix upload"); }
-    *out = m;
+    if (compute_units) *compute_units = c.props.multiProcessorCount;
+    if (hbm_bytes) *hbm_bytes = c.props.totalGlobalMem;
     return ESP_OK;
 }
 
-void matrix_release(DeviceMatrix *m) {
-    if (m->qs) (void)hipFree(m->qs);
-    if (m->scales) (void)hipFree(m->scales);
-    if (m->tiled) (void)hipFree(m->tiled);
-    *m = DeviceMatrix{};
-}
-
-}  // namespace esp
-
-extern "C" const char *esp_last_error(void) { return esp::last_error_text(); }
+}  // extern "C"

@@ -44,9 +44,10 @@ int device_alloc(T **out, size_t count) {
     return ESP_OK;
 }
 
-// Looks up the device address of the fixed scratch array of esp_gemv_device_noalloc for `device`, which must be the
-// current device (capi_ops.cpp; called once from ensure_init).
-int noalloc_setup(int device);
+// Something a part of the library sets up once per device, called by ensure_init with the current device (a static object registers it).
+struct DeviceSetup {
+    explicit DeviceSetup(int (*setup)(int device));
+};
 
 // Uploads GGUF-layout blocks (host memory) into a DeviceMatrix laid out for the GEMV kernels.
 int matrix_upload(int format, const void *gguf_blocks, int rows, int cols, DeviceMatrix *out);

@@ -5,7 +5,7 @@
 #include <cstdint>
 #include <vector>
 
-#include "llama_runtime.h"
+#include "decoder_runtime.h"
 
 namespace esp {
 

@@ -1,4 +1,4 @@
-// RealModelInferenceEngine for the llama decode path, GPU-resident.  Mirrors the reference's entry
+// RealModelInferenceEngine for every registered runtime family, GPU-resident.  Mirrors the reference's entry
 // points (Sources/RealModelInference/RealModelInferenceEngine.swift): build(config:weightDir:tokenizerDir:)
 // :1377, generate(...) :1405 in its token-id form, generateTokensExactCPUForTesting :1838, and the
 // exact two-token draft selection through ESPRESSO_BUNDLE_DRAFT_* (:5324-5390).
@@ -9,13 +9,12 @@
 #include <string>
 #include <vector>
 
-#include "../llama_runtime.h"
+#include "../decoder_runtime.h"
 #include "model_support.h"
+#include "runtime_registry.h"
 #include "tokenizer.h"
 
 namespace esp {
-
-using Environment = std::map<std::string, std::string>;
 
 // GenerationResult (:17-55); `text` is filled by the prompt-text entry point only
 struct GenerationResult {
@@ -56,14 +55,12 @@ class RealModelInferenceEngine {
 
   private:
     RealModelInferenceEngine() = default;
-    static int loadRuntime(const MultiModelConfig &config, const std::string &weightDir, const Environment &environment,
-                           std::unique_ptr<LlamaRuntime> *out);
-    static int loadLayered(const MultiModelConfig &config, const std::string &modelDir, const Environment &environment,
+    static int loadRuntime(const MultiModelConfig &config, const std::string &modelDir, const Environment &environment,
                            std::unique_ptr<DecoderRuntime> *out);
     MultiModelConfig config_;
     std::string weight_dir_;
     std::unique_ptr<DecoderRuntime> runtime_;
-    std::unique_ptr<LlamaRuntime> draft_runtime_;
+    std::unique_ptr<DecoderRuntime> draft_runtime_;
     std::unique_ptr<Tokenizer> tokenizer_;
     std::string draft_dir_loaded_;
     double build_ms_ = 0;

@@ -4,6 +4,7 @@
 #include <cstring>
 
 #include "../generation.h"
+#include "runtime_registry.h"
 #include "safetensors.h"
 
 namespace esp {
@@ -137,5 +138,28 @@ int make_synthetic_layered_model(const LayeredConfig &config, const LayeredOptio
     SyntheticWeights weights(seed, std_dev);
     return create(config, options, weights, out);
 }
+
+namespace {
+// The engine's loader: ESPRESSO_HIP_PRECISION = bf16 | f32, ESPRESSO_HIP_MAX_SEQUENCES = sequence slots.
+int load_layered(const MultiModelConfig &config, const std::string &modelDir, const Environment &env, std::unique_ptr<DecoderRuntime> *out) {
+    LayeredOptions o;
+    o.max_seq = config.maxSeq;
+    o.eos_token = config.hasEosToken ? (int)config.eosToken : -1;
+    auto get = [&](const char *k) { auto it = env.find(k); return it == env.end() ? std::string() : it->second; };
+    const std::string precision = get("ESPRESSO_HIP_PRECISION"), sequences = get("ESPRESSO_HIP_MAX_SEQUENCES");
+    if (!precision.empty() && precision != "bf16" && precision != "f32") return fail(ESP_ERR_INVALID_ARGUMENT, "ESPRESSO_HIP_PRECISION must be bf16 or f32, not %s", precision.c_str());
+    if (precision == "f32") o.precision = Precision::f32;
+    if (!sequences.empty()) o.max_sequences = std::atoi(sequences.c_str());
+    std::unique_ptr<LayeredRuntime> rt;
+    const int rc = load_layered_model(modelDir, o, &rt);
+    if (rc != ESP_OK) return rc;
+    if (rt->shape().vocab != config.vocab || rt->shape().d_model != config.dModel || (int)rt->config().layers.size() != config.nLayer)
+        return fail(ESP_ERR_INVALID_ARGUMENT, "config.json of %s does not match the given configuration", modelDir.c_str());
+    *out = std::move(rt);
+    return ESP_OK;
+}
+
+const RuntimeFamilyRegistration registration(MultiModelConfig::Architecture::layered, load_layered);
+}  // namespace
 
 }  // namespace esp

@@ -53,9 +53,10 @@ _declared = False
 
 def _L():
     global _declared
-    L = _lib.load_library()
+    lib = _lib.load_library()
     if _declared:
-        return L
+        return lib
+    L = _lib._Present(lib)
     vp, sz, i32, cp = C.c_void_p, C.c_size_t, C.c_int, C.c_char_p
     L.esp_weight_blob_bytes.restype = sz; L.esp_weight_blob_bytes.argtypes = [sz]
     L.esp_weight_blob_build.restype = i32; L.esp_weight_blob_build.argtypes = [vp, sz, vp]
@@ -78,7 +79,7 @@ def _L():
     L.esp_exact_two_token_harness_generate.restype = i32
     L.esp_exact_two_token_harness_generate.argtypes = [C.POINTER(ExactTwoTokenModelStruct), vp, vp, vp, i32, i32, vp, C.POINTER(i32), vp, vp, C.POINTER(i32)]
     _declared = True
-    return L
+    return lib
 
 
 def _ptr(a):

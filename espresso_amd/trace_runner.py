@@ -49,6 +49,11 @@ def run(model, lines, out_dir: str, vocab: int, answer) -> None:
         answer(f"done {step['step']}")
 
 
+def engine_kind(model_dir: str) -> str:
+    """"layered" for a directory with a config.json, "llama" for one with metadata.json."""
+    return "layered" if os.path.exists(os.path.join(model_dir, "config.json")) else "llama"
+
+
 def main(argv: list[str]) -> int:
     ap = argparse.ArgumentParser(prog="trace_run", description="Feed given token ids through a model and write logits.")
     ap.add_argument("--model", required=True, help="model directory (config.json, model.safetensors)")
@@ -56,7 +61,9 @@ def main(argv: list[str]) -> int:
     ap.add_argument("--out", required=True, help="directory for <step>.f32 files")
     ap.add_argument("--max-tokens", type=int, required=True, help="most tokens that live requests hold at any time")
     a = ap.parse_args(argv)
-    from . import engine, ops
+    from . import _lib, engine, ops
+    if engine_kind(a.model) == "layered":
+        _lib.load_library("layered")   # in a checkout with nothing built, this part of the library is all the model needs
     ops.init()
     cfg = engine.load_model_config(a.model, a.max_tokens)
     env = {"ESPRESSO_HIP_PRECISION": "f32" if a.dtype == "float32" else "bf16", "ESPRESSO_HIP_MAX_SEQUENCES": str(MAX_LIVE_REQUESTS)}

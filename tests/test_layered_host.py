@@ -83,6 +83,15 @@ def test_broken_files_are_refused(tmp_path):
             eng.RealModelInferenceEngine(c, str(tmp_path))
 
 
+def test_the_layered_part_of_the_library_is_listed_and_stands_alone():
+    """Its sources exist, and none of them includes a header of the llama runtime."""
+    import espresso_amd.build as build
+    for s in build.COMPONENTS["layered"]:
+        text = open(os.path.join(build.CSRC, s)).read()
+        assert "llama_runtime.h" not in text, s
+    assert build.component_path("layered") != build.LIB_PATH
+
+
 # ---- trace replay ---------------------------------------------------------------------------------
 class FakeModel:
     """Three sequence slots; a token's logits are (sequence-wide token count so far, token)."""
