@@ -45,7 +45,7 @@ class LayeredRuntime : public DecoderRuntime {
     size_t resident_weight_bytes() const override { return weight_bytes_ + (size_t)c_.vocab * c_.width * 2; }
     // what one sequence holds in states and cached latents
     size_t sequence_bytes() const { return sequence_bytes_; }
-    static constexpr int kMinBlockRows = 4;
+    static constexpr int kMinBlockRows = 3;
     // Blocks shorter than this run token by token (tests and measurements move it; default kMinBlockRows).
     void set_min_block_rows(int rows) { min_block_rows_ = rows < 1 ? 1 : rows; }
     // Residual stream after every layer of a block, one call per layer (tests).

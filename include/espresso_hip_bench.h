@@ -95,7 +95,7 @@ int esp_llama_time_kernel_dispatch(ESPLlamaRuntime *runtime, int kernel_class, i
 /* Layered runtimes (models whose config.json lists their layers).  A runtime of a configuration (the text of a config.json) with
  * seeded random weights; float32 = 1: fp32 operands and caches.  Freed with esp_llama_free. */
 ESPLlamaRuntime *esp_layered_create_synthetic(const char *config_json, int float32, int max_seq, int max_sequences, uint64_t seed, float std_dev);
-/* Portions of fewer tokens than this run token by token (default 4). */
+/* Portions of fewer tokens than this run token by token (default 3). */
 int esp_layered_set_min_block_rows(ESPLlamaRuntime *runtime, int rows);
 /* Appends up to 512 tokens as one block and copies the residual stream after every layer: out [layers][count][width]. */
 int esp_layered_trace_layers(ESPLlamaRuntime *runtime, int sequence, const uint32_t *tokens, int count, float *out);

@@ -71,7 +71,7 @@ def test_portions_of_any_size(mixed, precision, portions):
     for least in (1, 1000):        # every portion through the block kernels, down to one row; then every token through the decode kernels
         layered.set_min_block_rows(rt, least)
         assert lu.error(lu.feed(rt, t, portions, 0 if least == 1 else 1), want) < lu.limit(precision), least
-    layered.set_min_block_rows(rt, 4)
+    layered.set_min_block_rows(rt, 3)
     assert lu.error(lu.feed(rt, t, portions, 2), want) < lu.limit(precision)
 
 
