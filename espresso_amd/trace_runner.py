@@ -62,6 +62,9 @@ def main(argv: list[str]) -> int:
     ap.add_argument("--max-tokens", type=int, required=True, help="most tokens that live requests hold at any time")
     a = ap.parse_args(argv)
     from . import _lib, engine, ops
+    if engine_kind(a.model) == "llama" and a.dtype == "float32":
+        sys.stderr.write("trace_run: llama runtimes have no all-32-bit arithmetic\n")
+        return 3
     if engine_kind(a.model) == "layered":
         _lib.load_library("layered")   # in a checkout with nothing built, this part of the library is all the model needs
     ops.init()

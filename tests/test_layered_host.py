@@ -130,6 +130,11 @@ def test_trace_replay_orders_rows_and_returns_slots(tmp_path):
     assert m.log[-1] == (0, [9])          # the slot of "a" serves "c"
 
 
+def test_a_llama_directory_is_refused_in_float32(tmp_path):
+    (tmp_path / "metadata.json").write_text("{}")
+    assert tr.main(["--model", str(tmp_path), "--dtype", "float32", "--out", str(tmp_path), "--max-tokens", "4"]) == 3
+
+
 def test_command_lines_explain_themselves():
     for cmd in ([os.path.join(ROOT, "bin", "trace_run"), "--help"], [sys.executable, "-m", "espresso_amd.run_model", "--help"]):
         p = subprocess.run(cmd, capture_output=True, text=True, cwd=ROOT)
