@@ -21,10 +21,11 @@ LIB_PATH = os.path.join(LIB_DIR, "libespresso_hip.so")
 # Parts of the library that can be built alone (a checkout with nothing built that serves one model): the sources under csrc/.
 COMPONENTS = {
     "layered": [
-        "context.cpp", "decoder_runtime.cpp", "generation.cpp", "layered_runtime.cpp", "capi_runtime.cpp", "capi_engine.cpp", "capi_layered.cpp",
+        "context.cpp", "decoder_runtime.cpp", "generation.cpp", "layered_runtime.cpp", "layered_mixers.cpp", "capi_runtime.cpp", "capi_engine.cpp", "capi_layered.cpp",
         "host/engine.cpp", "host/runtime_registry.cpp", "host/layered_loader.cpp", "host/layered_config.cpp", "host/safetensors.cpp", "host/json_min.cpp",
         "host/model_support.cpp", "host/tokenizer.cpp", "host/regex_min.cpp", "kernels/decode_ops.hip", "kernels/dense_gemv.hip", "kernels/dense_gemm.hip",
-        "kernels/layer_ops.hip", "kernels/retention.hip", "kernels/latent_attention.hip",
+        "kernels/layer_ops.hip", "kernels/retention.hip", "kernels/mamba2.hip",
+        "kernels/latent_attention.hip", "kernels/window_attention.hip", "kernels/block_attention.hip",
     ],
 }
 

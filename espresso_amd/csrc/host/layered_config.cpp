@@ -12,7 +12,9 @@ void RotarySpec::frequencies(std::vector<double> *f, double *amplitude) const {
     f->resize(pairs);
     *amplitude = 1.0;
     for (int i = 0; i < pairs; i++) (*f)[i] = std::pow(base, -2.0 * i / dims);
-    if (!scaled) return;
+    if (scaling == Scaling::linear)
+        for (double &v : *f) v /= factor;
+    if (scaling != Scaling::yarn) return;
     const double two_pi = 6.283185307179586476925286766559;
     // the pair whose wave makes `turns` turns over the original context
     auto pair_at = [&](double turns) { return dims * std::log(original / (two_pi * turns)) / (2.0 * std::log(base)); };
@@ -25,12 +27,13 @@ void RotarySpec::frequencies(std::vector<double> *f, double *amplitude) const {
 }
 
 bool RotarySpec::operator==(const RotarySpec &o) const {
-    return dims == o.dims && base == o.base && interleaved == o.interleaved && scaled == o.scaled && factor == o.factor &&
+    return dims == o.dims && base == o.base && interleaved == o.interleaved && scaling == o.scaling && factor == o.factor &&
            original == o.original && fast == o.fast && slow == o.slow;
 }
 
 std::vector<LayeredConfig::TensorSpec> LayeredConfig::tensors() const {
-    std::vector<TensorSpec> t = {{"embed", vocab, width}, {"embed.norm", width, 0}};
+    std::vector<TensorSpec> t = {{"embed", vocab, width}};
+    if (embed_norm) t.push_back({"embed.norm", width, 0});
     for (size_t i = 0; i < layers.size(); i++) {
         const LayerSpec &L = layers[i];
         const std::string p = "l" + std::to_string(i) + ".", x = p + "mix.";
@@ -41,6 +44,21 @@ std::vector<LayeredConfig::TensorSpec> LayeredConfig::tensors() const {
             t.push_back({x + "k", L.heads * L.dim, width});
             t.push_back({x + "v", L.heads * L.vdim, width});
             t.push_back({x + "g", L.heads * L.vdim, width});
+        } else if (L.mixer == MixerKind::attention) {
+            t.push_back({x + "q", L.heads * L.dim, width});
+            t.push_back({x + "q.norm", L.heads * L.dim, 0});
+            if (L.kv_from < 0) {
+                t.push_back({x + "k", L.kv_heads * L.dim, width});
+                t.push_back({x + "k.norm", L.kv_heads * L.dim, 0});
+                t.push_back({x + "v", L.kv_heads * L.vdim, width});
+            }
+        } else if (L.mixer == MixerKind::mamba2) {
+            const int inner = L.heads * L.vdim, channels = inner + 2 * L.groups * L.state;
+            t.push_back({x + "in", inner + channels + L.heads, width});
+            t.push_back({x + "conv", channels, L.conv});
+            t.push_back({x + "conv.b", channels, 0});
+            for (const char *name : {"dt_bias", "A_log", "D"}) t.push_back({x + name, L.heads, 0});
+            t.push_back({x + "norm", inner, 0});
         } else {
             t.push_back({x + "q", L.heads * (L.dim + L.rot_dim), width});
             if (L.kv_from < 0) {
@@ -60,7 +78,7 @@ std::vector<LayeredConfig::TensorSpec> LayeredConfig::tensors() const {
         }
     }
     t.push_back({"final.norm", width, 0});
-    t.push_back({"head", vocab, width});
+    if (!tied_head) t.push_back({"head", vocab, width});
     return t;
 }
 
@@ -109,7 +127,8 @@ class Fields {
     bool ok_ = true;
 };
 
-bool parse_rotary(Fields &mixer, bool interleaved, int head_size, RotarySpec *r) {
+// `scaling`: what an object of that name means in this architecture.
+bool parse_rotary(Fields &mixer, bool interleaved, RotarySpec::Scaling scaling, int head_size, RotarySpec *r) {
     Fields f = mixer.object("rot");
     if (!mixer.take(f)) return false;
     r->dims = f.count("dims");
@@ -120,70 +139,117 @@ bool parse_rotary(Fields &mixer, bool interleaved, int head_size, RotarySpec *r)
     if (f.ok() && f.member("scaling")) {
         Fields s = f.object("scaling");
         if (f.take(s)) {
-            r->scaled = true;
+            r->scaling = scaling;
             r->factor = s.number("factor");
-            r->original = s.number("original");
-            r->fast = s.number("fast");
-            r->slow = s.number("slow");
-            if (s.ok() && !(r->factor > 0 && r->original > 0 && r->fast > 0 && r->slow > 0)) s.complain("factor", "or one of its neighbours is not positive");
+            if (s.ok() && !(r->factor > 0)) s.complain("factor", "is not positive");
+            if (scaling == RotarySpec::Scaling::yarn) {
+                r->original = s.number("original");
+                r->fast = s.number("fast");
+                r->slow = s.number("slow");
+                if (s.ok() && !(r->original > 0 && r->fast > 0 && r->slow > 0)) s.complain("original", "or one of its neighbours is not positive");
+            }
             f.take(s);
         }
     }
     return mixer.take(f);
 }
 
-// Layers of a retention or latent-attention mixer with a gated SiLU feed-forward.
-bool parse_layer(const JsonNode &node, size_t index, LayerSpec *L, std::string *error) {
+bool parse_window(Fields &mixer, LayerSpec *L) {
+    Fields m = mixer.object("mask");
+    if (!mixer.take(m)) return false;
+    L->window = m.count("size");
+    return mixer.take(m);
+}
+
+bool parse_retention(Fields &x, LayerSpec *L) {
+    L->mixer = MixerKind::retention;
+    L->dim = x.count("dim");
+    L->vdim = x.count("vdim");
+    if (!x.ok() || !parse_rotary(x, false, RotarySpec::Scaling::yarn, L->dim, &L->rot)) return false;
+    const JsonNode *d = x.member("decay");
+    if (!d || !d->is(JsonNode::Array) || (int)d->items.size() != L->heads) { x.complain("decay", "does not list one decay per head"); return false; }
+    for (const JsonNode &v : d->items) {
+        if (!v.is(JsonNode::Number) || v.number < 0) { x.complain("decay", "holds something other than a decay"); return false; }
+        L->decay.push_back(v.number);
+    }
+    return true;
+}
+
+bool parse_latent_attention(Fields &x, LayerSpec *L) {
+    L->mixer = MixerKind::latent_attention;
+    L->dim = x.count("dim");
+    L->vdim = x.count("vdim");
+    L->kv_rank = x.count("kv_rank");
+    L->rot_dim = x.count("rot_dim");
+    L->scale = x.number("scale");
+    if (!x.ok() || !parse_rotary(x, true, RotarySpec::Scaling::yarn, L->rot_dim, &L->rot) || !parse_window(x, L)) return false;
+    if (x.member("kv_from")) L->kv_from = x.count("kv_from", 0);
+    return x.ok();
+}
+
+// Grouped heads, normed queries and keys, rotation of a part of a head in halves, a sliding window.
+bool parse_attention(Fields &x, LayerSpec *L) {
+    L->mixer = MixerKind::attention;
+    L->dim = x.count("dim");
+    L->vdim = x.count("vdim");
+    L->kv_heads = x.count("kv_heads");
+    L->scale = x.number("scale");
+    if (x.ok() && L->heads % L->kv_heads) x.complain("kv_heads", "does not divide the query heads");
+    if (!x.ok() || !parse_rotary(x, false, RotarySpec::Scaling::linear, L->dim, &L->rot) || !parse_window(x, L)) return false;
+    if (x.member("kv_from")) L->kv_from = x.count("kv_from", 0);
+    return x.ok();
+}
+
+bool parse_mamba2(Fields &x, LayerSpec *L) {
+    L->mixer = MixerKind::mamba2;
+    L->vdim = x.count("vdim");
+    L->state = x.count("state");
+    L->groups = x.count("groups");
+    L->conv = x.count("conv");
+    L->norm_groups = x.count("norm_groups");
+    if (x.ok() && L->heads % L->groups) x.complain("groups", "does not divide the heads");
+    if (x.ok() && (long long)L->heads * L->vdim % L->norm_groups) x.complain("norm_groups", "does not divide the values of all heads");
+    return x.ok();
+}
+
+struct MixerReader {
+    const char *type;
+    bool (*parse)(Fields &mixer, LayerSpec *L);
+};
+
+// The members every architecture's layers have: a mixer of one of the given types, and a gated feed-forward or none.
+bool parse_layer(const JsonNode &node, size_t index, const std::vector<MixerReader> &mixers, Activation activation, LayerSpec *L, std::string *error) {
     Fields f(&node, "layers[" + std::to_string(index) + "].", error);
     const std::string type = f.string("type");
     Fields x = f.object("mixer");
     if (!f.ok()) return false;
     L->heads = x.count("heads");
-    L->dim = x.count("dim");
-    L->vdim = x.count("vdim");
     if (!x.ok()) return false;
-    if (type == "retention") {
-        L->mixer = MixerKind::retention;
-        if (!parse_rotary(x, false, L->dim, &L->rot)) return false;
-        const JsonNode *d = x.member("decay");
-        if (!d || !d->is(JsonNode::Array) || (int)d->items.size() != L->heads) { x.complain("decay", "does not list one decay per head"); return false; }
-        for (const JsonNode &v : d->items) {
-            if (!v.is(JsonNode::Number) || v.number < 0) { x.complain("decay", "holds something other than a decay"); return false; }
-            L->decay.push_back(v.number);
-        }
-    } else if (type == "latent_attention") {
-        L->mixer = MixerKind::latent_attention;
-        L->kv_rank = x.count("kv_rank");
-        L->rot_dim = x.count("rot_dim");
-        L->scale = x.number("scale");
-        if (!x.ok() || !parse_rotary(x, true, L->rot_dim, &L->rot)) return false;
-        Fields m = x.object("mask");
-        if (!x.take(m)) return false;
-        L->window = m.count("size");
-        if (!x.take(m)) return false;
-        if (x.member("kv_from")) L->kv_from = x.count("kv_from", 0);
-    } else {
-        f.complain("type", ("names no mixer of this library: " + type).c_str());
-        return false;
-    }
-    if (!x.ok()) return false;
+    const MixerReader *reader = nullptr;
+    for (const MixerReader &r : mixers) if (type == r.type) reader = &r;
+    if (!reader) { f.complain("type", ("names no mixer of this architecture: " + type).c_str()); return false; }
+    if (!reader->parse(x, L) || !x.ok()) return false;
     if (f.member("mlp")) {
         Fields m = f.object("mlp");
         if (!f.take(m)) return false;
         if (m.string("kind") != "dense" && m.ok()) m.complain("kind", "is not dense");
         L->ff = m.count("ff");
+        L->activation = activation;
         if (!m.ok()) return false;
     }
     return true;
 }
 
-bool parse_ranavik(const JsonNode &root, LayeredConfig *c, std::string *error) {
-    Fields f(&root, "", error);
-    c->block = BlockKind::parallel_two_norms;
+// Whether a layer can read the other one's cache.
+bool cache_fits(const LayerSpec &L, const LayerSpec &source) {
+    if (source.mixer != L.mixer || source.kv_from >= 0 || !(source.rot == L.rot)) return false;
+    if (L.mixer == MixerKind::latent_attention) return source.kv_rank == L.kv_rank && source.rot_dim == L.rot_dim;
+    return source.heads == L.heads && source.kv_heads == L.kv_heads && source.dim == L.dim && source.vdim == L.vdim;
+}
+
+bool parse_model(Fields &f, const std::vector<MixerReader> &mixers, Activation activation, LayeredConfig *c, std::string *error) {
     c->vocab = f.count("vocab");
     c->width = f.count("width");
-    c->residual_mult = f.number("residual_mult");
-    c->logit_softcap = f.number_or("logit_softcap", 0.0);
     Fields n = f.object("norm");
     if (!f.take(n)) return false;
     c->norm_eps = n.number("eps");
@@ -192,25 +258,38 @@ bool parse_ranavik(const JsonNode &root, LayeredConfig *c, std::string *error) {
     if (!layers || !layers->is(JsonNode::Array) || layers->items.empty()) { f.complain("layers", "is not a list of layers"); return false; }
     for (size_t i = 0; i < layers->items.size(); i++) {
         LayerSpec L;
-        if (!parse_layer(layers->items[i], i, &L, error)) return false;
+        if (!parse_layer(layers->items[i], i, mixers, activation, &L, error)) return false;
         if (L.kv_from >= 0) {
             const std::string at = "config.json: layers[" + std::to_string(i) + "].mixer.kv_from ";
             if (L.kv_from >= (int)i) { if (error) *error = at + "does not name an earlier layer"; return false; }
-            const LayerSpec &S = c->layers[L.kv_from];
-            if (S.mixer != MixerKind::latent_attention || S.kv_from >= 0 || S.kv_rank != L.kv_rank || S.rot_dim != L.rot_dim || !(S.rot == L.rot)) {
-                if (error) *error = at + "names a layer without fitting latents of its own";
-                return false;
-            }
+            if (!cache_fits(L, c->layers[L.kv_from])) { if (error) *error = at + "names a layer without a fitting cache of its own"; return false; }
         }
         c->layers.push_back(L);
     }
     return true;
 }
 
+bool parse_ranavik(const JsonNode &root, LayeredConfig *c, std::string *error) {
+    Fields f(&root, "", error);
+    c->block = BlockKind::parallel_two_norms;
+    c->residual_mult = f.number("residual_mult");
+    c->logit_softcap = f.number_or("logit_softcap", 0.0);
+    return parse_model(f, {{"retention", parse_retention}, {"latent_attention", parse_latent_attention}}, Activation::silu, c, error);
+}
+
+// Mamba-2 layers come in two kinds of equal mechanism, each with sizes of its own.
+bool parse_forovik(const JsonNode &root, LayeredConfig *c, std::string *error) {
+    Fields f(&root, "", error);
+    c->block = BlockKind::sequential_post_norms;
+    c->embed_norm = false;
+    c->tied_head = true;
+    return parse_model(f, {{"attention", parse_attention}, {"mamba2", parse_mamba2}, {"mamba2_2", parse_mamba2}}, Activation::gelu_tanh, c, error);
+}
+
 }  // namespace
 
 const std::vector<LayeredArchitecture> &layered_architectures() {
-    static const std::vector<LayeredArchitecture> table = {{"Ranavik", parse_ranavik}};
+    static const std::vector<LayeredArchitecture> table = {{"Ranavik", parse_ranavik}, {"Forovik", parse_forovik}};
     return table;
 }
 

@@ -13,14 +13,17 @@ struct RotarySpec {
     int dims = 0;
     double base = 0;
     bool interleaved = false;        // pairs (2i, 2i + 1); otherwise (i, i + dims / 2)
-    bool scaled = false;             // YaRN: frequencies between the `fast` and `slow` turn counts blend towards 1 / factor
+    // linear: every frequency over the factor.  yarn: frequencies between the `fast` and `slow` turn counts blend towards 1 / factor
+    enum class Scaling { none, linear, yarn } scaling = Scaling::none;
     double factor = 1, original = 0, fast = 0, slow = 0;
     // frequency of every pair, and the factor on cosine and sine
     void frequencies(std::vector<double> *f, double *amplitude) const;
     bool operator==(const RotarySpec &o) const;
 };
 
-enum class MixerKind { retention, latent_attention };
+enum class MixerKind { retention, latent_attention, attention, mamba2 };
+inline bool has_cache(MixerKind m) { return m == MixerKind::latent_attention || m == MixerKind::attention; }
+enum class Activation { silu, gelu_tanh };   // of a gated feed-forward's gate
 
 struct LayerSpec {
     MixerKind mixer = MixerKind::retention;
@@ -28,21 +31,28 @@ struct LayerSpec {
     RotarySpec rot;
     std::vector<double> decay;       // retention: one per head
     int kv_rank = 0, rot_dim = 0;    // latent attention: latent size, size of the shared rotated key part
-    int kv_from = -1;                // latent attention: the layer whose cached latents this layer reads (-1: its own)
-    int window = 0;                  // latent attention: a token sees itself and the window - 1 tokens before it
+    int kv_heads = 0;                // attention: query head h reads key and value head h / (heads / kv_heads)
+    int kv_from = -1;                // either attention: the layer whose cache this layer reads (-1: its own)
+    int window = 0;                  // either attention: a token sees itself and the window - 1 tokens before it
     double scale = 0;
+    int state = 0, groups = 0;       // mamba2: state size; groups of heads that share B and C
+    int conv = 0, norm_groups = 0;   // mamba2: taps of the causal convolution; parts of the output norm
     int ff = 0;                      // width of the gated feed-forward, 0 = none
+    Activation activation = Activation::silu;
 };
 
 // How a layer's branches join the residual stream.
 enum class BlockKind {
     parallel_two_norms,              // x + m * (mixer(norm1 x) + ff(norm2 x))
+    sequential_post_norms,           // x + norm1(mixer(x)), then x + norm2(ff(x))
 };
 
 struct LayeredConfig {
     std::string architecture;
     BlockKind block = BlockKind::parallel_two_norms;
     int vocab = 0, width = 0;
+    bool embed_norm = true;          // the embedding is normed ("embed.norm")
+    bool tied_head = false;          // the head is the embedding table (no "head")
     double norm_eps = 0, residual_mult = 1, logit_softcap = 0;   // softcap 0 = none
     std::vector<LayerSpec> layers;
     // [(name, rows, cols)] of every tensor a model of this configuration has (cols 0: a vector)

@@ -83,9 +83,16 @@ class SyntheticWeights : public LayeredWeights {
     }
     int vector(const std::string &name, int count, std::vector<float> *out) override {
         SplitMix64 g{seed_ ^ start(name)};
-        const bool sink = name.size() >= 4 && name.compare(name.size() - 4, 4, "sink") == 0;
+        auto is = [&](const char *end) { const size_t n = std::strlen(end); return name.size() >= n && name.compare(name.size() - n, n, end) == 0; };
         out->resize(count);
-        for (float &v : *out) v = (float)(sink ? g.unit() - 0.5 : 0.9 + 0.2 * g.unit());
+        for (float &v : *out) {
+            const double u = g.unit();
+            if (is("sink")) v = (float)(u - 0.5);
+            else if (is("A_log")) v = (float)std::log(1.0 + 15.0 * u);   // decays and step sizes of a trained model's range
+            else if (is("dt_bias")) v = (float)(-6.9 + 4.6 * u);
+            else if (is("conv.b")) v = (float)(0.1 * (u - 0.5));
+            else v = (float)(0.9 + 0.2 * u);
+        }
         return ESP_OK;
     }
 
@@ -118,7 +125,7 @@ int layered_model_config(const std::string &model_dir, int max_seq, MultiModelCo
     m.name = c.architecture;
     m.architecture = MultiModelConfig::Architecture::layered;
     m.nLayer = (int)c.layers.size(); m.dModel = c.width; m.vocab = c.vocab; m.maxSeq = max_seq; m.normEps = (float)c.norm_eps;
-    m.nHead = m.nKVHead = c.layers[0].heads; m.headDim = c.layers[0].dim;   // layers differ: the first one's, for reports
+    m.nHead = m.nKVHead = c.layers[0].heads; m.headDim = c.layers[0].dim ? c.layers[0].dim : c.layers[0].vdim;   // layers differ: the first one's, for reports
     for (const LayerSpec &L : c.layers) m.hiddenDim = std::max(m.hiddenDim, L.ff);
     *out = m;
     return ESP_OK;

@@ -31,7 +31,7 @@ struct DenseGemmArgs {
     void *y;
     int ldy, mix_cols;
     void *act;
-    int ld_act, n_store;
+    int ld_act, gate_function, n_store;
     float cap;
 };
 
@@ -75,7 +75,7 @@ __global__ __launch_bounds__(64 * WM * WN) void dense_gemm_kernel(DenseGemmArgs 
     const int m0 = mt * BM, n0 = nt * BN;
     const int t_begin = blockIdx.y * a.tiles_per_split;
     const int t_end = t_begin + a.tiles_per_split < a.tiles ? t_begin + a.tiles_per_split : a.tiles, t_last = t_end - 1;
-    const bool after_mix = a.out == (int)GemmOut::mix_swiglu && n0 >= a.mix_cols;
+    const bool after_mix = a.out == (int)GemmOut::mix_gated && n0 >= a.mix_cols;
     const TA *ap = static_cast<const TA *>(after_mix ? a.a2 : a.a);
     const TB *bp = static_cast<const TB *>(a.b);
 
@@ -166,12 +166,12 @@ __global__ __launch_bounds__(64 * WM * WN) void dense_gemm_kernel(DenseGemmArgs 
                 if (after_mix) {   // even lanes hold gates, their right neighbours the ups
                     const float up = __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, v), 0xB1, 0xF, 0xF, false));   // quad_perm [1,0,3,2]
                     if (!(lane & 1) && m < a.m && n < a.n)
-                        static_cast<E *>(a.act)[(size_t)m * a.ld_act + (n - a.mix_cols) / 2] = Op<E>::from_float(matrix::silu(v) * up);
+                        static_cast<E *>(a.act)[(size_t)m * a.ld_act + (n - a.mix_cols) / 2] = Op<E>::from_float(matrix::gated(a.gate_function, v, up));
                     continue;
                 }
                 if (m >= a.m || n >= a.n) continue;
                 if (a.out == (int)GemmOut::planes) static_cast<float *>(a.y)[((size_t)blockIdx.y * a.m + m) * a.ldy + n] = v;
-                else if (a.out == (int)GemmOut::mix_swiglu) static_cast<float *>(a.y)[(size_t)m * a.ldy + n] = v;
+                else if (a.out == (int)GemmOut::mix_gated) static_cast<float *>(a.y)[(size_t)m * a.ldy + n] = v;
                 else if (a.out == (int)GemmOut::elems) static_cast<E *>(a.y)[(size_t)m * a.ldy + n] = Op<E>::from_float(v);
                 else if (n < a.n_store) static_cast<float *>(a.y)[(size_t)m * a.ldy + n] = a.cap > 0.0f ? a.cap * tanhf(v / a.cap) : v;
             }
@@ -198,7 +198,7 @@ hipError_t run(const DenseGemm &p, hipStream_t s) {
     a.tiles_per_split = ceil_div(a.tiles, p.splits);
     if ((p.splits - 1) * a.tiles_per_split >= a.tiles) return hipErrorInvalidValue;   // a split without work would leave its plane unwritten
     a.m_tiles = ceil_div(p.m, t.bm); a.n_tiles = ceil_div(p.n, t.bn);
-    a.out = (int)p.out; a.y = p.y; a.ldy = p.ldy; a.mix_cols = p.mix_cols; a.act = p.act; a.ld_act = p.ld_act; a.n_store = p.n_store; a.cap = p.cap;
+    a.out = (int)p.out; a.y = p.y; a.ldy = p.ldy; a.mix_cols = p.mix_cols; a.act = p.act; a.ld_act = p.ld_act; a.gate_function = (int)p.gate_function; a.n_store = p.n_store; a.cap = p.cap;
     const dim3 grid(ceil_div(a.n_tiles, kDies) * kDies * a.m_tiles, p.splits);
     if constexpr (!f32) {
         if (t.bm == 32) {
@@ -227,9 +227,10 @@ int gemm_planes_splits(int m, int n, int k, size_t workspace_floats) {
 }
 
 hipError_t launch_dense_gemm(const DenseGemm &p, hipStream_t s) {
-    if (!p.a || !p.b || !p.y || p.m < 1 || p.n < 1 || p.k < 64 || p.k % 64 || p.splits < 1 || p.lda < p.k || p.ldb < p.k || p.lda % 8 || p.ldb % 8) return hipErrorInvalidValue;
+    const bool gated_only = p.out == GemmOut::mix_gated && p.mix_cols == 0;
+    if (!p.a || !p.b || (!p.y && !gated_only) || p.m < 1 || p.n < 1 || p.k < 64 || p.k % 64 || p.splits < 1 || p.lda < p.k || p.ldb < p.k || p.lda % 8 || p.ldb % 8) return hipErrorInvalidValue;
     if (p.out != GemmOut::planes && p.splits != 1) return hipErrorInvalidValue;
-    if (p.out == GemmOut::mix_swiglu && (p.mix_cols % 128 || p.n % 2 || (p.n > p.mix_cols && (!p.a2 || !p.act)))) return hipErrorInvalidValue;
+    if (p.out == GemmOut::mix_gated && (p.mix_cols % 128 || p.n % 2 || (p.n > p.mix_cols && (!p.a2 || !p.act)))) return hipErrorInvalidValue;
     if (p.a_type == Precision::bf16 && p.b_type == Precision::bf16) return run<uint16_t, uint16_t>(p, s);
     if (p.a_type == Precision::f32 && p.b_type == Precision::bf16) return run<float, uint16_t>(p, s);
     if (p.a_type == Precision::bf16 && p.b_type == Precision::f32) return run<uint16_t, float>(p, s);

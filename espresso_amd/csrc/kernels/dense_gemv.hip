@@ -7,7 +7,8 @@
 //     of their own, so that a lane's two 128-bit reads are free of bank conflicts) and then walks units of weight rows: four rows per
 //     wavefront, two or one where the matrix has too few rows to give every compute unit work (the loads run further ahead then);
 //   * what surrounds the product lives in the staging and the epilogue: RMS norm (its scale factors out of the dot product), the
-//     per-head norm and gate of a retention output, SiLU(gate) * up, the residual sum, the soft cap of the logits;
+//     per-head norm and gate of a retention output, the norm by parts of a Mamba-2 output, f(gate) * up, the residual sum, the soft cap
+//     of the logits; where branches are normed as they join the stream, that sum too (the first workgroup keeps it);
 //   * the input side of a parallel layer is one launch over two activation rows: workgroups are dealt to the mixer's rows (norm1)
 //     and the feed-forward's (norm2) in proportion.
 #include <hip/hip_runtime.h>
@@ -31,11 +32,18 @@ struct DenseGemvArgs {
     int units_a, units_b, blocks_a;     // KIND_IN: units of the mixer and of the feed-forward; workgroups of the mixer
     int mix_rows;
     const float *x, *norm_a, *norm_b;
+    const float *branch, *branch_norm;
+    float *x_out;
+    int gate_function;
     int width;
     float eps;
     float *y, *act_out;
     const float *mix, *act, *squares, *gate;
     int mix_cols, act_at, act_cols, parts, heads, vdim, vdim_p;
+    const int *part_of, *part_starts;   // KIND_OUT: norm by parts
+    const float *part_norm;
+    int part_count, part_pieces;
+    float part_size;
     float mult, cap;
     const float *residual;
     int vocab;
@@ -50,8 +58,8 @@ __device__ __forceinline__ int staged_at(int k, int k_pad) { return (k >> 3) * 4
 template <int KIND, int RPW, int AHEAD>
 __global__ __launch_bounds__(kGemvThreads) void dense_gemv_kernel(DenseGemvArgs a) {
     constexpr int kUnitRows = kGemvWaves * RPW;
-    extern __shared__ float xs[];   // [k_pad], then [heads]
-    __shared__ float red[kGemvWaves];
+    extern __shared__ float xs[];   // [k_pad], then [heads] or [part_count * part_pieces]
+    __shared__ float red[2 * kGemvWaves];
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
     const bool second = KIND == KIND_IN && (int)blockIdx.x >= a.blocks_a;
     float scale = 1.0f;
@@ -79,6 +87,79 @@ __global__ __launch_bounds__(kGemvThreads) void dense_gemv_kernel(DenseGemvArgs 
                 v = *reinterpret_cast<const float4 *>(a.act + (k - a.act_at));
             }
             *reinterpret_cast<float4 *>(xs + staged_at(k, a.k_pad)) = v;
+        }
+        __syncthreads();
+        if (a.part_of) {   // sums of squares of every part, in part_pieces shares; then the values in place
+            for (int i = wave; i < a.part_count * a.part_pieces; i += kGemvWaves) {
+                const int g = i / a.part_pieces, to = a.part_starts[g + 1];
+                float s = 0.0f;
+                for (int k = a.part_starts[g] + (i % a.part_pieces) * 64 + lane; k < to; k += 64 * a.part_pieces) {
+                    const float v = xs[staged_at(k, a.k_pad)];
+                    s += v * v;
+                }
+                s = wave_sum(s);
+                if (lane == 0) head_inv[i] = s;
+            }
+            __syncthreads();
+            for (int k = tid * 4; k < a.mix_cols; k += kGemvThreads * 4) {
+                const int4 g = *reinterpret_cast<const int4 *>(a.part_of + k);
+                const float4 n = *reinterpret_cast<const float4 *>(a.part_norm + k);
+                auto scale_of = [&](int part) {
+                    float s = 0.0f;
+                    for (int i = 0; i < a.part_pieces; i++) s += head_inv[part * a.part_pieces + i];
+                    return 1.0f / sqrtf(s / a.part_size + a.eps);
+                };
+                const float f = scale_of(g.x), l = g.w == g.x ? f : scale_of(g.w);
+                float4 v = *reinterpret_cast<const float4 *>(xs + staged_at(k, a.k_pad));
+                v.x *= f * n.x;
+                v.y *= (g.y == g.x ? f : g.y == g.w ? l : scale_of(g.y)) * n.y;
+                v.z *= (g.z == g.x ? f : g.z == g.w ? l : scale_of(g.z)) * n.z;
+                v.w *= l * n.w;
+                *reinterpret_cast<float4 *>(xs + staged_at(k, a.k_pad)) = v;
+            }
+            __syncthreads();
+        }
+    } else if (KIND == KIND_IN && !a.norm_a) {
+        // the stream as it is, or with a branch that is normed as it joins; both are kept in registers up to 8192 columns
+        constexpr int kHeld = 4;
+        float4 x[kHeld], b[kHeld], g[kHeld];
+        const float4 zero = make_float4(0.f, 0.f, 0.f, 0.f);
+        auto at = [](const float *p, int k) { return *reinterpret_cast<const float4 *>(p + k); };
+        float s = 0.0f, inv = 0.0f;
+#pragma unroll
+        for (int c = 0; c < kHeld; c++) {
+            const int k = (tid + c * kGemvThreads) * 4;
+            const bool in = k < a.ld;
+            x[c] = in ? at(a.x, k) : zero;
+            b[c] = in && a.branch ? at(a.branch, k) : zero;
+            g[c] = in && a.branch ? at(a.branch_norm, k) : zero;
+        }
+        if (a.branch) {
+#pragma unroll
+            for (int c = 0; c < kHeld; c++) s += b[c].x * b[c].x + b[c].y * b[c].y + b[c].z * b[c].z + b[c].w * b[c].w;
+            for (int k = (tid + kHeld * kGemvThreads) * 4; k < a.ld; k += kGemvThreads * 4) {
+                const float4 v = at(a.branch, k);
+                s += v.x * v.x + v.y * v.y + v.z * v.z + v.w * v.w;
+            }
+            s = wave_sum(s);
+            if (lane == 0) red[wave] = s;
+            __syncthreads();
+            const float total = ((red[0] + red[1]) + (red[2] + red[3])) + ((red[4] + red[5]) + (red[6] + red[7]));
+            inv = 1.0f / sqrtf(total / (float)a.width + a.eps);
+        }
+        auto put = [&](int k, float4 v, const float4 &y, const float4 &w) {
+            v.x += y.x * inv * w.x; v.y += y.y * inv * w.y; v.z += y.z * inv * w.z; v.w += y.w * inv * w.w;
+            *reinterpret_cast<float4 *>(xs + staged_at(k, a.k_pad)) = v;
+            if (a.branch && blockIdx.x == 0 && k < a.ld) *reinterpret_cast<float4 *>(a.x_out + k) = v;
+        };
+#pragma unroll
+        for (int c = 0; c < kHeld; c++) {
+            const int k = (tid + c * kGemvThreads) * 4;
+            if (k < a.k_pad) put(k, x[c], b[c], g[c]);
+        }
+        for (int k = (tid + kHeld * kGemvThreads) * 4; k < a.k_pad; k += kGemvThreads * 4) {
+            const bool in = k < a.ld;
+            put(k, in ? at(a.x, k) : zero, in && a.branch ? at(a.branch, k) : zero, in && a.branch ? at(a.branch_norm, k) : zero);
         }
         __syncthreads();
     } else {
@@ -153,11 +234,11 @@ __global__ __launch_bounds__(kGemvThreads) void dense_gemv_kernel(DenseGemvArgs 
             } else {
                 const int i = (row0 - a.mix_rows) / 2;
 #pragma unroll
-                for (int r = 0; r + 1 < RPW; r += 2) a.act_out[i + r / 2] = matrix::silu(acc[r]) * acc[r + 1];
+                for (int r = 0; r + 1 < RPW; r += 2) a.act_out[i + r / 2] = matrix::gated(a.gate_function, acc[r], acc[r + 1]);
             }
         } else if constexpr (KIND == KIND_OUT) {
 #pragma unroll
-            for (int r = 0; r < RPW; r++) a.y[row0 + r] = a.residual[row0 + r] + a.mult * acc[r];
+            for (int r = 0; r < RPW; r++) a.y[row0 + r] = a.residual ? a.residual[row0 + r] + a.mult * acc[r] : acc[r];
         } else {
 #pragma unroll
             for (int r = 0; r < RPW; r++) {
@@ -194,7 +275,7 @@ int resident_workgroups() {
 
 template <int KIND, int RPW, int AHEAD>
 hipError_t run(DenseGemvArgs a, int grid, hipStream_t s) {
-    const size_t lds = (size_t)(a.k_pad + a.heads) * 4;
+    const size_t lds = (size_t)(a.k_pad + a.heads + a.part_count * a.part_pieces) * 4;
     if (lds > 150 * 1024 || grid < 1) return hipErrorInvalidValue;
     static size_t allowed = 0;
     if (lds > 48 * 1024 && lds > allowed) {
@@ -211,18 +292,20 @@ int at_most(int units) { return units < resident_workgroups() ? units : resident
 }  // namespace
 
 hipError_t launch_dense_gemv_in(const DenseGemvIn &p, hipStream_t s) {
-    if (!p.w.w || p.w.ld % 64 || p.mix_rows % kRowAlign || p.w.rows % kRowAlign || p.w.rows < p.mix_rows || p.mix_rows < kRowAlign) return hipErrorInvalidValue;
+    if (!p.w.w || p.w.ld % 64 || p.mix_rows % kRowAlign || p.w.rows % kRowAlign || p.w.rows < p.mix_rows || p.w.rows < kRowAlign || p.mix_rows < 0) return hipErrorInvalidValue;
+    if ((p.branch && (!p.branch_norm || !p.x_out || p.x_out == p.x || p.norm1)) || (p.w.rows > p.mix_rows && p.mix_rows && !p.norm1 != !p.norm2)) return hipErrorInvalidValue;
     DenseGemvArgs a{};
     a.w = p.w.w; a.ld = p.w.ld; a.k_pad = round_up(p.w.ld, kStep); a.mix_rows = p.mix_rows;
     a.x = p.x; a.norm_a = p.norm1; a.norm_b = p.norm2; a.width = p.width; a.eps = p.eps; a.y = p.y; a.act_out = p.act;
+    a.branch = p.branch; a.branch_norm = p.branch_norm; a.x_out = p.x_out; a.gate_function = (int)p.gate_function;
     const int unit = p.w.rows >= resident_workgroups() * kGemvWaves * 4 ? kGemvWaves * 4 : kGemvWaves * 2;   // (gate, up) pairs stay together
     a.units_a = p.mix_rows / unit; a.units_b = (p.w.rows - p.mix_rows) / unit;
     const int units = a.units_a + a.units_b, wanted = at_most(units);
     a.blocks_a = (int)((long long)wanted * a.units_a / units);
-    if (a.blocks_a < 1) a.blocks_a = 1;
+    if (a.blocks_a < 1 && a.units_a) a.blocks_a = 1;
     int grid = wanted;
     if (a.units_b == 0) a.blocks_a = grid;
-    else if (a.blocks_a >= grid) grid = a.blocks_a + 1;
+    else if (a.units_a && a.blocks_a >= grid) grid = a.blocks_a + 1;
     return unit == kGemvWaves * 4 ? run<KIND_IN, 4, 2>(a, grid, s) : run<KIND_IN, 2, 3>(a, grid, s);
 }
 
@@ -230,8 +313,11 @@ hipError_t launch_dense_gemv_out(const DenseGemvOut &p, hipStream_t s) {
     if (!p.w.w || p.w.ld % 64 || p.rows % kRowAlign || p.w.rows < p.rows || p.mix_cols % 32 || p.act_cols % 32 || p.act_at < p.mix_cols || p.act_at + p.act_cols > p.w.ld || p.rows < kRowAlign)
         return hipErrorInvalidValue;
     if (p.squares && (p.vdim_p <= 0 || p.mix_cols % p.vdim_p || !p.gate)) return hipErrorInvalidValue;
+    if (p.part_of && (p.squares || p.part_count < 1 || !p.part_starts || !p.part_norm || !(p.part_size > 0))) return hipErrorInvalidValue;
     DenseGemvArgs a{};
     a.w = p.w.w; a.ld = p.w.ld; a.k_pad = round_up(p.w.ld, kStep);
+    a.part_of = p.part_of; a.part_starts = p.part_starts; a.part_norm = p.part_norm; a.part_count = p.part_of ? p.part_count : 0; a.part_size = p.part_size;
+    a.part_pieces = !p.part_of || p.part_count >= kGemvWaves ? 1 : kGemvWaves / p.part_count;
     a.mix = p.mix; a.act = p.act; a.squares = p.squares; a.gate = p.gate; a.mix_cols = p.mix_cols; a.act_at = p.act_at; a.act_cols = p.act_cols; a.parts = p.parts;
     a.heads = p.squares ? p.mix_cols / p.vdim_p : 0; a.vdim = p.vdim; a.vdim_p = p.vdim_p; a.eps = p.eps; a.mult = p.mult; a.residual = p.residual; a.y = p.out;
     const int cus = resident_workgroups() / 2;   // long rows: a workgroup per compute unit

@@ -10,9 +10,7 @@
 // window go to different workgroups, which leave (maximum, sum, weighted latents); the merge adds the sink once.
 //
 // Prompt blocks (launch_latent_block): keys and values of the visible span are products of the gathered latents (done by the
-// caller as two dense products, values transposed), then attention in tiles of 64 keys: a wavefront owns 32 queries and half of every tile; scores are
-// computed transposed (keys as rows), so a lane holds one query's column, the softmax needs one exchange between the lane halves,
-// and the weights are the B operand of the value product without passing through LDS.
+// caller as two dense products, values transposed), then attention in tiles of 64 keys (block_attention.hip).
 // With bf16 operands queries of the decode form and softmax weights enter the products as a high and a low bf16.
 #include <hip/hip_runtime.h>
 
@@ -125,13 +123,6 @@ struct PartialLayout {   // LDS of latent_partial_kernel: a tile of 32 cached ro
 };
 typedef uint32_t uintx4 __attribute__((ext_vector_type(4)));
 
-// Products and exponentials of scores: bf16 models use the hardware's exponential directly.
-template <typename T>
-__device__ __forceinline__ float weight_exp(float x) {
-    if constexpr (Op<T>::kSplit) return __expf(x);
-    else return expf(x);
-}
-
 // grid (splits, groups of 32 heads, rows).  NT: tiles of 32 ranks per wavefront.  KS: rows of up to 128 KS values have their queries
 // and the next tile in registers (KS steps of 16 per wavefront, KS pieces of eight per thread); 0: any width, from memory as needed.
 template <typename T, int NT, int KS>
@@ -229,10 +220,10 @@ __global__ __launch_bounds__(kPartialThreads) void latent_partial_kernel(LatentS
             best = fmaxf(best, w[r]);
         }
         best = fmaxf(fmaxf(best, __shfl_xor(best, 32)), top);
-        const float keep = weight_exp<T>(top - best);
+        const float keep = matrix::weight_exp<T>(top - best);
         float add = 0.0f;
 #pragma unroll
-        for (int r = 0; r < 16; r++) { w[r] = weight_exp<T>(w[r] - best); add += w[r]; }
+        for (int r = 0; r < 16; r++) { w[r] = matrix::weight_exp<T>(w[r] - best); add += w[r]; }
         add += __shfl_xor(add, 32);
         sum = sum * keep + add;
         top = best;
@@ -356,157 +347,6 @@ __global__ __launch_bounds__(256) void latent_queries_kernel(LatentShape l, Late
     }
 }
 
-constexpr int kQueries = 64, kKeys = 64, kValues = 128;   // per workgroup and tile
-template <typename T>
-struct BlockLayout {
-    static constexpr int kPad = 16 / sizeof(T);
-    static size_t bytes(int qk) {
-        const size_t tiles = ((size_t)kKeys * (qk + kPad) + (size_t)kValues * (kKeys + kPad)) * sizeof(T), merge = (size_t)2 * 64 * 66 * 4;
-        return tiles > merge ? tiles : merge;
-    }
-};
-
-// grid (blocks of 64 queries, heads, slices of 128 values).  Wavefront w takes queries 32 (w % 2) .. and, of every tile of 64 keys, keys
-// 32 (w / 2) ..; the two halves' softmax states meet in LDS at the end.  NQ: steps of 16 query dimensions held in registers (the next
-// tile too), 0 = any number, read when needed.
-template <typename T, int NQ>
-__global__ __launch_bounds__(256) void latent_block_kernel(LatentShape l, LatentBlock p, int rows_p) {
-    extern __shared__ char smem[];
-    constexpr int kPad = BlockLayout<T>::kPad, LDV = kKeys + kPad, kVec = sizeof(T) / 2;
-    constexpr int PK = NQ ? NQ / 2 : 1, PV = kValues * kKeys / 8 / 256;   // pieces of eight per thread: keys (64 rows of 2 NQ pieces), values
-    const int qk = l.dim_p + l.rot_p, ldk = qk + kPad;
-    T *kt = reinterpret_cast<T *>(smem), *vt = kt + kKeys * ldk;
-    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, half = lane >> 5, col = lane & 31, qt = wave & 1, set = wave >> 1;
-    const int h = blockIdx.y, q0 = blockIdx.x * kQueries, v0 = blockIdx.z * kValues;
-    const int values = l.vdim_p - v0 < kValues ? l.vdim_p - v0 : kValues;
-    const int m = q0 + qt * 32 + col, at = p.base - p.first_key + m;   // this lane's query: row and place among the keys
-    const int wave_at = p.base - p.first_key + q0 + qt * 32;           // the wavefront's first query
-    const int block_at = p.base - p.first_key + q0, seen = block_at - l.window + 1;
-    const int k_begin = seen > 0 ? seen / kKeys * kKeys : 0;
-    const int last = q0 + kQueries < p.rows ? q0 + kQueries : p.rows, k_end = p.base - p.first_key + last;
-    const int row_pieces = l.dim_p / 8, k_pieces = row_pieces + l.rot_p / 8;
-    const T *keys = static_cast<const T *>(p.k) + h * l.dim_p, *key_rot = static_cast<const T *>(p.key_rot);
-    const T *vals = static_cast<const T *>(p.vt) + ((size_t)h * l.vdim_p + v0) * p.keys_p;
-    auto key_piece = [&](int k0, int i) {
-        const int row = i / k_pieces, part = i % k_pieces;
-        return reinterpret_cast<const uintx4 *>(part < row_pieces ? keys + (size_t)(k0 + row) * l.heads * l.dim_p + part * 8 : key_rot + (size_t)(k0 + row) * l.rot_p + (part - row_pieces) * 8);
-    };
-    auto value_piece = [&](int k0, int i) { return reinterpret_cast<const uintx4 *>(vals + (size_t)(i / (kKeys / 8)) * p.keys_p + k0 + i % (kKeys / 8) * 8); };
-    auto key_place = [&](int i) { return reinterpret_cast<uintx4 *>(kt + i / k_pieces * ldk + i % k_pieces * 8); };
-    auto value_place = [&](int i) { return reinterpret_cast<uintx4 *>(vt + i / (kKeys / 8) * LDV + i % (kKeys / 8) * 8); };
-    const int n_key = kKeys * k_pieces, n_value = values * (kKeys / 8);
-    uintx4 ahead_k[PK], ahead_v[NQ ? PV : 1];   // bf16 only: one word per piece
-    auto fetch = [&](int k0) {
-        if constexpr (NQ > 0) {
-#pragma unroll
-            for (int i = 0; i < PK; i++) ahead_k[i] = *key_piece(k0, tid + i * 256 < n_key ? tid + i * 256 : 0);
-#pragma unroll
-            for (int i = 0; i < PV; i++) ahead_v[i] = *value_piece(k0, tid + i * 256 < n_value ? tid + i * 256 : 0);
-        }
-    };
-    fetch(k_begin);
-    const T *q = static_cast<const T *>(p.q) + ((size_t)h * rows_p + (m < rows_p ? m : rows_p - 1)) * qk + 8 * half;
-    typename Op<T>::frag qf[NQ ? NQ : 1];
-    if constexpr (NQ > 0) {
-#pragma unroll
-        for (int i = 0; i < NQ; i++) qf[i] = Op<T>::load(q + (i * 16 < qk ? i * 16 : 0));
-    }
-    float top = l.sink[h], sum = set == 0 ? 1.0f : 0.0f;   // the sink: one more term of the denominator, without a value
-    floatx16 out[4];
-#pragma unroll
-    for (int i = 0; i < 4; i++) out[i] = matrix::zero_accumulator();
-    for (int k0 = k_begin; k0 < k_end; k0 += kKeys) {
-        __syncthreads();
-        if constexpr (NQ > 0) {
-#pragma unroll
-            for (int i = 0; i < PK; i++)
-                if (tid + i * 256 < n_key) *key_place(tid + i * 256) = ahead_k[i];
-#pragma unroll
-            for (int i = 0; i < PV; i++)
-                if (tid + i * 256 < n_value) *value_place(tid + i * 256) = ahead_v[i];
-            if (k0 + kKeys < k_end) fetch(k0 + kKeys);
-        } else {
-            for (int i = tid; i < n_key; i += 256) {
-#pragma unroll
-                for (int v = 0; v < kVec; v++) key_place(i)[v] = key_piece(k0, i)[v];
-            }
-            for (int i = tid; i < n_value; i += 256) {
-#pragma unroll
-                for (int v = 0; v < kVec; v++) value_place(i)[v] = value_piece(k0, i)[v];
-            }
-        }
-        __syncthreads();
-        const int ks = k0 + set * 32;
-        if (ks > wave_at + 31 || ks + 31 <= wave_at - l.window) continue;   // no query of this wavefront sees these keys
-        floatx16 s = matrix::zero_accumulator();
-        const T *kp = kt + (set * 32 + col) * ldk + 8 * half;
-        if constexpr (NQ > 0) {
-#pragma unroll
-            for (int i = 0; i < NQ; i++)
-                if (i * 16 < qk) s = Op<T>::mma(Op<T>::load(kp + i * 16), qf[i], s);
-        } else {
-            for (int d = 0; d < qk; d += 16) s = Op<T>::mma(Op<T>::load(kp + d), Op<T>::load(q + d), s);
-        }
-        float w[16], best = -INFINITY;
-#pragma unroll
-        for (int r = 0; r < 16; r++) {
-            const int gap = at - (ks + matrix::accumulator_row(r, half));
-            w[r] = gap >= 0 && gap < l.window ? s[r] * l.scale : -INFINITY;
-            best = fmaxf(best, w[r]);
-        }
-        best = fmaxf(fmaxf(best, __shfl_xor(best, 32)), top);
-        const float keep = weight_exp<T>(top - best);
-        float add = 0.0f;
-#pragma unroll
-        for (int r = 0; r < 16; r++) { w[r] = weight_exp<T>(w[r] - best); add += w[r]; }
-        add += __shfl_xor(add, 32);
-        sum = sum * keep + add;
-        top = best;
-#pragma unroll
-        for (int i = 0; i < 4; i++) {
-            if (i * 32 >= values) continue;
-#pragma unroll
-            for (int r = 0; r < 16; r++) out[i][r] *= keep;
-        }
-#pragma unroll
-        for (int st = 0; st < 2; st++) {
-            float f[8];
-#pragma unroll
-            for (int j = 0; j < 8; j++) f[j] = w[st * 8 + j];
-#pragma unroll
-            for (int i = 0; i < 4; i++) {
-                if (i * 32 >= values) continue;
-                const T *vp = vt + (i * 32 + col) * LDV + set * 32 + st * 16 + 4 * half;
-                out[i] = matrix::mma_values<T>(Op<T>::load_pair(vp, vp + 8), f, out[i]);
-            }
-        }
-    }
-    // the second half of the keys joins the first: per query tile 64 lanes x (64 sums, maximum, denominator), 66 words apart
-    __syncthreads();
-    float *meet = reinterpret_cast<float *>(smem) + (size_t)(qt * 64 + lane) * 66;
-    if (set == 1) {
-#pragma unroll
-        for (int i = 0; i < 4; i++)
-#pragma unroll
-            for (int r = 0; r < 16; r++) meet[i * 16 + r] = out[i][r];
-        meet[64] = top;
-        meet[65] = sum;
-    }
-    __syncthreads();
-    if (set == 1 || m >= p.rows) return;
-    const float all = fmaxf(top, meet[64]), mine = weight_exp<T>(top - all), theirs = weight_exp<T>(meet[64] - all);
-    const float factor = matrix::sigmoid(p.mixed[(size_t)m * l.ld_mix + l.gate_at + h]) / (sum * mine + meet[65] * theirs);
-    T *dst = static_cast<T *>(p.act) + (size_t)m * p.ld_act + h * l.vdim_p + v0;
-#pragma unroll
-    for (int i = 0; i < 4; i++) {
-        if (i * 32 >= values) continue;
-#pragma unroll
-        for (int g = 0; g < 4; g++)
-#pragma unroll
-            for (int k = 0; k < 4; k++) dst[i * 32 + g * 8 + 4 * half + k] = Op<T>::from_float((out[i][4 * g + k] * mine + meet[i * 16 + 4 * g + k] * theirs) * factor);
-    }
-}
-
 bool shape_ok(const LatentShape &l) {
     return l.heads > 0 && l.dim_p % 32 == 0 && l.vdim_p % 32 == 0 && l.rot_p % 32 == 0 && l.rank_p % 64 == 0 && l.dim <= l.dim_p && l.vdim <= l.vdim_p && l.rot_dim <= l.rot_p &&
            l.kv_rank <= l.rank_p && l.rot_dims <= l.rot_dim && l.rot_dims % 2 == 0 && l.window >= 1 && l.ring >= 1 && l.cache && l.rank_p <= kLatentMaxRank && l.dim_p <= 4096;
@@ -532,16 +372,6 @@ hipError_t run_step(const LatentShape &l, const LatentStep &p, hipStream_t s) {
     else e = run_partial<T, 4, 0>(l, p, s);
     if (e != hipSuccess) return e;
     hipLaunchKernelGGL((latent_merge_kernel<T>), dim3(l.vdim_p / 32, l.heads, p.rows), dim3(256), (size_t)(l.rank_p + 64) * 4, s, l, p);
-    return hipGetLastError();
-}
-
-template <typename T, int NQ>
-hipError_t run_block(const LatentShape &l, const LatentBlock &p, int rows_p, hipStream_t s) {
-    const size_t lds = BlockLayout<T>::bytes(l.dim_p + l.rot_p);
-    if (lds > 158 * 1024) return hipErrorInvalidValue;
-    const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void *>(&latent_block_kernel<T, NQ>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
-    if (e != hipSuccess) return e;
-    hipLaunchKernelGGL((latent_block_kernel<T, NQ>), dim3((p.rows + kQueries - 1) / kQueries, l.heads, (l.vdim_p + kValues - 1) / kValues), dim3(256), lds, s, l, p, rows_p);
     return hipGetLastError();
 }
 
@@ -588,9 +418,11 @@ hipError_t launch_latent_queries(const LatentShape &l, const LatentBlock &p, Pre
 
 hipError_t launch_latent_block(const LatentShape &l, const LatentBlock &p, Precision type, hipStream_t s) {
     if (!block_ok(l, p)) return hipErrorInvalidValue;
-    const int rows_p = padded_rows(p.rows), qk = l.dim_p + l.rot_p;
-    if (type == Precision::f32) return run_block<float, 0>(l, p, rows_p, s);
-    return qk <= 96 ? run_block<uint16_t, 6>(l, p, rows_p, s) : qk <= 192 ? run_block<uint16_t, 12>(l, p, rows_p, s) : run_block<uint16_t, 0>(l, p, rows_p, s);
+    BlockAttention b;
+    b.heads = b.kv_heads = l.heads; b.dim_p = l.dim_p; b.rot_p = l.rot_p; b.vdim_p = l.vdim_p; b.window = l.window; b.scale = l.scale;
+    b.rows = p.rows; b.before = p.base - p.first_key; b.keys_p = p.keys_p;
+    b.q = p.q; b.k = p.k; b.key_rot = p.key_rot; b.vt = p.vt; b.sink = l.sink; b.gate = p.mixed + l.gate_at; b.ld_gate = l.ld_mix; b.act = p.act; b.ld_act = p.ld_act;
+    return launch_block_attention(b, type, s);
 }
 
 }  // namespace esp

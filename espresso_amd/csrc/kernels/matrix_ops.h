@@ -113,6 +113,16 @@ __device__ __forceinline__ floatx16 mma_values(const typename Op<T>::frag &a, co
 
 __device__ __forceinline__ float sigmoid(float z) { return 1.0f / (1.0f + expf(-z)); }
 __device__ __forceinline__ float silu(float z) { return z / (1.0f + expf(-z)); }
+// 0.5 z (1 + tanh u) = z / (1 + exp(-2 u)), u = sqrt(2 / pi) (z + 0.044715 z^3)
+__device__ __forceinline__ float gelu_tanh(float z) { return z / (1.0f + expf(-1.5957691216057308f * (z + 0.044715f * z * z * z))); }
+// A gated feed-forward's value (function: GateFunction).
+__device__ __forceinline__ float gated(int function, float gate, float up) { return (function ? gelu_tanh(gate) : silu(gate)) * up; }
+// Exponentials of scores: bf16 models use the hardware's exponential directly.
+template <typename T>
+__device__ __forceinline__ float weight_exp(float x) {
+    if constexpr (Op<T>::kSplit) return __expf(x);
+    else return expf(x);
+}
 
 }  // namespace matrix
 }  // namespace esp

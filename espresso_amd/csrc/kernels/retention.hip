@@ -8,16 +8,11 @@
 // eight rows; q and k are rotated by every workgroup of the head.  The norm of the output needs the whole head, so a workgroup
 // leaves the sum of squares of its part and the output product's staging finishes it.
 //
-// A prompt block runs in chunks of 64 tokens, three launches:
-//   prepare   rotates q and k, writes them and v in the layouts the products read (k and v transposed, k times the decay that is
-//             left at the end of its chunk);
-//   states    one wavefront per 32 x 32 tile of a head's state walks the chunks: it stores the state before the chunk, then
-//             S = decay^64 S + V^T K' on the matrix cores;
-//   outputs   o = decay^(t + 1) S^T q + sum over the chunk's keys s <= t of decay^(t - s) (q . k_s) v_s; scores are computed transposed,
-//             so that their accumulator is the operand of the second product and no score passes through LDS.
-// With bf16 operands, what belongs to the recurrence (states, decayed keys, scores) enters the products as a high and a low bf16.
+// A prompt block runs in chunks of 64 tokens (chunk_recurrence.h) after one launch of its own: prepare rotates q and k, writes them and
+// v in the layouts the products read (k and v transposed, k times the decay that is left at the end of its chunk).
 #include <hip/hip_runtime.h>
 
+#include "chunk_recurrence.h"
 #include "gemv_device.h"
 #include "layer_ops.h"
 #include "matrix_ops.h"
@@ -25,11 +20,10 @@
 namespace esp {
 namespace {
 
-using matrix::floatx16;
+using chunked::C;
 using matrix::Op;
 
 constexpr int kStepRows = 32;   // rows of a transposed state per workgroup of a step
-constexpr int C = kRetentionChunk;
 
 // Element i of a head's q or k at `position`, rotated: pairs (i, i + dims / 2) of the first dims elements.
 __device__ __forceinline__ float rotated_half(const float *x, int i, int dims, const float *cos, const float *sin) {
@@ -84,18 +78,6 @@ __global__ __launch_bounds__(256) void retention_step_kernel(RetentionShape r, R
     if (tid == 0) p.squares[((size_t)m * r.heads + h) * gridDim.x + part] = total;
 }
 
-template <typename T>
-__device__ __forceinline__ void store8(T *p, const float (&x)[8]);
-template <>
-__device__ __forceinline__ void store8<uint16_t>(uint16_t *p, const float (&x)[8]) {
-    *reinterpret_cast<uint4 *>(p) = make_uint4(matrix::pack_bf16(x[0], x[1]), matrix::pack_bf16(x[2], x[3]), matrix::pack_bf16(x[4], x[5]), matrix::pack_bf16(x[6], x[7]));
-}
-template <>
-__device__ __forceinline__ void store8<float>(float *p, const float (&x)[8]) {
-    reinterpret_cast<float4 *>(p)[0] = make_float4(x[0], x[1], x[2], x[3]);
-    reinterpret_cast<float4 *>(p)[1] = make_float4(x[4], x[5], x[6], x[7]);
-}
-
 struct BlockArgs {
     RetentionShape r;
     const float *mixed;
@@ -147,140 +129,10 @@ __global__ __launch_bounds__(256) void retention_prepare_kernel(BlockArgs a) {
 #pragma unroll
     for (int i = 0; i < 8; i++) x[i] = slab[col][part + i];
     if (values) {
-        store8<T>(static_cast<T *>(a.vt) + ((size_t)h * r.vdim_p + first) * a.R + t0 + part, x);
+        chunked::store8<T>(static_cast<T *>(a.vt) + ((size_t)h * r.vdim_p + first) * a.R + t0 + part, x);
     } else {
         const size_t o = ((size_t)h * r.dim_p + first) * a.R + t0 + part;
-        store8<T>(static_cast<T *>(a.kt_hi) + o, x);
-        if constexpr (Op<T>::kSplit) {
-#pragma unroll
-            for (int i = 0; i < 8; i++) x[i] -= Op<T>::to_float(Op<T>::from_float(x[i]));
-            store8<T>(static_cast<T *>(a.kt_lo) + o, x);
-        }
-    }
-}
-
-// One wavefront per tile of 32 v x 32 d of one head's state; workgroups of four tiles along d.
-template <typename T>
-__global__ __launch_bounds__(256) void retention_states_kernel(BlockArgs a) {
-    const RetentionShape &r = a.r;
-    const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, half = lane >> 5;
-    const int h = blockIdx.z, v0 = blockIdx.y * 32, d0 = (blockIdx.x * 4 + wave) * 32;
-    if (d0 >= r.dim_p) return;
-    const size_t tile = (size_t)v0 * r.dim_p + d0 + (lane & 31), head = (size_t)r.vdim_p * r.dim_p;
-    float *state = r.state + ((size_t)a.seq * r.heads + h) * head;
-    floatx16 acc = matrix::zero_accumulator();
-    if (a.base > 0) {
-#pragma unroll
-        for (int i = 0; i < 16; i++) acc[i] = state[tile + (size_t)matrix::accumulator_row(i, half) * r.dim_p];
-    }
-    const T *vt = static_cast<const T *>(a.vt) + ((size_t)h * r.vdim_p + v0 + (lane & 31)) * a.R + 8 * half;
-    const T *kh = static_cast<const T *>(a.kt_hi) + ((size_t)h * r.dim_p + d0 + (lane & 31)) * a.R + 8 * half;
-    const T *kl = static_cast<const T *>(a.kt_lo) + ((size_t)h * r.dim_p + d0 + (lane & 31)) * a.R + 8 * half;
-    const int chunks = a.R / C;
-    for (int c = 0; c < chunks; c++) {
-        const int len = a.rows - c * C < C ? a.rows - c * C : C;
-        T *hi = static_cast<T *>(a.states_hi) + ((size_t)c * r.heads + h) * head, *lo = static_cast<T *>(a.states_lo) + ((size_t)c * r.heads + h) * head;
-        const float factor = r.powers[h * (C + 1) + len];
-        typename Op<T>::frag v[C / 16], w[C / 16], x[C / 16];   // on their way while the state before the chunk is stored
-#pragma unroll
-        for (int ks = 0; ks < C / 16; ks++) {
-            v[ks] = Op<T>::load(vt + c * C + ks * 16);
-            w[ks] = Op<T>::load(kh + c * C + ks * 16);
-            if constexpr (Op<T>::kSplit) x[ks] = Op<T>::load(kl + c * C + ks * 16);
-        }
-#pragma unroll
-        for (int i = 0; i < 16; i++) {
-            const size_t o = tile + (size_t)matrix::accumulator_row(i, half) * r.dim_p;
-            const T b = Op<T>::from_float(acc[i]);
-            hi[o] = b;
-            if constexpr (Op<T>::kSplit) lo[o] = Op<T>::from_float(acc[i] - Op<T>::to_float(b));
-            acc[i] *= factor;
-        }
-#pragma unroll
-        for (int ks = 0; ks < C / 16; ks++) {
-            acc = Op<T>::mma(v[ks], w[ks], acc);
-            if constexpr (Op<T>::kSplit) acc = Op<T>::mma(v[ks], x[ks], acc);
-        }
-    }
-#pragma unroll
-    for (int i = 0; i < 16; i++) state[tile + (size_t)matrix::accumulator_row(i, half) * r.dim_p] = acc[i];
-}
-
-// grid (chunks, heads, slices of 128 v): wavefront w takes queries 32 (w % 2) .. of the chunk and 64 v from 64 (w / 2) of the slice.
-template <typename T>
-__global__ __launch_bounds__(256) void retention_outputs_kernel(BlockArgs a) {
-    const RetentionShape &r = a.r;
-    const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, half = lane >> 5;
-    const int c = blockIdx.x, h = blockIdx.y, qt = wave & 1, v0 = blockIdx.z * 128 + (wave >> 1) * 64;
-    if (v0 >= r.vdim_p || c * C + qt * 32 >= a.rows) return;
-    const bool two = v0 + 32 < r.vdim_p;   // a second tile of 32 v
-    const int t_local = qt * 32 + (lane & 31);   // this lane's query, in the chunk
-    const T *q = static_cast<const T *>(a.q) + ((size_t)h * a.R + c * C + t_local) * r.dim_p + 8 * half;
-    const T *k = static_cast<const T *>(a.k) + ((size_t)h * a.R + c * C + (lane & 31)) * r.dim_p + 8 * half;
-    const size_t head = (size_t)r.vdim_p * r.dim_p, s_at = ((size_t)c * r.heads + h) * head + (size_t)(v0 + (lane & 31)) * r.dim_p + 8 * half;
-    const T *shi = static_cast<const T *>(a.states_hi) + s_at, *slo = static_cast<const T *>(a.states_lo) + s_at;
-    const size_t next = two ? (size_t)32 * r.dim_p : 0;
-    floatx16 score[2], out[2];
-#pragma unroll
-    for (int i = 0; i < 2; i++) score[i] = out[i] = matrix::zero_accumulator();
-    constexpr int kAhead = Op<T>::kSplit ? 2 : 1;   // steps of 16 dimensions whose loads are in flight together (dim_p is a multiple of 32)
-    const size_t k_next = qt ? (size_t)32 * r.dim_p : 0;
-    for (int d0 = 0; d0 < r.dim_p; d0 += 16 * kAhead) {
-        typename Op<T>::frag qf[kAhead], kf[kAhead][2], sf[kAhead][2], tf[kAhead][2];
-#pragma unroll
-        for (int u = 0; u < kAhead; u++) {
-            const int d = d0 + 16 * u;
-            qf[u] = Op<T>::load(q + d);
-#pragma unroll
-            for (int i = 0; i < 2; i++) {
-                kf[u][i] = Op<T>::load(k + i * k_next + d);
-                sf[u][i] = Op<T>::load(shi + i * next + d);
-                if constexpr (Op<T>::kSplit) tf[u][i] = Op<T>::load(slo + i * next + d);
-            }
-        }
-#pragma unroll
-        for (int u = 0; u < kAhead; u++)
-#pragma unroll
-            for (int i = 0; i < 2; i++) {
-                score[i] = Op<T>::mma(kf[u][i], qf[u], score[i]);
-                out[i] = Op<T>::mma(sf[u][i], qf[u], out[i]);
-                if constexpr (Op<T>::kSplit) out[i] = Op<T>::mma(tf[u][i], qf[u], out[i]);
-            }
-    }
-    const float *powers = r.powers + h * (C + 1);
-    const float reach = powers[t_local + 1];
-#pragma unroll
-    for (int i = 0; i < 2; i++)
-#pragma unroll
-        for (int j = 0; j < 16; j++) out[i][j] *= reach;
-    const T *vt = static_cast<const T *>(a.vt) + ((size_t)h * r.vdim_p + v0 + (lane & 31)) * a.R + c * C + 4 * half;
-    const size_t next_v = two ? (size_t)32 * a.R : 0;
-    for (int kt = 0; kt <= qt; kt++) {
-#pragma unroll
-        for (int st = 0; st < 2; st++) {
-            float w[8];
-#pragma unroll
-            for (int j = 0; j < 8; j++) {
-                const int s_local = kt * 32 + matrix::accumulator_row(st * 8 + j, half), gap = t_local - s_local;
-                const float x = kt ? score[1][st * 8 + j] : score[0][st * 8 + j];
-                w[j] = gap >= 0 ? x * powers[gap] : 0.0f;
-            }
-#pragma unroll
-            for (int i = 0; i < 2; i++) {
-                const T *p = vt + i * next_v + kt * 32 + st * 16;
-                out[i] = matrix::mma_values<T>(Op<T>::load_pair(p, p + 8), w, out[i]);
-            }
-        }
-    }
-    const int t = c * C + t_local;
-    if (t >= a.rows) return;
-    float *o = a.o + (size_t)t * r.heads * r.vdim_p + h * r.vdim_p + v0;
-#pragma unroll
-    for (int i = 0; i < 2; i++) {
-        if (i && !two) break;
-#pragma unroll
-        for (int g = 0; g < 4; g++)
-            *reinterpret_cast<float4 *>(o + i * 32 + g * 8 + 4 * half) = make_float4(out[i][4 * g], out[i][4 * g + 1], out[i][4 * g + 2], out[i][4 * g + 3]);
+        chunked::store8_split<T>(static_cast<T *>(a.kt_hi) + o, static_cast<T *>(a.kt_lo) + o, x);
     }
 }
 
@@ -308,8 +160,11 @@ hipError_t run_block(const BlockArgs &a, hipStream_t s) {
     const RetentionShape &r = a.r;
     const int chunks = a.R / C;
     hipLaunchKernelGGL((retention_prepare_kernel<T>), dim3(chunks, r.heads, (r.dim_p + r.vdim_p) / 32), dim3(256), 0, s, a);
-    hipLaunchKernelGGL((retention_states_kernel<T>), dim3((r.dim_p + 127) / 128, r.vdim_p / 32, r.heads), dim3(256), 0, s, a);
-    hipLaunchKernelGGL((retention_outputs_kernel<T>), dim3(chunks, r.heads, (r.vdim_p + 127) / 128), dim3(256), 0, s, a);
+    chunked::Block c{};
+    c.heads = r.heads; c.key_share = 1; c.dim_p = r.dim_p; c.vdim_p = r.vdim_p; c.rows = a.rows; c.R = a.R; c.base = a.base;
+    c.q = a.q; c.k = a.k; c.vt = c.state_v = a.vt; c.state_k = a.kt_hi; c.state_k_lo = a.kt_lo;
+    c.state = r.state + (size_t)a.seq * r.heads * r.vdim_p * r.dim_p; c.states_hi = a.states_hi; c.states_lo = a.states_lo; c.o = a.o;
+    chunked::launch_states_and_outputs<T>(c, chunked::FixedDecay{r.powers}, s);
     return hipGetLastError();
 }
 

@@ -9,7 +9,7 @@ import numpy as np
 
 from . import _lib, llama
 
-KERNEL_CLASSES = ("in", "retention", "latent", "out", "head", "norm")
+KERNEL_CLASSES = ("in", "retention", "latent", "out", "head", "norm", "attention", "mamba2")
 
 
 class LayeredRuntime(llama.LlamaRuntime):
@@ -20,7 +20,7 @@ class LayeredRuntime(llama.LlamaRuntime):
         layers = config["layers"]
         self.config = config
         self.cfg = llama.MultiModelConfig(n_layer=len(layers), n_head=layers[0]["mixer"]["heads"], n_kv_head=layers[0]["mixer"]["heads"],
-                                          d_model=config["width"], head_dim=layers[0]["mixer"]["dim"],
+                                          d_model=config["width"], head_dim=layers[0]["mixer"].get("dim", layers[0]["mixer"]["vdim"]),
                                           hidden_dim=max((l["mlp"] or {}).get("ff", 0) for l in layers), vocab=config["vocab"], max_seq=max_seq,
                                           name=config["architecture"], architecture="layered")
         self._L.esp_layered_create_synthetic.restype = C.c_void_p

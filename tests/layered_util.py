@@ -31,19 +31,47 @@ def latent(heads=3, dim=16, vdim=24, kv_rank=40, rot_dim=8, window=20, scale=Non
     return {"type": "latent_attention", "mixer": m, "mlp": {"kind": "dense", "ff": ff} if ff else None}
 
 
+def attention(heads=4, kv_heads=2, dim=16, vdim=24, dims=8, window=20, scale=None, base=10000.0, factor=None, kv_from=None, ff=48):
+    m = {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim, "scale": dim ** -0.5 if scale is None else scale, "mask": {"size": window},
+         "rot": rotary(dims, base, None if factor is None else {"factor": factor})}
+    if kv_from is not None:
+        m["kv_from"] = kv_from
+    return {"type": "attention", "mixer": m, "mlp": {"kind": "dense", "ff": ff} if ff else None}
+
+
+def mamba2(heads=4, vdim=16, state=24, groups=2, conv=4, norm_groups=2, ff=0, kind="mamba2"):
+    return {"type": kind, "mixer": {"heads": heads, "vdim": vdim, "state": state, "groups": groups, "conv": conv, "norm_groups": norm_groups},
+            "mlp": {"kind": "dense", "ff": ff} if ff else None}
+
+
+def sequential(layers, vocab=96, width=56, eps=1e-5):
+    return {"architecture": "Forovik", "vocab": vocab, "width": width, "norm": {"eps": eps}, "layers": layers}
+
+
 def config(layers, vocab=96, width=56, residual_mult=0.7, softcap=25.0, eps=1e-5):
     return {"architecture": "Ranavik", "vocab": vocab, "width": width, "residual_mult": residual_mult, "logit_softcap": softcap, "norm": {"eps": eps},
             "layers": layers}
 
 
 def tensor_shapes(cfg):
-    d, out = cfg["width"], {"embed": (cfg["vocab"], cfg["width"]), "embed.norm": (cfg["width"],), "final.norm": (cfg["width"],), "head": (cfg["vocab"], cfg["width"])}
+    d, out = cfg["width"], {"embed": (cfg["vocab"], cfg["width"]), "final.norm": (cfg["width"],)}
+    if cfg["architecture"] == "Ranavik":
+        out.update({"embed.norm": (d,), "head": (cfg["vocab"], d)})
     for i, layer in enumerate(cfg["layers"]):
         m, p = layer["mixer"], f"l{i}."
         out[p + "norm1"] = (d,)
         if layer["type"] == "retention":
             qk, v = m["heads"] * m["dim"], m["heads"] * m["vdim"]
             out.update({p + "mix.q": (qk, d), p + "mix.k": (qk, d), p + "mix.v": (v, d), p + "mix.g": (v, d), p + "mix.o": (d, v)})
+        elif layer["type"].startswith("mamba2"):
+            h, inner, shared = m["heads"], m["heads"] * m["vdim"], m["groups"] * m["state"]
+            out.update({p + "mix.in": (2 * inner + 2 * shared + h, d), p + "mix.conv": (inner + 2 * shared, m["conv"]), p + "mix.conv.b": (inner + 2 * shared,),
+                        p + "mix.dt_bias": (h,), p + "mix.A_log": (h,), p + "mix.D": (h,), p + "mix.norm": (inner,), p + "mix.o": (d, inner)})
+        elif layer["type"] == "attention":
+            q, k = m["heads"] * m["dim"], m["kv_heads"] * m["dim"]
+            out.update({p + "mix.q": (q, d), p + "mix.q.norm": (q,), p + "mix.o": (d, m["heads"] * m["vdim"])})
+            if m.get("kv_from") is None:
+                out.update({p + "mix.k": (k, d), p + "mix.k.norm": (k,), p + "mix.v": (m["kv_heads"] * m["vdim"], d)})
         else:
             h = m["heads"]
             out.update({p + "mix.q": (h * (m["dim"] + m["rot_dim"]), d), p + "mix.uk": (h * m["dim"], m["kv_rank"]), p + "mix.uv": (h * m["vdim"], m["kv_rank"]),
@@ -63,12 +91,19 @@ def to_bf16(x):
 
 
 def random_weights(cfg, seed, gain=1.0, sink=None):
-    """Linears ~N(0, gain / sqrt(inputs)), norms around 1, sinks ~N(0, 1) (or the given value); every value is a bf16 number."""
+    """Linears ~N(0, gain / sqrt(inputs)), norms around 1, sinks ~N(0, 1) (or the given value), decays from a few tokens to hundreds; every
+    value is a bf16 number."""
     rng = np.random.default_rng(seed)
     w = {}
     for name, shape in sorted(tensor_shapes(cfg).items()):
         if name.endswith("sink"):
             a = rng.normal(0, 1, shape) if sink is None else np.full(shape, sink)
+        elif name.endswith("A_log"):
+            a = rng.uniform(-3.0, 1.0, shape)
+        elif name.endswith("dt_bias"):
+            a = rng.uniform(-3.0, 1.0, shape)
+        elif name.endswith("conv.b"):
+            a = rng.normal(0, 0.3, shape)
         elif len(shape) == 1:
             a = rng.uniform(0.6, 1.4, shape)
         else:

@@ -51,9 +51,9 @@ def test_a_llama_directory_is_still_found_by_its_metadata(tmp_path):
     (lambda c: c["layers"][1]["mixer"]["rot"].update(dims=7), "odd"),
     (lambda c: c["layers"][0]["mixer"]["mask"].update(size=0), "size is not a usable count"),
     (lambda c: c["layers"][0]["mixer"].pop("scale"), "scale is not a number"),
-    (lambda c: c["layers"][2]["mixer"].update(kv_from=1), "without fitting latents"),
+    (lambda c: c["layers"][2]["mixer"].update(kv_from=1), "without a fitting cache"),
     (lambda c: c["layers"][2]["mixer"].update(kv_from=2), "earlier layer"),
-    (lambda c: c["layers"][2]["mixer"].update(kv_rank=48), "without fitting latents"),
+    (lambda c: c["layers"][2]["mixer"].update(kv_rank=48), "without a fitting cache"),
     (lambda c: c["layers"][0]["mlp"].update(kind="experts"), "kind is not dense"),
 ])
 def test_configurations_that_do_not_fit_are_refused(tmp_path, change, message):
