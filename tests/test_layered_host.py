@@ -20,6 +20,10 @@ ROOT = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
 BASE = lu.config([lu.latent(), lu.retention(), lu.latent(kv_from=0, window=7), lu.retention(ff=0)])
 
 
+SEQUENTIAL = lu.sequential([lu.mamba2(), lu.attention(factor=4.0), lu.mamba2(heads=6, vdim=20, state=40, groups=3, conv=3, norm_groups=4, kind="mamba2_2", ff=40),
+                            lu.attention(kv_from=1, factor=4.0, window=7, ff=0)])
+
+
 def load(tmp_path, cfg, max_seq=64):
     with open(tmp_path / "config.json", "w") as f:
         f.write(cfg if isinstance(cfg, str) else json.dumps(cfg))
@@ -30,6 +34,12 @@ def test_registered_and_read_from_a_directory(tmp_path):
     assert "Ranavik" in eng.layered_architectures()
     c = load(tmp_path, BASE, 77)
     assert (c.architecture, c.name, c.n_layer, c.d_model, c.vocab, c.max_seq, c.hidden_dim, c.eos_token) == ("layered", "Ranavik", 4, 56, 96, 77, 48, -1)
+
+
+def test_a_sequential_design_is_read_from_a_directory(tmp_path):
+    assert "Forovik" in eng.layered_architectures()
+    c = load(tmp_path, SEQUENTIAL, 77)
+    assert (c.architecture, c.name, c.n_layer, c.d_model, c.vocab, c.max_seq, c.hidden_dim) == ("layered", "Forovik", 4, 56, 96, 77, 48)
 
 
 def test_a_llama_directory_is_still_found_by_its_metadata(tmp_path):
@@ -61,6 +71,42 @@ def test_configurations_that_do_not_fit_are_refused(tmp_path, change, message):
     change(c)
     with pytest.raises(lib.EspressoError, match=message):
         load(tmp_path, c)
+
+
+@pytest.mark.parametrize("change,message", [
+    (lambda c: c["layers"][0].update(type="retention"), "names no mixer of this architecture: retention"),
+    (lambda c: c["layers"][0]["mixer"].update(groups=3), "groups does not divide the heads"),
+    (lambda c: c["layers"][0]["mixer"].update(norm_groups=5), "norm_groups does not divide"),
+    (lambda c: c["layers"][0]["mixer"].pop("conv"), "conv is not a number"),
+    (lambda c: c["layers"][0]["mixer"].update(state=0), "state is not a usable count"),
+    (lambda c: c["layers"][1]["mixer"].update(kv_heads=3), "kv_heads does not divide"),
+    (lambda c: c["layers"][1]["mixer"]["rot"].update(dims=20), "larger than what it rotates"),
+    (lambda c: c["layers"][1]["mixer"]["rot"]["scaling"].update(factor=0), "factor is not positive"),
+    (lambda c: c["layers"][1]["mixer"].pop("mask"), "mask is not an object"),
+    (lambda c: c["layers"][3]["mixer"].update(kv_from=0), "without a fitting cache"),
+    (lambda c: c["layers"][3]["mixer"].update(kv_from=3), "earlier layer"),
+    (lambda c: c["layers"][3]["mixer"].update(dim=18), "without a fitting cache"),
+    (lambda c: c["layers"][3]["mixer"]["rot"].update(base=5.0), "without a fitting cache"),
+    (lambda c: c["layers"][1].update(mlp={"kind": "experts", "ff": 8}), "kind is not dense"),
+])
+def test_sequential_configurations_that_do_not_fit_are_refused(tmp_path, change, message):
+    c = copy.deepcopy(SEQUENTIAL)
+    change(c)
+    with pytest.raises(lib.EspressoError, match=message):
+        load(tmp_path, c)
+
+
+@pytest.mark.parametrize("layer,message", [(lu.attention(dim=1040, dims=8), "1040 values per attention head exceed 1024"), (lu.mamba2(conv=300), "300 taps of a convolution exceed 256"),
+                                           (lu.mamba2(state=4100), "4100 values of a state exceed 4096")])
+def test_sizes_past_the_kernels_are_refused(tmp_path, layer, message):
+    c = lu.sequential([layer], width=8, vocab=4)
+    lu.write_model(str(tmp_path), c, lu.random_weights(c, 1))
+    with pytest.raises(lib.EspressoError, match=message):
+        eng.RealModelInferenceEngine(eng.load_model_config(str(tmp_path), 16), str(tmp_path))
+
+
+def test_the_tensors_of_a_sequential_model():
+    assert set(lu.tensor_shapes(SEQUENTIAL)) >= {"l0.mix.A_log", "l1.mix.k.norm", "l3.mix.q.norm"} and not {"head", "embed.norm", "l3.mix.k", "l0.norm2"} & set(lu.tensor_shapes(SEQUENTIAL))
 
 
 def test_broken_files_are_refused(tmp_path):
@@ -193,5 +239,56 @@ def test_a_small_mistake_moves_the_logits_past_the_gpu_tests_limit(change):
     t = lu.tokens(BASE, 40)
     want = ref.forward(BASE, w, t)
     c, w2 = copy.deepcopy(BASE), dict(w)
+    change(c, w2)
+    assert lu.error(ref.forward(c, w2, t), want) > 3 * lu.F32_LIMIT
+
+
+def test_selective_recurrence_is_a_weighted_sum_over_earlier_tokens():
+    rng = np.random.default_rng(3)
+    x, b, c, dt, rate = rng.normal(size=(9, 2, 4)), rng.normal(size=(9, 2, 3)), rng.normal(size=(9, 2, 3)), rng.uniform(0.1, 2, (9, 2)), np.array([0.3, 2.0])
+    y, _ = ref.selective_recurrence(x, b, c, dt, rate)
+    for h in range(2):
+        for t in range(9):
+            want = sum(np.exp(-rate[h] * dt[s + 1:t + 1, h].sum()) * dt[s, h] * (b[s, h] @ c[t, h]) * x[s, h] for s in range(t + 1))
+            assert np.allclose(y[t, h], want)
+    half = ref.selective_recurrence(x[:5], b[:5], c[:5], dt[:5], rate)[1]
+    assert np.allclose(ref.selective_recurrence(x[5:], b[5:], c[5:], dt[5:], rate, half)[0], y[5:])
+
+
+def test_convolution_window_norm_and_gate():
+    x = np.arange(12.0).reshape(6, 2)
+    y = ref.causal_convolution(x, np.array([[0., 0., 1.], [1., 0., 0.]]), np.array([0.5, 0.0]))
+    assert np.allclose(y[:, 0], x[:, 0] + 0.5) and np.allclose(y[:, 1], [0, 0, 1, 3, 5, 7])
+    assert np.allclose(ref.causal_convolution(x[3:], np.ones((2, 3)), np.zeros(2), x[1:3]), ref.causal_convolution(x, np.ones((2, 3)), np.zeros(2))[3:])
+    w = ref.window_softmax(np.zeros((1, 5, 5)), range(5), range(5), 2)
+    assert np.allclose(w[0, 4], [0, 0, 0, .5, .5]) and np.allclose(w[0, 0], [1, 0, 0, 0, 0])
+    n = ref.grouped_rms_norm(np.array([[3., 4., 0., 10.]]), np.ones(4), 2, 0.0)
+    assert np.allclose(n, [[3 / np.sqrt(12.5), 4 / np.sqrt(12.5), 0, np.sqrt(2)]])
+    assert np.allclose(ref.gelu_tanh(np.array([-2., 0., 1.])), [-0.0454023, 0, 0.841192], atol=1e-6)
+    f, one = ref.rotary_frequencies(lu.rotary(8, 100.0, {"factor": 4.0}))
+    assert one == 1.0 and np.allclose(f, ref.rotary_frequencies(lu.rotary(8, 100.0))[0] / 4.0)
+
+
+@pytest.mark.parametrize("change", [
+    lambda c, w: c["layers"][1]["mixer"]["mask"].update(size=21),
+    lambda c, w: c["layers"][1]["mixer"]["mask"].update(size=19),
+    lambda c, w: c["layers"][3]["mixer"]["mask"].update(size=8),
+    lambda c, w: c["layers"][1]["mixer"].update(scale=0.2501),
+    lambda c, w: c["layers"][3]["mixer"].update(rot=lu.rotary(8, 10000.0, {"factor": 4.2})),
+    lambda c, w: c["layers"][1]["mixer"]["rot"].update(dims=6),
+    lambda c, w: c["layers"][0]["mixer"].update(norm_groups=1),
+    lambda c, w: c["norm"].update(eps=2e-3),
+    lambda c, w: w["l0.mix.D"].__imul__(1.01),
+    lambda c, w: w["l0.mix.dt_bias"].__iadd__(0.01),
+    lambda c, w: w["l0.mix.A_log"].__iadd__(0.01),
+    lambda c, w: w["l2.mix.conv"][:, 0].__imul__(0.98),
+    lambda c, w: w["l2.mix.conv.b"].__imul__(0.98),
+    lambda c, w: w["l1.mix.k.norm"].__imul__(1.01),
+])
+def test_a_small_mistake_moves_a_sequential_models_logits_past_the_limit(change):
+    w = lu.random_weights(SEQUENTIAL, 7, gain=2.0)
+    t = lu.tokens(SEQUENTIAL, 40)
+    want = ref.forward(SEQUENTIAL, w, t)
+    c, w2 = copy.deepcopy(SEQUENTIAL), {k: v.copy() for k, v in w.items()}
     change(c, w2)
     assert lu.error(ref.forward(c, w2, t), want) > 3 * lu.F32_LIMIT
