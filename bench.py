@@ -339,8 +339,8 @@ def run_two_token_8b(steps: int) -> dict:
 
 
 def run_layered(names, steps: int, prompt: int = 512) -> dict:
-    """Layered models (retention and latent attention, bf16 weights) beside llama models of equal width, feed-forward, vocabulary and
-    depth with fp16 weights: six random-init layers each, prefill of one block-aligned prompt (the second walk, every kernel warm)
+    """Layered models (bf16 weights): those of retention and latent attention beside llama models of equal width, feed-forward,
+    vocabulary and depth with fp16 weights, those of Mamba-2 and grouped attention beside those.  Six random-init layers each, prefill of one block-aligned prompt (the second walk, every kernel warm)
     and greedy decode at batch 1 behind it, as captured graphs.  step_weight_bytes: what a decode step reads of weights."""
     import espresso_amd.layered as layered
     import espresso_amd.llama as ll
@@ -366,10 +366,8 @@ def run_layered(names, steps: int, prompt: int = 512) -> dict:
                 "decode_tok_s": round(1.0 / per_step, 1), "step_weight_bytes": rt.weight_bytes,
                 "step_weight_gbps": round(rt.weight_bytes / per_step / 1e9, 1), "frac_hbm_peak": round(rt.weight_bytes / per_step / 1e9 / HBM_PEAK_GBPS, 3)}
 
-    results = {}
-    for name in names:
-        config, llama = syn.LAYERED_SIZES[name]
-        rt = layered.LayeredRuntime(config, max_seq=llama["max_seq"], seed=5)
+    def measure_layered(config, max_seq):
+        rt = layered.LayeredRuntime(config, max_seq=max_seq, seed=5)
         own = measure(rt, config["vocab"])
         own["sequence_state_bytes"] = layered.sequence_bytes(rt)
         ll.set_graph_replay(rt, False)
@@ -382,13 +380,24 @@ def run_layered(names, steps: int, prompt: int = 512) -> dict:
             t = layered.kernel_times(rt)
             own[phase + "_kernel_us"] = {k: round(v["total_us"] / count, 1) for k, v in t.items() if v["brackets"]}
         rt.close()
-        peer, _ = syn.build_runtime(ll.MultiModelConfig(**llama), _lib.FORMAT_F16, seed=3, kv_format=_lib.FORMAT_F16)
-        other = measure(peer, llama["vocab"])
-        peer.close()
-        results[name] = {"layered": own, "llama_f16": other,
+        return own
+
+    results = {}
+    for name in names:
+        if name in syn.SEQUENTIAL_SIZES:
+            config, size = syn.SEQUENTIAL_SIZES[name]
+            peer_name, max_seq = "layered_" + size, syn.LAYERED_SIZES[size][1]["max_seq"]
+            own, other = measure_layered(config, max_seq), measure_layered(syn.LAYERED_SIZES[size][0], max_seq)
+        else:
+            config, llama = syn.LAYERED_SIZES[name]
+            own, peer_name = measure_layered(config, llama["max_seq"]), "llama_f16"
+            peer, _ = syn.build_runtime(ll.MultiModelConfig(**llama), _lib.FORMAT_F16, seed=3, kv_format=_lib.FORMAT_F16)
+            other = measure(peer, llama["vocab"])
+            peer.close()
+        results[name] = {"layered": own, peer_name: other,
                          "prefill_ratio_per_weight": round((own["prefill_tok_s"] * own["step_weight_bytes"]) / (other["prefill_tok_s"] * other["step_weight_bytes"]), 3),
                          "decode_ratio_per_weight": round(own["step_weight_gbps"] / other["step_weight_gbps"], 3)}
-    return {"metric": "layered model prefill and decode tok/s (6 layers, bf16) beside llama f16 of equal size", "unit": "tok/s", "n_gpus": 1, "data": "synthetic",
+    return {"metric": "layered model prefill and decode tok/s (6 layers, bf16) beside a model of equal size", "unit": "tok/s", "n_gpus": 1, "data": "synthetic",
             "prompt_tokens": prompt, "steps": steps, "results": results,
             "note": "kernel_us: an event pair around each layer's launches of a class, launches one by one (no graph); event overhead included"}
 
@@ -454,7 +463,8 @@ def main() -> None:
     ap.add_argument("--stamps", action="store_true", help="per-wavefront time stamps inside one Q4_K GEMV launch, per decode shape and kernel")
     ap.add_argument("--two-token", action="store_true", help="exact two-token draft/verify decode on the 6-layer model instead of plain decode")
     ap.add_argument("--layered", nargs="*", metavar="SIZE", default=None,
-                    help="layered models (retention and latent attention) beside llama f16 models of equal size: d768, d2048, d4096 (default all)")
+                    help="layered models: d768, d2048, d4096 (retention and latent attention, beside llama f16 models of equal size), forovik-d768, "
+                         "forovik-d2048, forovik-d4096 (Mamba-2 and grouped attention, beside the former); default all")
     args = ap.parse_args()
     if args.gpus != 1:
         raise SystemExit("bench.py measures one GPU: this path is a batch-1 decode on a single MI355X; run with --gpus 1")
@@ -469,7 +479,7 @@ def main() -> None:
         print(json.dumps(out))
         return
     if args.layered is not None:
-        print(json.dumps(run_layered(args.layered or ["d768", "d2048", "d4096"], args.steps or 128)))
+        print(json.dumps(run_layered(args.layered or ["d768", "d2048", "d4096", "forovik-d768", "forovik-d2048", "forovik-d4096"], args.steps or 128)))
         return
     if args.stamps:
         print(json.dumps(run_stamps()))

@@ -24,7 +24,10 @@ using detail::wave_sum;
 
 constexpr int kGemvThreads = 512, kGemvWaves = 8, kRowAlign = 32;
 constexpr int kStep = 512;   // columns a wavefront takes per step: 64 lanes x 8
-enum GemvKind : int { KIND_IN, KIND_OUT, KIND_HEAD };
+// What a workgroup stages, and what becomes of a row's sum: the input side of a layer over normed rows, and over the stream itself (with
+// the branch that joins it); the output side, and the same with a norm by parts; the head.
+enum GemvKind : int { KIND_IN, KIND_IN_STREAM, KIND_OUT, KIND_OUT_PARTS, KIND_HEAD };
+__host__ __device__ constexpr bool is_in(int kind) { return kind == KIND_IN || kind == KIND_IN_STREAM; }
 
 struct DenseGemvArgs {
     const uint16_t *w;
@@ -43,6 +46,7 @@ struct DenseGemvArgs {
     const int *part_of, *part_starts;   // KIND_OUT: norm by parts
     const float *part_norm;
     int part_count, part_pieces;
+    bool part_by_eight;                 // every part starts at a multiple of eight columns
     float part_size;
     float mult, cap;
     const float *residual;
@@ -59,9 +63,9 @@ template <int KIND, int RPW, int AHEAD>
 __global__ __launch_bounds__(kGemvThreads) void dense_gemv_kernel(DenseGemvArgs a) {
     constexpr int kUnitRows = kGemvWaves * RPW;
     extern __shared__ float xs[];   // [k_pad], then [heads] or [part_count * part_pieces]
-    __shared__ float red[2 * kGemvWaves];
+    __shared__ float red[kGemvWaves];
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
-    const bool second = KIND == KIND_IN && (int)blockIdx.x >= a.blocks_a;
+    const bool second = is_in(KIND) && (int)blockIdx.x >= a.blocks_a;
     float scale = 1.0f;
     if constexpr (KIND == KIND_OUT) {
         float *head_inv = xs + a.k_pad;
@@ -89,37 +93,78 @@ __global__ __launch_bounds__(kGemvThreads) void dense_gemv_kernel(DenseGemvArgs 
             *reinterpret_cast<float4 *>(xs + staged_at(k, a.k_pad)) = v;
         }
         __syncthreads();
-        if (a.part_of) {   // sums of squares of every part, in part_pieces shares; then the values in place
-            for (int i = wave; i < a.part_count * a.part_pieces; i += kGemvWaves) {
-                const int g = i / a.part_pieces, to = a.part_starts[g + 1];
-                float s = 0.0f;
-                for (int k = a.part_starts[g] + (i % a.part_pieces) * 64 + lane; k < to; k += 64 * a.part_pieces) {
+    } else if constexpr (KIND == KIND_OUT_PARTS) {
+        // parts over their root mean squares: the values times the norm's weights wait in registers (up to four loads per thread, the rest is
+        // read again) while the values as they are pass through LDS and every part's squares are summed in part_pieces shares
+        constexpr int kHeld = 4, kSpan = kGemvThreads * 4;
+        float *sums = xs + a.k_pad;
+        float4 held[kHeld];
+        int4 part[kHeld];
+        auto at = [](const float *p, int k) { return *reinterpret_cast<const float4 *>(p + k); };
+        auto place = [&](int k, const float4 &v) { *reinterpret_cast<float4 *>(xs + staged_at(k, a.k_pad)) = v; };
+        auto squared = [](const float4 &v) { return v.x * v.x + v.y * v.y + v.z * v.z + v.w * v.w; };
+        auto value = [&](int k) {
+            const bool act = k >= a.act_at && k < a.act_at + a.act_cols;
+            const float4 v = act ? at(a.act, k - a.act_at) : at(a.mix, k < a.mix_cols ? k : 0);
+            const float keep = act || k < a.mix_cols ? 1.0f : 0.0f;
+            return make_float4(v.x * keep, v.y * keep, v.z * keep, v.w * keep);
+        };
+        {
+            float4 weight[kHeld];
+#pragma unroll
+            for (int c = 0; c < kHeld; c++) {
+                const int k = c * kSpan + tid * 4, in = k < a.mix_cols ? k : 0;
+                held[c] = value(k);
+                weight[c] = at(a.part_norm, in);
+                part[c] = *reinterpret_cast<const int4 *>(a.part_of + in);
+            }
+#pragma unroll
+            for (int c = 0; c < kHeld; c++) {
+                if (c * kSpan + tid * 4 < a.k_pad) place(c * kSpan + tid * 4, held[c]);
+                held[c].x *= weight[c].x; held[c].y *= weight[c].y; held[c].z *= weight[c].z; held[c].w *= weight[c].w;
+            }
+        }
+        for (int k = kHeld * kSpan + tid * 4; k < a.k_pad; k += kSpan) place(k, value(k));
+        __syncthreads();
+        for (int i = wave; i < a.part_count * a.part_pieces; i += kGemvWaves) {
+            const int g = i / a.part_pieces, piece = i % a.part_pieces, from = a.part_starts[g], to = a.part_starts[g + 1];
+            float s = 0.0f;
+            if (a.part_by_eight) {   // both halves of every eight, four at a time
+                for (int k = from / 2 + (piece * 64 + lane) * 4; k < to / 2; k += 256 * a.part_pieces) s += squared(at(xs, k)) + squared(at(xs + a.k_pad / 2, k));
+            } else {
+                for (int k = from + piece * 64 + lane; k < to; k += 64 * a.part_pieces) {
                     const float v = xs[staged_at(k, a.k_pad)];
                     s += v * v;
                 }
-                s = wave_sum(s);
-                if (lane == 0) head_inv[i] = s;
             }
-            __syncthreads();
-            for (int k = tid * 4; k < a.mix_cols; k += kGemvThreads * 4) {
-                const int4 g = *reinterpret_cast<const int4 *>(a.part_of + k);
-                const float4 n = *reinterpret_cast<const float4 *>(a.part_norm + k);
-                auto scale_of = [&](int part) {
-                    float s = 0.0f;
-                    for (int i = 0; i < a.part_pieces; i++) s += head_inv[part * a.part_pieces + i];
-                    return 1.0f / sqrtf(s / a.part_size + a.eps);
-                };
-                const float f = scale_of(g.x), l = g.w == g.x ? f : scale_of(g.w);
-                float4 v = *reinterpret_cast<const float4 *>(xs + staged_at(k, a.k_pad));
-                v.x *= f * n.x;
-                v.y *= (g.y == g.x ? f : g.y == g.w ? l : scale_of(g.y)) * n.y;
-                v.z *= (g.z == g.x ? f : g.z == g.w ? l : scale_of(g.z)) * n.z;
-                v.w *= l * n.w;
-                *reinterpret_cast<float4 *>(xs + staged_at(k, a.k_pad)) = v;
-            }
-            __syncthreads();
+            s = wave_sum(s);
+            if (lane == 0) sums[i] = s;
         }
-    } else if (KIND == KIND_IN && !a.norm_a) {
+        __syncthreads();
+        auto scale_of = [&](int g) {
+            float s = 0.0f;
+            for (int i = 0; i < a.part_pieces; i++) s += sums[g * a.part_pieces + i];
+            return 1.0f / sqrtf(s / a.part_size + a.eps);
+        };
+        auto put = [&](int k, float4 v, const int4 &g) {   // part indices ascend
+            const float f = scale_of(g.x), l = g.w == g.x ? f : scale_of(g.w);
+            v.x *= f;
+            v.y *= g.y == g.x ? f : g.y == g.w ? l : scale_of(g.y);
+            v.z *= g.z == g.x ? f : g.z == g.w ? l : scale_of(g.z);
+            v.w *= l;
+            place(k, v);
+        };
+#pragma unroll
+        for (int c = 0; c < kHeld; c++)
+            if (c * kSpan + tid * 4 < a.mix_cols) put(c * kSpan + tid * 4, held[c], part[c]);
+        for (int k = kHeld * kSpan + tid * 4; k < a.mix_cols; k += kSpan) {
+            float4 v = value(k);
+            const float4 w = at(a.part_norm, k);
+            v.x *= w.x; v.y *= w.y; v.z *= w.z; v.w *= w.w;
+            put(k, v, *reinterpret_cast<const int4 *>(a.part_of + k));
+        }
+        __syncthreads();
+    } else if constexpr (KIND == KIND_IN_STREAM) {
         // the stream as it is, or with a branch that is normed as it joins; both are kept in registers up to 8192 columns
         constexpr int kHeld = 4;
         float4 x[kHeld], b[kHeld], g[kHeld];
@@ -182,7 +227,7 @@ __global__ __launch_bounds__(kGemvThreads) void dense_gemv_kernel(DenseGemvArgs 
     }
 
     const int first = second ? (int)blockIdx.x - a.blocks_a : (int)blockIdx.x;
-    const int stride = KIND == KIND_IN ? (second ? (int)gridDim.x - a.blocks_a : a.blocks_a) : (int)gridDim.x;
+    const int stride = is_in(KIND) ? (second ? (int)gridDim.x - a.blocks_a : a.blocks_a) : (int)gridDim.x;
     const int units = second ? a.units_b : a.units_a, base_row = second ? a.mix_rows : 0;
     const int steps = a.k_pad / kStep;
     float best = -INFINITY;
@@ -227,7 +272,7 @@ __global__ __launch_bounds__(kGemvThreads) void dense_gemv_kernel(DenseGemvArgs 
 #pragma unroll
         for (int r = 0; r < RPW; r++) acc[r] = wave_sum(acc[r]) * scale;
         if (lane != 0) continue;
-        if constexpr (KIND == KIND_IN) {
+        if constexpr (is_in(KIND)) {
             if (!second) {
 #pragma unroll
                 for (int r = 0; r < RPW; r++) a.y[row0 + r] = acc[r];
@@ -236,7 +281,7 @@ __global__ __launch_bounds__(kGemvThreads) void dense_gemv_kernel(DenseGemvArgs 
 #pragma unroll
                 for (int r = 0; r + 1 < RPW; r += 2) a.act_out[i + r / 2] = matrix::gated(a.gate_function, acc[r], acc[r + 1]);
             }
-        } else if constexpr (KIND == KIND_OUT) {
+        } else if constexpr (KIND != KIND_HEAD) {
 #pragma unroll
             for (int r = 0; r < RPW; r++) a.y[row0 + r] = a.residual ? a.residual[row0 + r] + a.mult * acc[r] : acc[r];
         } else {
@@ -293,7 +338,7 @@ int at_most(int units) { return units < resident_workgroups() ? units : resident
 
 hipError_t launch_dense_gemv_in(const DenseGemvIn &p, hipStream_t s) {
     if (!p.w.w || p.w.ld % 64 || p.mix_rows % kRowAlign || p.w.rows % kRowAlign || p.w.rows < p.mix_rows || p.w.rows < kRowAlign || p.mix_rows < 0) return hipErrorInvalidValue;
-    if ((p.branch && (!p.branch_norm || !p.x_out || p.x_out == p.x || p.norm1)) || (p.w.rows > p.mix_rows && p.mix_rows && !p.norm1 != !p.norm2)) return hipErrorInvalidValue;
+    if ((p.branch && (!p.branch_norm || !p.x_out || p.x_out == p.x || p.norm1)) || (p.mix_rows && p.norm2 && !p.norm1) || (p.w.rows > p.mix_rows && p.norm1 && !p.norm2)) return hipErrorInvalidValue;
     DenseGemvArgs a{};
     a.w = p.w.w; a.ld = p.w.ld; a.k_pad = round_up(p.w.ld, kStep); a.mix_rows = p.mix_rows;
     a.x = p.x; a.norm_a = p.norm1; a.norm_b = p.norm2; a.width = p.width; a.eps = p.eps; a.y = p.y; a.act_out = p.act;
@@ -306,7 +351,17 @@ hipError_t launch_dense_gemv_in(const DenseGemvIn &p, hipStream_t s) {
     int grid = wanted;
     if (a.units_b == 0) a.blocks_a = grid;
     else if (a.units_a && a.blocks_a >= grid) grid = a.blocks_a + 1;
+    if (!p.norm1 && !p.norm2) return unit == kGemvWaves * 4 ? run<KIND_IN_STREAM, 4, 2>(a, grid, s) : run<KIND_IN_STREAM, 2, 3>(a, grid, s);
     return unit == kGemvWaves * 4 ? run<KIND_IN, 4, 2>(a, grid, s) : run<KIND_IN, 2, 3>(a, grid, s);
+}
+
+template <int KIND>
+static hipError_t run_out(DenseGemvArgs a, int rows, hipStream_t s) {
+    const int cus = resident_workgroups() / 2;   // long rows: a workgroup per compute unit
+    if (rows >= cus * kGemvWaves * 4) { a.units_a = rows / (kGemvWaves * 4); return run<KIND, 4, 2>(a, at_most(a.units_a), s); }
+    if (rows >= cus * kGemvWaves * 2) { a.units_a = rows / (kGemvWaves * 2); return run<KIND, 2, 4>(a, at_most(a.units_a), s); }
+    a.units_a = rows / kGemvWaves;
+    return run<KIND, 1, 6>(a, at_most(a.units_a), s);
 }
 
 hipError_t launch_dense_gemv_out(const DenseGemvOut &p, hipStream_t s) {
@@ -317,14 +372,11 @@ hipError_t launch_dense_gemv_out(const DenseGemvOut &p, hipStream_t s) {
     DenseGemvArgs a{};
     a.w = p.w.w; a.ld = p.w.ld; a.k_pad = round_up(p.w.ld, kStep);
     a.part_of = p.part_of; a.part_starts = p.part_starts; a.part_norm = p.part_norm; a.part_count = p.part_of ? p.part_count : 0; a.part_size = p.part_size;
+    a.part_by_eight = p.part_by_eight;
     a.part_pieces = !p.part_of || p.part_count >= kGemvWaves ? 1 : kGemvWaves / p.part_count;
     a.mix = p.mix; a.act = p.act; a.squares = p.squares; a.gate = p.gate; a.mix_cols = p.mix_cols; a.act_at = p.act_at; a.act_cols = p.act_cols; a.parts = p.parts;
     a.heads = p.squares ? p.mix_cols / p.vdim_p : 0; a.vdim = p.vdim; a.vdim_p = p.vdim_p; a.eps = p.eps; a.mult = p.mult; a.residual = p.residual; a.y = p.out;
-    const int cus = resident_workgroups() / 2;   // long rows: a workgroup per compute unit
-    if (p.rows >= cus * kGemvWaves * 4) { a.units_a = p.rows / (kGemvWaves * 4); return run<KIND_OUT, 4, 2>(a, at_most(a.units_a), s); }
-    if (p.rows >= cus * kGemvWaves * 2) { a.units_a = p.rows / (kGemvWaves * 2); return run<KIND_OUT, 2, 4>(a, at_most(a.units_a), s); }
-    a.units_a = p.rows / kGemvWaves;
-    return run<KIND_OUT, 1, 6>(a, at_most(a.units_a), s);
+    return p.part_of ? run_out<KIND_OUT_PARTS>(a, p.rows, s) : run_out<KIND_OUT>(a, p.rows, s);
 }
 
 int dense_gemv_head_workgroups(const DenseMatrix &w) { return at_most(w.rows / (kGemvWaves * 4)); }

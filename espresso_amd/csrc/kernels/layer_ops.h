@@ -56,6 +56,7 @@ struct DenseGemvOut {
     const float *part_norm = nullptr;                       // [mix_cols]
     int part_count = 0;
     float part_size = 0;                                    // values per part (columns without a value are zero)
+    bool part_by_eight = false;                             // every part starts at a multiple of eight columns
     float eps = 0, mult = 1;
     const float *residual = nullptr;
     float *out = nullptr;
@@ -181,10 +182,11 @@ struct Mamba2Shape {
     int vdim_p, state_p;
     int ld_mix;                              // columns of the mixed rows: z | x | B | C | dt, heads and groups padded
     int max_seq;
-    const float *conv, *conv_bias;           // [channels][taps], last column the current token's; [channels], channels x | B | C
+    const float *conv, *conv_bias;           // [taps][channels], last row the current token's; [channels], channels x | B | C
     const float *dt_bias, *rate, *skip;      // [heads]; rate: a token's decay is exp(-rate dt)
     const float *norm;                       // [heads * vdim_p]
     const int *norm_part, *norm_starts;      // part of a value [heads * vdim_p]; first value of a part [norm_groups + 1]
+    bool norm_by_eight;                      // every part starts at a multiple of eight values
     float *state_of;                         // [sequence][heads][vdim_p][state_p] (transposed), fp32
     float *inputs;                           // [sequence][taps][channels]: the convolution's input of position p at row p % taps
 };

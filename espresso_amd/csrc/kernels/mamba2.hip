@@ -34,38 +34,68 @@ __host__ __device__ __forceinline__ int values_of(const Mamba2Shape &r) { return
 __host__ __device__ __forceinline__ int channels_of(const Mamba2Shape &r) { return values_of(r) + 2 * r.groups * r.state_p; }
 __device__ __forceinline__ float softplus(float v) { return v > 20.0f ? v : log1pf(expf(v)); }
 
+// TAPS: taps of the convolution, 0 = any number.  Every load that needs no other is requested before the first is used.
+template <int TAPS>
 __global__ __launch_bounds__(256) void mamba2_step_kernel(Mamba2Shape r, Mamba2Step p) {
     extern __shared__ float lds[];   // B [state_p], C [state_p]
     const int part = blockIdx.x, h = blockIdx.y, m = blockIdx.z, tid = threadIdx.x;
     const int pos = p.pos[m], seq = p.seq[m];
-    const bool again = p.halt && *p.halt, fresh = pos == 0 && !again;
     const int e = tid & 7, v = part * kStepRows + (tid >> 3), values = values_of(r), channels = channels_of(r);
-    float *state = r.state_of + (((size_t)seq * r.heads + h) * r.vdim_p + v) * r.state_p + e * 4;
-    // up to eight pieces of the row are on their way meanwhile
-    constexpr int kHeld = 8;
-    float4 held[kHeld];
-#pragma unroll
-    for (int i = 0; i < kHeld; i++) held[i] = *reinterpret_cast<const float4 *>(state + (i * 32 < r.state_p ? i * 32 : 0));
     const float *row = p.mixed + (size_t)m * r.ld_mix, *inputs = row + values;
     float *past = r.inputs + (size_t)seq * r.taps * channels;
-    auto convolved = [&](int channel) {
-        const float *w = r.conv + (size_t)channel * r.taps;
-        float s = r.conv_bias[channel] + w[r.taps - 1] * inputs[channel];
-        const int reach = pos < r.taps - 1 ? pos : r.taps - 1;
-        for (int j = 1; j <= reach; j++) s += w[r.taps - 1 - j] * past[(size_t)((pos - j) % r.taps) * channels + channel];
+    constexpr int kTaps = TAPS ? TAPS : 1;
+    struct Window {   // what one channel's convolution reads
+        float in[kTaps], w[kTaps], bias;
+    };
+    auto request = [&](int channel) {
+        Window g;
+        g.bias = r.conv_bias[channel];
+        g.in[0] = inputs[channel];
+        g.w[0] = r.conv[(size_t)(r.taps - 1) * channels + channel];
+#pragma unroll
+        for (int j = 1; j < kTaps; j++) {
+            const int at = pos - j;
+            g.w[j] = r.conv[(size_t)(kTaps - 1 - j) * channels + channel];
+            g.in[j] = past[(size_t)(at > 0 ? at % kTaps : 0) * channels + channel];
+        }
+        return g;
+    };
+    auto convolved = [&](const Window &g, int channel) {
+        float s = g.bias + g.w[0] * g.in[0];
+#pragma unroll
+        for (int j = 1; j < kTaps; j++) s += pos >= j ? g.w[j] * g.in[j] : 0.0f;
+        if constexpr (TAPS == 0) {
+            const int reach = pos < r.taps - 1 ? pos : r.taps - 1;
+            for (int j = 1; j <= reach; j++) s += r.conv[(size_t)(r.taps - 1 - j) * channels + channel] * past[(size_t)((pos - j) % r.taps) * channels + channel];
+        }
         return matrix::silu(s);
     };
     const int share = r.heads / r.groups, group = h / share;
+    auto shared_channel = [&](int i) { return values + (i < r.state_p ? group * r.state_p + i : (r.groups + group) * r.state_p + i - r.state_p); };
+    const int x_channel = h * r.vdim_p + v, first = tid < 2 * r.state_p ? shared_channel(tid) : values;
+    const Window of_x = request(x_channel), of_shared = request(first);
+    const float z = row[h * r.vdim_p + v], raw_dt = inputs[channels + h], dt_bias = r.dt_bias[h], rate = r.rate[h], skip = r.skip[h];
+    float *state = r.state_of + (((size_t)seq * r.heads + h) * r.vdim_p + v) * r.state_p + e * 4;
+    constexpr int kHeld = 8;   // pieces of the state's row
+    float4 held[kHeld];
+#pragma unroll
+    for (int i = 0; i < kHeld; i++) held[i] = *reinterpret_cast<const float4 *>(state + (i * 32 < r.state_p ? i * 32 : 0));
+    const bool again = p.halt && *p.halt, fresh = pos == 0 && !again;
     const bool keeps = part == 0 && h % share == 0;   // the workgroup that keeps the group's inputs
     float *now = past + (size_t)(pos % r.taps) * channels;
-    for (int i = tid; i < 2 * r.state_p; i += 256) {
-        const int channel = values + (i < r.state_p ? group * r.state_p + i : (r.groups + group) * r.state_p + i - r.state_p);
-        lds[i] = convolved(channel);
-        if (keeps) now[channel] = inputs[channel];
+    if (tid < 2 * r.state_p) {
+        lds[tid] = convolved(of_shared, first);
+        if (keeps) now[first] = of_shared.in[0];
     }
-    const float x = convolved(h * r.vdim_p + v), z = row[h * r.vdim_p + v];
-    if (e == 0) now[h * r.vdim_p + v] = inputs[h * r.vdim_p + v];
-    const float dt = softplus(inputs[channels + h] + r.dt_bias[h]), decay = expf(-r.rate[h] * dt), value = dt * x;
+    for (int i = tid + 256; i < 2 * r.state_p; i += 256) {
+        const int channel = shared_channel(i);
+        const Window g = request(channel);
+        lds[i] = convolved(g, channel);
+        if (keeps) now[channel] = g.in[0];
+    }
+    const float x = convolved(of_x, x_channel);
+    if (e == 0) now[x_channel] = of_x.in[0];
+    const float dt = softplus(raw_dt + dt_bias), decay = expf(-rate * dt), value = dt * x;
     __syncthreads();
     float o = 0.0f;
     auto piece = [&](int d0, float4 s) {
@@ -84,7 +114,7 @@ __global__ __launch_bounds__(256) void mamba2_step_kernel(Mamba2Shape r, Mamba2S
     o += detail::dpp_term<0xB1, 0xF>(o);    // the eight lanes of a row
     o += detail::dpp_term<0x4E, 0xF>(o);
     o += detail::dpp_term<0x141, 0xF>(o);
-    if (e == 0) p.y[(size_t)m * values + h * r.vdim_p + v] = (o + r.skip[h] * x) * matrix::silu(z);
+    if (e == 0) p.y[(size_t)m * values + h * r.vdim_p + v] = (o + skip * x) * matrix::silu(z);
 }
 
 struct BlockArgs {
@@ -131,12 +161,11 @@ __global__ __launch_bounds__(256) void mamba2_prepare_kernel(BlockArgs a) {
     }
     __syncthreads();
     const float bias = r.conv_bias[channel];
-    const float *w = r.conv + (size_t)channel * r.taps;
     float y[C / 8];
 #pragma unroll
     for (int i = 0; i < C / 8; i++) y[i] = bias;
     for (int j = 0; j < r.taps; j++) {
-        const float f = w[j];
+        const float f = r.conv[(size_t)j * channels + channel];
 #pragma unroll
         for (int i = 0; i < C / 8; i++) {
             const int t = (tid >> 5) + 8 * i;
@@ -172,7 +201,9 @@ __global__ __launch_bounds__(256) void mamba2_prepare_kernel(BlockArgs a) {
 }
 
 // One workgroup per row: parts of the row over their root mean squares; and a block's last inputs into the sequence's ring.
-constexpr int kNormWaves = 4;
+constexpr int kNormWaves = 8;
+__device__ __forceinline__ void store4(uint16_t *p, const float4 &v) { *reinterpret_cast<uint2 *>(p) = make_uint2(matrix::pack_bf16(v.x, v.y), matrix::pack_bf16(v.z, v.w)); }
+__device__ __forceinline__ void store4(float *p, const float4 &v) { *reinterpret_cast<float4 *>(p) = v; }
 template <typename T>
 __global__ __launch_bounds__(64 * kNormWaves) void mamba2_norm_kernel(Mamba2Shape r, Mamba2Norm p) {
     extern __shared__ float lds[];   // [norm_groups * pieces] sums, then scales [norm_groups]
@@ -185,9 +216,17 @@ __global__ __launch_bounds__(64 * kNormWaves) void mamba2_norm_kernel(Mamba2Shap
         for (int i = tid; i < channels; i += 64 * kNormWaves) now[i] = inputs[i];
     }
     for (int i = wave; i < r.norm_groups * pieces; i += kNormWaves) {
-        const int g = i / pieces, from = r.norm_starts[g], to = r.norm_starts[g + 1];
+        const int g = i / pieces, at = (i % pieces) * 64 + lane, from = r.norm_starts[g], to = r.norm_starts[g + 1];
         float s = 0.0f;
-        for (int k = from + (i % pieces) * 64 + lane; k < to; k += 64 * pieces) s += y[k] * y[k];
+        if (r.norm_by_eight) {
+#pragma unroll 4
+            for (int k = from + at * 4; k < to; k += 256 * pieces) {
+                const float4 v = *reinterpret_cast<const float4 *>(y + k);
+                s += v.x * v.x + v.y * v.y + v.z * v.z + v.w * v.w;
+            }
+        } else {
+            for (int k = from + at; k < to; k += 64 * pieces) s += y[k] * y[k];
+        }
         s = detail::wave_sum(s);
         if (lane == 0) lds[i] = s;
     }
@@ -201,7 +240,12 @@ __global__ __launch_bounds__(64 * kNormWaves) void mamba2_norm_kernel(Mamba2Shap
     }
     __syncthreads();
     T *dst = static_cast<T *>(p.act) + (size_t)m * p.ld_act;
-    for (int k = tid; k < values; k += 64 * kNormWaves) dst[k] = Op<T>::from_float(y[k] * scale[r.norm_part[k]] * r.norm[k]);
+#pragma unroll 4
+    for (int k = tid * 4; k < values; k += 256 * kNormWaves) {
+        const float4 v = *reinterpret_cast<const float4 *>(y + k), n = *reinterpret_cast<const float4 *>(r.norm + k);
+        const int4 g = *reinterpret_cast<const int4 *>(r.norm_part + k);
+        store4(dst + k, make_float4(v.x * scale[g.x] * n.x, v.y * scale[g.y] * n.y, v.z * scale[g.z] * n.z, v.w * scale[g.w] * n.w));
+    }
 }
 
 bool shape_ok(const Mamba2Shape &r) {
@@ -227,7 +271,14 @@ hipError_t run_block(const BlockArgs &a, hipStream_t s) {
 
 hipError_t launch_mamba2_step(const Mamba2Shape &r, const Mamba2Step &p, hipStream_t s) {
     if (!shape_ok(r) || p.rows < 1) return hipErrorInvalidValue;
-    hipLaunchKernelGGL(mamba2_step_kernel, dim3(r.vdim_p / kStepRows, r.heads, p.rows), dim3(256), (size_t)r.state_p * 8, s, r, p);
+    const dim3 grid(r.vdim_p / kStepRows, r.heads, p.rows);
+    const size_t lds = (size_t)r.state_p * 8;
+    switch (r.taps) {
+        case 2: hipLaunchKernelGGL((mamba2_step_kernel<2>), grid, dim3(256), lds, s, r, p); break;
+        case 3: hipLaunchKernelGGL((mamba2_step_kernel<3>), grid, dim3(256), lds, s, r, p); break;
+        case 4: hipLaunchKernelGGL((mamba2_step_kernel<4>), grid, dim3(256), lds, s, r, p); break;
+        default: hipLaunchKernelGGL((mamba2_step_kernel<0>), grid, dim3(256), lds, s, r, p); break;
+    }
     return hipGetLastError();
 }
 

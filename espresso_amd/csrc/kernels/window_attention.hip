@@ -49,15 +49,34 @@ __device__ __forceinline__ void load8(const float *p, float (&f)[8]) {
     f[0] = a.x; f[1] = a.y; f[2] = a.z; f[3] = a.w; f[4] = b.x; f[5] = b.y; f[6] = b.z; f[7] = b.w;
 }
 
+// The same eight as they are loaded, to be unpacked later.
+template <typename T>
+struct Piece;
+template <>
+struct Piece<uint16_t> {
+    uint4 v;
+    __device__ __forceinline__ void load(const uint16_t *p) { v = *reinterpret_cast<const uint4 *>(p); }
+    __device__ __forceinline__ void unpack(float (&f)[8]) const { matrix::unpack_bf16(v, f); }
+};
+template <>
+struct Piece<float> {
+    float4 a, b;
+    __device__ __forceinline__ void load(const float *p) { a = reinterpret_cast<const float4 *>(p)[0]; b = reinterpret_cast<const float4 *>(p)[1]; }
+    __device__ __forceinline__ void unpack(float (&f)[8]) const { f[0] = a.x; f[1] = a.y; f[2] = a.z; f[3] = a.w; f[4] = b.x; f[5] = b.y; f[6] = b.z; f[7] = b.w; }
+};
+
 constexpr int kTile = 32;   // keys per pass of a workgroup: eight lanes each
 
+constexpr int kKeyPieces = 4, kValuePieces = 2;   // pieces of eight per thread that are requested ahead; longer heads read the rest when needed
+
 // grid (splits, key heads x chunks of Q query heads, rows).  LDS: queries [Q][dim_p], scores [Q][kTile], running (maximum, sum, rescale)
-// [Q][3], and for the end the value sums [parts][vdim_p].
+// [Q][4], the row's own key [dim_p] and value [vdim_p], and for the end the value sums [parts][vdim_p].  A tile's keys and values are
+// requested a tile ahead, the first ones before the norms.
 template <typename T, int Q>
 __global__ __launch_bounds__(256) void attention_partial_kernel(AttentionShape l, AttentionStep p) {
     extern __shared__ float lds[];
     __shared__ float red[8];
-    float *q = lds, *scores = q + Q * l.dim_p, *running = scores + Q * kTile, *meet = running + Q * 4;
+    float *q = lds, *scores = q + Q * l.dim_p, *running = scores + Q * kTile, *own_key = running + Q * 4, *own_value = own_key + l.dim_p, *meet = own_value + l.vdim_p;
     const int tid = threadIdx.x, lane = tid & 63, split = blockIdx.x, m = blockIdx.z, pos = p.pos[m], seq = p.seq[m];
     const int share = l.heads / l.kv_heads, chunks = (share + Q - 1) / Q, kv = blockIdx.y / chunks, h0 = kv * share + blockIdx.y % chunks * Q;
     const int live = (kv + 1) * share - h0 < Q ? (kv + 1) * share - h0 : Q;
@@ -68,8 +87,24 @@ __global__ __launch_bounds__(256) void attention_partial_kernel(AttentionShape l
     const int width = cached_row(l);
     T *cache = static_cast<T *>(l.cache) + (size_t)seq * l.ring * width;
     const bool owner = l.k_at >= 0 && split == (tiles - 1) % p.splits;   // the last tile holds the row's own token
+    const int e = tid & 7, key_in = tid >> 3;
+    const int pieces = l.vdim_p / 8, parts = 256 / pieces < kTile ? 256 / pieces : kTile, piece = tid % pieces, part = tid / pieces;   // value phase: eight values, every parts-th key
+    const T *keys = cache + kv * l.dim_p, *values = cache + l.kv_heads * l.dim_p + kv * l.vdim_p + piece * 8;
+    auto row_of = [&](int key) { return (size_t)((key < pos ? key : pos) % l.ring) * width; };   // keys past the query repeat it and weigh nothing
+    Piece<T> key_ahead[kKeyPieces], value_ahead[kValuePieces];
+    auto request = [&](int t) {
+        const int k0 = lo + t * kTile;
+        const T *from = keys + row_of(k0 + key_in);
+#pragma unroll
+        for (int i = 0; i < kKeyPieces; i++) key_ahead[i].load(from + (e * 8 + i * 64 < l.dim_p ? e * 8 + i * 64 : 0));
+#pragma unroll
+        for (int i = 0; i < kValuePieces; i++) value_ahead[i].load(values + row_of(k0 + (part + i * parts < kTile ? part + i * parts : 0)));
+    };
     {
-        float sq = detail::wave_sum(squares(row, l.heads * l.dim_p)), sk = owner ? detail::wave_sum(squares(row + l.k_at, l.kv_heads * l.dim_p)) : 0.0f;
+        float sq = squares(row, l.heads * l.dim_p), sk = owner ? squares(row + l.k_at, l.kv_heads * l.dim_p) : 0.0f;
+        request(split);
+        sq = detail::wave_sum(sq);
+        sk = detail::wave_sum(sk);
         if (lane == 0) { red[tid >> 6] = sq; red[4 + (tid >> 6)] = sk; }
         __syncthreads();
         sq = (red[0] + red[1]) + (red[2] + red[3]);
@@ -79,35 +114,37 @@ __global__ __launch_bounds__(256) void attention_partial_kernel(AttentionShape l
             const int r = i / l.dim_p, d = i - r * l.dim_p, at = (h0 + (r < live ? r : 0)) * l.dim_p;   // heads past the group repeat its first
             q[i] = l.scale * normed_rotated(row + at, l.q_norm + at, inv_q, d, l.rot_dims, cos, sin);
         }
-        if (owner) {   // every chunk of the group's heads writes the same
+        if (owner) {   // every chunk of the group's heads writes the same; here they are read from LDS
             T *own = cache + (size_t)(pos % l.ring) * width;
             for (int d = tid; d < l.dim_p; d += 256) {
                 const int at = kv * l.dim_p;
-                own[at + d] = Op<T>::from_float(normed_rotated(row + l.k_at + at, l.k_norm + at, inv_k, d, l.rot_dims, cos, sin));
+                const T k = Op<T>::from_float(normed_rotated(row + l.k_at + at, l.k_norm + at, inv_k, d, l.rot_dims, cos, sin));
+                own[at + d] = k;
+                own_key[d] = Op<T>::to_float(k);
             }
             const float *v = row + l.k_at + l.kv_heads * l.dim_p + kv * l.vdim_p;
-            for (int d = tid; d < l.vdim_p; d += 256) own[l.kv_heads * l.dim_p + kv * l.vdim_p + d] = Op<T>::from_float(v[d]);
+            for (int d = tid; d < l.vdim_p; d += 256) {
+                const T x = Op<T>::from_float(v[d]);
+                own[l.kv_heads * l.dim_p + kv * l.vdim_p + d] = x;
+                own_value[d] = Op<T>::to_float(x);
+            }
         }
         if (tid < Q) { running[tid * 4] = -INFINITY; running[tid * 4 + 1] = 0.0f; }
     }
     __syncthreads();
-    const int e = tid & 7, key_in = tid >> 3;
-    const int pieces = l.vdim_p / 8, parts = 256 / pieces < kTile ? 256 / pieces : kTile, piece = tid % pieces, part = tid / pieces;   // value phase: eight values, every parts-th key
     float acc[Q][8];
 #pragma unroll
     for (int r = 0; r < Q; r++)
 #pragma unroll
         for (int i = 0; i < 8; i++) acc[r][i] = 0.0f;
     for (int t = split; t < tiles; t += p.splits) {
-        const int k0 = lo + t * kTile, in = k0 + key_in <= pos;
-        const int key = in ? k0 + key_in : pos;
-        const T *keys = cache + (size_t)(key % l.ring) * width + kv * l.dim_p;
+        const int k0 = lo + t * kTile;
+        const bool in = k0 + key_in <= pos, mine = owner && k0 + key_in >= pos;
         float s[Q];
 #pragma unroll
         for (int r = 0; r < Q; r++) s[r] = 0.0f;
-        for (int d = e * 8; d < l.dim_p; d += 64) {
-            float k[8];
-            load8(keys + d, k);
+        auto score = [&](float (&k)[8], int d) {
+            if (mine) load8(own_key + d, k);
 #pragma unroll
             for (int r = 0; r < Q; r++) {
                 float x[8];
@@ -115,6 +152,17 @@ __global__ __launch_bounds__(256) void attention_partial_kernel(AttentionShape l
 #pragma unroll
                 for (int i = 0; i < 8; i++) s[r] = __builtin_fmaf(k[i], x[i], s[r]);
             }
+        };
+#pragma unroll
+        for (int i = 0; i < kKeyPieces; i++) {
+            float k[8];
+            key_ahead[i].unpack(k);
+            if (e * 8 + i * 64 < l.dim_p) score(k, e * 8 + i * 64);
+        }
+        for (int d = e * 8 + kKeyPieces * 64; d < l.dim_p; d += 64) {
+            float k[8];
+            load8(keys + row_of(k0 + key_in) + d, k);
+            score(k, d);
         }
 #pragma unroll
         for (int r = 0; r < Q; r++) {   // the eight lanes of a key
@@ -144,18 +192,28 @@ __global__ __launch_bounds__(256) void attention_partial_kernel(AttentionShape l
 #pragma unroll
                 for (int i = 0; i < 8; i++) acc[r][i] *= keep;
             }
-            for (int k = part; k < kTile; k += parts) {
-                const int at = k0 + k <= pos ? k0 + k : pos;   // keys past the query weigh nothing
-                float v[8];
-                load8(cache + (size_t)(at % l.ring) * width + l.kv_heads * l.dim_p + kv * l.vdim_p + piece * 8, v);
+            auto add = [&](float (&v)[8], int k) {
+                if (owner && k0 + k >= pos) load8(own_value + piece * 8, v);
 #pragma unroll
                 for (int r = 0; r < Q; r++) {
                     const float w = scores[r * kTile + k];
 #pragma unroll
                     for (int i = 0; i < 8; i++) acc[r][i] = __builtin_fmaf(w, v[i], acc[r][i]);
                 }
+            };
+#pragma unroll
+            for (int i = 0; i < kValuePieces; i++) {
+                float v[8];
+                value_ahead[i].unpack(v);
+                if (part + i * parts < kTile) add(v, part + i * parts);
+            }
+            for (int k = part + kValuePieces * parts; k < kTile; k += parts) {
+                float v[8];
+                load8(values + row_of(k0 + k), v);
+                add(v, k);
             }
         }
+        if (t + p.splits < tiles) request(t + p.splits);
         __syncthreads();
     }
     const size_t first = ((size_t)m * p.splits + split) * l.heads + h0;
@@ -277,7 +335,7 @@ int heads_together(const AttentionShape &l) {
 template <typename T, int Q>
 hipError_t run_partial(const AttentionShape &l, const AttentionStep &p, hipStream_t s) {
     const int chunks = (l.heads / l.kv_heads + Q - 1) / Q, parts = 256 / (l.vdim_p / 8) < kTile ? 256 / (l.vdim_p / 8) : kTile;
-    const size_t lds = (size_t)(Q * (l.dim_p + kTile + 4) + parts * l.vdim_p) * 4;
+    const size_t lds = (size_t)(Q * (l.dim_p + kTile + 4) + l.dim_p + l.vdim_p + parts * l.vdim_p) * 4;
     if (lds > 62 * 1024) return hipErrorInvalidValue;
     hipLaunchKernelGGL((attention_partial_kernel<T, Q>), dim3(p.splits, l.kv_heads * chunks, p.rows), dim3(256), lds, s, l, p);
     return hipGetLastError();

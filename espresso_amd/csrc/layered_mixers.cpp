@@ -214,7 +214,7 @@ int LayeredRuntime::build_mamba2(size_t index, LayeredWeights &weights) {
         bias[padded(c)] = v[c];
         for (int j = 0; j < S.conv; j++) {
             const uint32_t wide = (uint32_t)taps[(size_t)c * S.conv + j] << 16;
-            std::memcpy(&conv[padded(c) * S.conv + j], &wide, 4);
+            std::memcpy(&conv[j * channels_p + padded(c)], &wide, 4);
         }
     }
     if ((rc = upload_floats(conv, &L.vectors[0])) != ESP_OK || (rc = upload_floats(bias, &L.vectors[1])) != ESP_OK) return rc;
@@ -227,7 +227,11 @@ int LayeredRuntime::build_mamba2(size_t index, LayeredWeights &weights) {
     const int part_size = inner / S.norm_groups;
     std::vector<int> part(values), starts(S.norm_groups + 1, (int)values);
     for (size_t k = 0; k < values; k++) part[k] = std::min((int)(k / vp * S.vdim + std::min<size_t>(k % vp, S.vdim - 1)) / part_size, S.norm_groups - 1);
-    for (int g = 0; g < S.norm_groups; g++) starts[g] = (int)padded(g * part_size);
+    bool by_eight = true;
+    for (int g = 0; g < S.norm_groups; g++) {
+        starts[g] = (int)padded(g * part_size);
+        by_eight = by_eight && starts[g] % 8 == 0;
+    }
     for (int i = 0; i < 2; i++) {
         const std::vector<int> &t = i ? starts : part;
         if ((rc = device_alloc(&L.tables[i], t.size())) != ESP_OK) return rc;
@@ -236,7 +240,7 @@ int LayeredRuntime::build_mamba2(size_t index, LayeredWeights &weights) {
     Mamba2Shape &r = L.mamba2;
     r.heads = H; r.vdim = S.vdim; r.state = S.state; r.groups = G; r.taps = S.conv; r.norm_groups = S.norm_groups; r.vdim_p = vp; r.state_p = sp; r.ld_mix = L.mix_rows;
     r.max_seq = shape_.max_seq; r.conv = L.vectors[0]; r.conv_bias = L.vectors[1]; r.dt_bias = L.vectors[2]; r.rate = L.vectors[3]; r.skip = L.vectors[4]; r.norm = L.vectors[5];
-    r.norm_part = L.tables[0]; r.norm_starts = L.tables[1];
+    r.norm_part = L.tables[0]; r.norm_starts = L.tables[1]; r.norm_by_eight = by_eight;
     L.state_floats = values * sp;
     L.input_floats = channels_p * S.conv;
     return ESP_OK;
@@ -340,7 +344,7 @@ int LayeredRuntime::mixer_step(Layer &L, DenseGemvOut *out) {
             if ((rc = time_begin(K_MAMBA2)) != ESP_OK) return rc;
             ESP_HIP_TRY(launch_mamba2_step(r, st, s));
             out->mix_cols = r.heads * r.vdim_p; out->part_of = r.norm_part; out->part_starts = r.norm_starts; out->part_norm = r.norm;
-            out->part_count = r.norm_groups; out->part_size = (float)(r.heads * r.vdim / r.norm_groups);
+            out->part_count = r.norm_groups; out->part_size = (float)(r.heads * r.vdim / r.norm_groups); out->part_by_eight = r.norm_by_eight;
             break;
         }
         case MixerKind::latent_attention: {

@@ -92,3 +92,30 @@ LAYERED_SIZES = {
     "d4096": (layered_config(4096, 14336, 32000, dict(heads=32, dim=128, vdim=128, rot_dim=64, kv_rank=512), dict(heads=16, dim=256, vdim=256)),
               dict(n_layer=6, n_head=32, n_kv_head=8, d_model=4096, head_dim=128, hidden_dim=14336, vocab=32000, max_seq=1024)),
 }
+
+
+def sequential_config(width: int, ff: int, vocab: int, attention: dict, mamba2: dict, mamba2_2: dict, layers: int = 6, window: int = 1024) -> dict:
+    """A config.json of a layered model of the other design: two Mamba-2 layers of different sizes and an attention layer with a
+    feed-forward, again and again; every second attention layer reads the keys and values of the one before."""
+    out = []
+    for i in range(layers):
+        if i % 3 < 2:
+            out.append({"type": ("mamba2", "mamba2_2")[i % 3], "mlp": None, "mixer": dict((mamba2, mamba2_2)[i % 3])})
+        else:
+            m = dict(attention, scale=attention["dim"] ** -0.5, mask={"size": window}, rot={"base": 1000000.0, "dims": attention["dim"] // 2, "scaling": {"factor": 2.0}})
+            if i % 6 == 5:
+                m["kv_from"] = i - 3
+            out.append({"type": "attention", "mlp": {"kind": "dense", "ff": ff}, "mixer": m})
+    return {"architecture": "Forovik", "vocab": vocab, "width": width, "norm": {"eps": 1e-6}, "layers": out}
+
+
+def _mamba2(heads: int, vdim: int, state: int, groups: int, conv: int = 4) -> dict:
+    return {"heads": heads, "vdim": vdim, "state": state, "groups": groups, "conv": conv, "norm_groups": groups}
+
+
+# The same widths and feed-forwards: (configuration, the size in LAYERED_SIZES to measure beside it).
+SEQUENTIAL_SIZES = {
+    "forovik-d768": (sequential_config(768, 2048, 32000, dict(heads=12, kv_heads=4, dim=64, vdim=64), _mamba2(24, 64, 128, 1), _mamba2(12, 128, 64, 2, 3)), "d768"),
+    "forovik-d2048": (sequential_config(2048, 8192, 32000, dict(heads=16, kv_heads=4, dim=128, vdim=128), _mamba2(64, 64, 128, 8), _mamba2(32, 128, 64, 4, 3)), "d2048"),
+    "forovik-d4096": (sequential_config(4096, 14336, 32000, dict(heads=32, kv_heads=8, dim=128, vdim=128), _mamba2(128, 64, 128, 8), _mamba2(64, 128, 64, 8, 3)), "d4096"),
+}
