@@ -99,17 +99,19 @@ ESPLlamaRuntime *esp_layered_create_synthetic(const char *config_json, int float
 int esp_layered_set_min_block_rows(ESPLlamaRuntime *runtime, int rows);
 /* Appends up to 512 tokens as one block and copies the residual stream after every layer: out [layers][count][width]. */
 int esp_layered_trace_layers(ESPLlamaRuntime *runtime, int sequence, const uint32_t *tokens, int count, float *out);
-/* What one sequence holds in recurrent states and cached latents. */
+/* What one sequence holds in recurrent states and caches. */
 long long esp_layered_sequence_bytes(const ESPLlamaRuntime *runtime);
 /* Event timing as esp_llama_kernel_times, by class of launches: the layers' input products, retention, latent attention, the layers'
- * output products, the head, residual sums and norms of blocks.  bytes: what the class reads in one decode step (all layers). */
+ * output products, the head, residual sums and norms, grouped attention, Mamba-2.  bytes: what the class reads in one decode step (all layers). */
 #define ESP_LAYERED_KERNEL_IN 0
 #define ESP_LAYERED_KERNEL_RETENTION 1
 #define ESP_LAYERED_KERNEL_LATENT 2
 #define ESP_LAYERED_KERNEL_OUT 3
 #define ESP_LAYERED_KERNEL_HEAD 4
 #define ESP_LAYERED_KERNEL_NORM 5
-#define ESP_LAYERED_KERNEL_CLASS_COUNT 6
+#define ESP_LAYERED_KERNEL_ATTENTION 6
+#define ESP_LAYERED_KERNEL_MAMBA2 7
+#define ESP_LAYERED_KERNEL_CLASS_COUNT 8
 int esp_layered_set_kernel_timing(ESPLlamaRuntime *runtime, int enabled);
 int esp_layered_kernel_times(ESPLlamaRuntime *runtime, double *total_us, int64_t *launches, uint64_t *bytes, int reset);
 
