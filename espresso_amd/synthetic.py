@@ -95,15 +95,15 @@ LAYERED_SIZES = {
 
 
 def sequential_config(width: int, ff: int, vocab: int, attention: dict, mamba2: dict, mamba2_2: dict, layers: int = 6, window: int = 1024) -> dict:
-    """A config.json of a layered model of the other design: two Mamba-2 layers of different sizes and an attention layer with a
-    feed-forward, again and again; every second attention layer reads the keys and values of the one before."""
+    """A config.json of a layered model of the other design: an attention layer with a feed-forward and two Mamba-2 layers of different
+    sizes, again and again; every second attention layer reads the keys and values of the one before."""
     out = []
     for i in range(layers):
-        if i % 3 < 2:
-            out.append({"type": ("mamba2", "mamba2_2")[i % 3], "mlp": None, "mixer": dict((mamba2, mamba2_2)[i % 3])})
+        if i % 3:
+            out.append({"type": ("mamba2", "mamba2_2")[i % 3 - 1], "mlp": None, "mixer": dict((mamba2, mamba2_2)[i % 3 - 1])})
         else:
-            m = dict(attention, scale=attention["dim"] ** -0.5, mask={"size": window}, rot={"base": 1000000.0, "dims": attention["dim"] // 2, "scaling": {"factor": 2.0}})
-            if i % 6 == 5:
+            m = dict(attention, scale=attention["dim"] ** -0.5, mask={"size": window}, rot={"base": 500000.0, "dims": attention["dim"] // 2, "scaling": {"factor": 2.0}})
+            if i % 6 == 3:
                 m["kv_from"] = i - 3
             out.append({"type": "attention", "mlp": {"kind": "dense", "ff": ff}, "mixer": m})
     return {"architecture": "Forovik", "vocab": vocab, "width": width, "norm": {"eps": 1e-6}, "layers": out}
